@@ -51,8 +51,9 @@ class LayerSpec:
     layer_input: PartSpec | None = None
     layer_input_place: str = "side."
     # something that stands between a norm and the sublayer that reads it (a part of the "sublayer_input" table, built
-    # once for the mixer and once for the feed-forward), and the places of the two
+    # once for each of the sublayers named in `sublayer_input_of`), and the places of the two
     sublayer_input: PartSpec | None = None
+    sublayer_input_of: tuple[str, ...] = ("mixer", "feed_forward")
     mixer_input_place: str = "mixer_input."
     feed_forward_input_place: str = "feed_forward_input."
     # for the arrangement on a residual of several streams ("hyper_connections"): how many streams (the model's
@@ -80,6 +81,9 @@ class Run:
     # tell the passes apart.
     add_embedding: bool = False
     add_vector: tuple[str, int] | None = None
+    # What takes the residual's place right before this run: the product of the tensor named here ([hidden, 2 * hidden])
+    # with the residual and the embedding's output, side by side.
+    pass_input: str | None = None
     # What goes on after this run in place of its own result: a weighted sum over the embedding's output and the results
     # of all runs so far, this one included (run i: i + 2 summands, in that order), with the weights of the tensor named
     # here ([i + 2]).  A model uses this for all of its runs or for none.
@@ -121,7 +125,8 @@ class ModelSpec:
         for layer in self.layers:
             if layer.streams != self.streams:
                 raise invalid_config("every layer works on as many streams of the residual as the model has")
-        if self.streams and any(run.add_embedding or run.add_vector is not None or run.depth_mix is not None for run in self.runs):
+        if self.streams and any(run.add_embedding or run.add_vector is not None or run.depth_mix is not None
+                                or run.pass_input is not None for run in self.runs):
             raise invalid_config("runs that add something to the residual do not go with a residual of several streams")
         for index, run in enumerate(self.runs):
             if not 0 <= run.layer < len(self.layers):
@@ -136,6 +141,11 @@ class ModelSpec:
                 shapes = [tensor.shape for tensor in self.shared_tensors if tensor.name == run.depth_mix]
                 if shapes != [(index + 2,)]:
                     raise invalid_config(f"run {index} mixes the results so far with '{run.depth_mix}', which is no shared tensor [{index + 2}]")
+            if run.pass_input is not None:
+                shapes = [tensor.shape for tensor in self.shared_tensors if tensor.name == run.pass_input]
+                if shapes != [(self.hidden_size, 2 * self.hidden_size)] or self.embedding.get("norm") is not None:
+                    raise invalid_config(f"run {index} forms its residual with '{run.pass_input}', which is no shared tensor "
+                                         "[hidden, 2 * hidden] (on an embedding whose output is its table's rows)")
             if run.add_vector is not None:
                 name, row = run.add_vector
                 shapes = [tensor.shape for tensor in self.shared_tensors if tensor.name == name]

@@ -1,7 +1,8 @@
 // Kernels around a sublayer's input that the framework's RMS-norm kernels do not cover:
 //
-//   layer_norm      residual += s1 * delta1 + s2 * delta2 (both optional), optionally a weighted sum over the
-//                   residuals of earlier layers in its place, then (x - mean) / sqrt(var + eps) * w + b
+//   layer_norm      residual += s1 * delta1 + s2 * delta2 (both optional; s2 may be multiplied by a number of the row's
+//                   own), optionally a weighted sum over the residuals of earlier layers in its place, then
+//                   (x - mean) / sqrt(var + eps) * w + b, or, not centred, x / sqrt(mean(x^2) + eps) * w + b
 //   input_conv      h + conv(h): a short causal convolution per channel over each sequence's tokens, whose last
 //                   inputs are a request's state
 //   token_shift     several blends of a token's input with the input of the token before it (a request's state)
@@ -16,19 +17,22 @@ namespace tlie {
 // One workgroup a row.  rows == nullptr: row t of the residual gets the deltas added in place.  With a history
 // (count > 0): the residual is the history's last entry, history[count - 1], and what is normed (and written to
 // `mixed`, the residual of the layer to come) is sum_j hw[j] * history[j][t].  rows != nullptr: only the rows named
-// there, nothing but `out` written.  out == nullptr: no norm, only the sums.
+// there, nothing but `out` written.  out == nullptr: no norm, only the sums.  row_scale (or null): row t's second delta
+// is multiplied by s2 * row_scale[t * row_scale_stride].  centred 0: an RMS norm (no mean is taken off).
 template <typename D1, typename D2, typename W, typename O>
 __global__ void __launch_bounds__(256)
 layer_norm_kernel(float* __restrict__ residual, const D1* __restrict__ d1, int n1, size_t stride1, float s1,
-                  const D2* __restrict__ d2, int n2, size_t stride2, float s2, const float* __restrict__ history,
-                  size_t history_stride, int history_count, const W* __restrict__ history_weight, float* __restrict__ mixed,
+                  const D2* __restrict__ d2, int n2, size_t stride2, float s2, const float* __restrict__ row_scale,
+                  int row_scale_stride, int centred, const float* __restrict__ history, size_t history_stride,
+                  int history_count, const W* __restrict__ history_weight, float* __restrict__ mixed,
                   const W* __restrict__ weight, const W* __restrict__ bias, float eps, O* __restrict__ out,
                   const int* __restrict__ rows, int hidden) {
   extern __shared__ float row_values[];
   __shared__ float scratch[16];
   const int t = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
   const size_t at = static_cast<size_t>(t) * hidden;
-  float sum = 0.f;
+  if (row_scale != nullptr) s2 *= row_scale[static_cast<size_t>(t) * row_scale_stride];
+  float sum = 0.f;                                     // of x, or (not centred) of x^2
   for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
     float x = residual[at + c];
     if (d1 != nullptr) x += s1 * sum_splits(d1 + at + c, n1, stride1);
@@ -41,16 +45,21 @@ layer_norm_kernel(float* __restrict__ residual, const D1* __restrict__ d1, int n
       if (rows == nullptr) mixed[at + c] = x;
     }
     row_values[c] = x;
-    sum += x;
+    sum += centred ? x : x * x;
   }
   if (out == nullptr) return;
-  const float mean = block_sum(sum, scratch) / static_cast<float>(hidden);
-  float squares = 0.f;
-  for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
-    const float d = row_values[c] - mean;
-    squares += d * d;
+  float mean = block_sum(sum, scratch) / static_cast<float>(hidden), mean_square = mean;
+  if (centred) {
+    float squares = 0.f;
+    for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
+      const float d = row_values[c] - mean;
+      squares += d * d;
+    }
+    mean_square = block_sum(squares, scratch) / static_cast<float>(hidden);
+  } else {
+    mean = 0.f;
   }
-  const float r = 1.f / sqrtf(block_sum(squares, scratch) / static_cast<float>(hidden) + eps);
+  const float r = 1.f / sqrtf(mean_square + eps);
   O* dst = out + static_cast<size_t>(blockIdx.x) * hidden;
   for (int c = threadIdx.x; c < hidden; c += blockDim.x) {
     float v = (row_values[c] - mean) * r * to_float(weight[c]);
@@ -75,15 +84,17 @@ __device__ __forceinline__ void load8_splits(const D* __restrict__ part, int nsp
 template <typename D1, typename D2, typename W, typename O>
 __global__ void __launch_bounds__(256)
 layer_norm_wide_kernel(float* __restrict__ residual, const D1* __restrict__ d1, int n1, size_t stride1, float s1,
-                       const D2* __restrict__ d2, int n2, size_t stride2, float s2, const float* __restrict__ history,
-                       size_t history_stride, int history_count, const W* __restrict__ history_weight, float* __restrict__ mixed,
+                       const D2* __restrict__ d2, int n2, size_t stride2, float s2, const float* __restrict__ row_scale,
+                       int row_scale_stride, int centred, const float* __restrict__ history, size_t history_stride,
+                  int history_count, const W* __restrict__ history_weight, float* __restrict__ mixed,
                        const W* __restrict__ weight, const W* __restrict__ bias, float eps, O* __restrict__ out,
                        const int* __restrict__ rows, int hidden) {
   extern __shared__ float row_values[];
   __shared__ float scratch[16];
   const int t = rows != nullptr ? rows[blockIdx.x] : blockIdx.x;
   const size_t at = static_cast<size_t>(t) * hidden;
-  float sum = 0.f;
+  if (row_scale != nullptr) s2 *= row_scale[static_cast<size_t>(t) * row_scale_stride];
+  float sum = 0.f;                                     // of x, or (not centred) of x^2
   for (int c = threadIdx.x * 8; c < hidden; c += blockDim.x * 8) {
     float x[8];
     load8(residual + at + c, x);
@@ -116,18 +127,23 @@ layer_norm_wide_kernel(float* __restrict__ residual, const D1* __restrict__ d1, 
     }
     store8(row_values + c, x);                        // (a thread reads back only what it wrote itself)
 #pragma unroll
-    for (int j = 0; j < 8; ++j) sum += x[j];
+    for (int j = 0; j < 8; ++j) sum += centred ? x[j] : x[j] * x[j];
   }
   if (out == nullptr) return;
-  const float mean = block_sum(sum, scratch) / static_cast<float>(hidden);
-  float squares = 0.f;
-  for (int c = threadIdx.x * 8; c < hidden; c += blockDim.x * 8) {
-    float x[8];
-    load8(row_values + c, x);
+  float mean = block_sum(sum, scratch) / static_cast<float>(hidden), mean_square = mean;
+  if (centred) {
+    float squares = 0.f;
+    for (int c = threadIdx.x * 8; c < hidden; c += blockDim.x * 8) {
+      float x[8];
+      load8(row_values + c, x);
 #pragma unroll
-    for (int j = 0; j < 8; ++j) squares += (x[j] - mean) * (x[j] - mean);
+      for (int j = 0; j < 8; ++j) squares += (x[j] - mean) * (x[j] - mean);
+    }
+    mean_square = block_sum(squares, scratch) / static_cast<float>(hidden);
+  } else {
+    mean = 0.f;
   }
-  const float r = 1.f / sqrtf(block_sum(squares, scratch) / static_cast<float>(hidden) + eps);
+  const float r = 1.f / sqrtf(mean_square + eps);
   O* dst = out + static_cast<size_t>(blockIdx.x) * hidden;
   for (int c = threadIdx.x * 8; c < hidden; c += blockDim.x * 8) {
     float x[8], w[8];
@@ -352,15 +368,18 @@ using namespace tlie;
 static inline bool aligned16(const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; }
 
 // residual: float [tokens, hidden] (changed in place when there are deltas and no rows); d1, d2 (or null): products of
-// d1_dtype, d2_dtype; history (or null, with history_count 0): float, entry j at history + j * history_stride, the last
+// d1_dtype, d2_dtype, added s1 times and s2 times (row t's d2 also row_scale[t * row_scale_stride] times, if there is a
+// row_scale); centred: take the mean off (0: an RMS norm); history (or null, with history_count 0): float, entry j at history + j * history_stride, the last
 // entry being the residual itself; history_weight: [history_count] of w_dtype; mixed: float [tokens, hidden]; weight,
 // bias (bias may be null) [hidden] of w_dtype; out (or null) [count, hidden] of out_dtype; rows (or null): int [count].
 extern "C" int tlie_layer_norm(float* residual, const void* d1, int d1_dtype, int n1, long long stride1, float s1,
-                               const void* d2, int d2_dtype, int n2, long long stride2, float s2, const float* history,
-                               long long history_stride, int history_count, const void* history_weight, float* mixed,
+                               const void* d2, int d2_dtype, int n2, long long stride2, float s2, const float* row_scale,
+                               int row_scale_stride, int centred, const float* history, long long history_stride,
+                               int history_count, const void* history_weight, float* mixed,
                                const void* weight, const void* bias, int w_dtype, float eps, void* out, int out_dtype,
                                const int* rows, int count, int hidden, void* stream) {
   if (count <= 0 || hidden <= 0 || hidden > 16000 || history_count < 0 || n1 < 1 || n2 < 1) return kBadArgument;
+  if (row_scale != nullptr && row_scale_stride < 1) return kBadArgument;
   if (history_count > 0 && (history == nullptr || history_weight == nullptr || (rows == nullptr && mixed == nullptr))) return kBadArgument;
   if (out != nullptr && (weight == nullptr || !(eps > 0.f))) return kBadArgument;
   hipStream_t s = (hipStream_t)stream;
@@ -375,14 +394,14 @@ extern "C" int tlie_layer_norm(float* residual, const void* d1, int d1_dtype, in
   if (d1_dtype == C1 && d2_dtype == C2 && w_dtype == WC && out_dtype == OC) {                                            \
     if (wide)                                                                                                            \
       hipLaunchKernelGGL((layer_norm_wide_kernel<D1, D2, W, O>), dim3(count), dim3(threads), lds, s, residual,            \
-                         (const D1*)d1, n1, (size_t)stride1, s1, (const D2*)d2, n2, (size_t)stride2, s2, history,         \
-                         (size_t)history_stride, history_count, (const W*)history_weight, mixed, (const W*)weight,        \
-                         (const W*)bias, eps, (O*)out, rows, hidden);                                                     \
+                         (const D1*)d1, n1, (size_t)stride1, s1, (const D2*)d2, n2, (size_t)stride2, s2, row_scale,     \
+                         row_scale_stride, centred, history, (size_t)history_stride, history_count,                        \
+                         (const W*)history_weight, mixed, (const W*)weight, (const W*)bias, eps, (O*)out, rows, hidden);  \
     else                                                                                                                 \
       hipLaunchKernelGGL((layer_norm_kernel<D1, D2, W, O>), dim3(count), dim3(256), lds, s, residual, (const D1*)d1, n1,  \
-                         (size_t)stride1, s1, (const D2*)d2, n2, (size_t)stride2, s2, history, (size_t)history_stride,    \
-                         history_count, (const W*)history_weight, mixed, (const W*)weight, (const W*)bias, eps, (O*)out,  \
-                         rows, hidden);                                                                                  \
+                         (size_t)stride1, s1, (const D2*)d2, n2, (size_t)stride2, s2, row_scale, row_scale_stride, centred,       \
+                         history, (size_t)history_stride, history_count, (const W*)history_weight, mixed, (const W*)weight,       \
+                         (const W*)bias, eps, (O*)out, rows, hidden);                                                    \
     return launch_status();                                                                                              \
   }
   TLIE_CASE(kF32, float, kF32, float, kF32, float, kF32, float)

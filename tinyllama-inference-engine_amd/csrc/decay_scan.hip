@@ -4,6 +4,7 @@
 //   KIND 2:      o = (S + diag(u) k v^T)^T q,   then S' = diag(w) S + k v^T   (u: a bonus per key channel that
 //                only the current token gets)
 // KIND 0 takes one decay a head (the same for every channel and token), KIND 1 and 2 one a token and channel.
+// An activation on the way in (silu, optional): q, k and v are z * sigmoid(z) of their products' columns.
 // S is the request's state (zero when it is admitted) and is carried from step to step; the state, the decays and
 // all sums are float whatever type q, k and v come in.  There is no softmax and no denominator.
 //
@@ -24,6 +25,9 @@ namespace tlie {
 
 constexpr int kScanBatch = 4, kScanSlice = 32;
 
+// silu(z), or z itself (an activation's code of the C interface).
+__device__ __forceinline__ float activated(float z, int silu) { return silu ? z / (1.f + expf(-z)) : z; }
+
 // Columns col .. of a product [nsplit][tokens][row] (possibly partial sums that lie `stride` elements apart).
 struct ScanColumns {
   const void* data;
@@ -40,7 +44,7 @@ struct ScanColumns {
 template <typename D, int DW, int WAVES, int MODE, int KIND>
 __global__ void __launch_bounds__(64 * WAVES)
 decay_scan_kernel(ScanColumns qc, ScanColumns kc, ScanColumns vc, const float* __restrict__ decay,
-                  const float* __restrict__ head_decay, const float* __restrict__ bonus, float q_scale, float k_scale,
+                  const float* __restrict__ head_decay, const float* __restrict__ bonus, int silu, float q_scale, float k_scale,
                   float* __restrict__ state, float* __restrict__ parts, const int* __restrict__ seq_start,
                   const int* __restrict__ seq_slot, float* __restrict__ out, int heads, int dim, int vdim, int tiles,
                   int slices, size_t slot_stride) {
@@ -95,11 +99,11 @@ decay_scan_kernel(ScanColumns qc, ScanColumns kc, ScanColumns vc, const float* _
       for (int j = 0; j < NJ; ++j) {
         const int d = base + lane + 64 * j;
         const bool there = b < nb && lane + 64 * j < DW && d < dim;
-        rq[b][j] = MODE != 1 && there ? sum_splits(qd + t * qc.row + qc.col + h * dim + d, qc.nsplit, static_cast<size_t>(qc.stride)) * q_scale : 0.f;
-        rk[b][j] = there ? sum_splits(kd + t * kc.row + kc.col + h * dim + d, kc.nsplit, static_cast<size_t>(kc.stride)) * k_scale : 0.f;
+        rq[b][j] = MODE != 1 && there ? activated(sum_splits(qd + t * qc.row + qc.col + h * dim + d, qc.nsplit, static_cast<size_t>(qc.stride)), silu) * q_scale : 0.f;
+        rk[b][j] = there ? activated(sum_splits(kd + t * kc.row + kc.col + h * dim + d, kc.nsplit, static_cast<size_t>(kc.stride)), silu) * k_scale : 0.f;
         rw[b][j] = KIND >= 1 && there ? decay[t * heads * dim + h * dim + d] : 1.f;
       }
-      rv[b] = b < nb && live ? sum_splits(vd + t * vc.row + vc.col + h * vdim + col, vc.nsplit, static_cast<size_t>(vc.stride)) : 0.f;
+      rv[b] = b < nb && live ? activated(sum_splits(vd + t * vc.row + vc.col + h * vdim + col, vc.nsplit, static_cast<size_t>(vc.stride)), silu) : 0.f;
     }
   };
   fetch(first);
@@ -312,7 +316,7 @@ using namespace tlie;
 
 // q, k, v: columns of products of one type (see ScanColumns), q and k `heads * dim` wide, v `heads * vdim`; decay:
 // float [tokens, heads * dim] (kind 1, 2) or null; head_decay: float [heads] (kind 0) or null; bonus: float
-// [heads * dim] (kind 2) or null; state: float [slots, heads, tiles, dim * 64], tiles = ceil(vdim / 64), a slot's row
+// [heads * dim] (kind 2) or null; silu: q, k and v are silu of the columns; state: float [slots, heads, tiles, dim * 64], tiles = ceil(vdim / 64), a slot's row
 // slot_stride floats after the one before it (a row may hold more than the scan's part); seq_start
 // [sequences + 1], seq_slot [sequences] (negative: skipped); out: float [tokens, heads * vdim].  slices 0: every
 // sequence's tokens are walked in order; slices > 0 (at least ceil(most tokens of a sequence / 32)): in slices of
@@ -320,7 +324,7 @@ using namespace tlie;
 extern "C" int tlie_decay_scan(const void* q, int q_nsplit, long long q_stride, int q_row, int q_col, const void* k,
                                int k_nsplit, long long k_stride, int k_row, int k_col, const void* v, int v_nsplit,
                                long long v_stride, int v_row, int v_col, int dtype, int kind, const float* decay,
-                               const float* head_decay, const float* bonus, float q_scale, float k_scale, float* state,
+                               const float* head_decay, const float* bonus, int silu, float q_scale, float k_scale, float* state,
                                const int* seq_start, const int* seq_slot, float* out, int sequences, int heads, int dim,
                                int vdim, int slices, float* parts, long long slot_stride, void* stream) {
   if (sequences <= 0 || heads <= 0 || dim <= 0 || dim > 256 || vdim <= 0 || kind < 0 || kind > 2) return kBadArgument;
@@ -337,7 +341,7 @@ extern "C" int tlie_decay_scan(const void* q, int q_nsplit, long long q_stride, 
       vc{v, v_nsplit, v_stride, v_row, v_col};
 #define TLIE_LAUNCH(D, DW, WAVES, MODE, KIND, GRID)                                                                   \
   hipLaunchKernelGGL((decay_scan_kernel<D, DW, WAVES, MODE, KIND>), GRID, dim3(64 * WAVES), 0, s, qc, kc, vc, decay,   \
-                     head_decay, bonus, q_scale, k_scale, state, parts, seq_start, seq_slot, out, heads, dim, vdim,    \
+                     head_decay, bonus, silu, q_scale, k_scale, state, parts, seq_start, seq_slot, out, heads, dim, vdim,    \
                      tiles, slices, (size_t)slot_stride)
 #define TLIE_SIZES(D, MODE, KIND, GRID)                                                                               \
   if (dim <= 32) TLIE_LAUNCH(D, 32, 1, MODE, KIND, GRID);                                                             \

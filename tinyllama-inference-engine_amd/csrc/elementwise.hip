@@ -286,6 +286,31 @@ __global__ void sigmoid_gate_wide_kernel(A* __restrict__ values, const D* __rest
   }
 }
 
+// ---- values[t, h * dv + e] *= sigmoid(pre[t, col + h]): one number a head, its pre-activations columns of a wider product.
+// V columns a thread (8: dv a multiple of 8, 16-byte aligned rows); the sigmoid and the product float --------------------
+template <typename D, typename A, int V>
+__global__ void head_gate_kernel(A* __restrict__ values, const D* __restrict__ pre, int nsplit, size_t split_stride,
+                                 int col, int row_width, size_t groups, int cols, int dv) {
+  const int per_row = cols / V;
+  for (size_t index = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; index < groups;
+       index += static_cast<size_t>(gridDim.x) * blockDim.x) {
+    const size_t t = index / per_row;
+    const int c = static_cast<int>(index % per_row) * V;
+    const float z = sum_splits(pre + t * row_width + col + c / dv, nsplit, split_stride);
+    const float gate = 1.f / (1.f + expf(-z));
+    A* at = values + t * cols + c;
+    if constexpr (V == 8) {
+      float v[8];
+      load8(at, v);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] *= gate;
+      store8(at, v);
+    } else {
+      at[0] = from_float<A>(to_float(at[0]) * gate);
+    }
+  }
+}
+
 // ---- x <- cap * tanh(x / cap), in place (capped logits) --------------------------------------------------------------
 __global__ void softcap_kernel(float* __restrict__ x, size_t total, float cap) {
   for (size_t index = blockIdx.x * static_cast<size_t>(blockDim.x) + threadIdx.x; index < total;
@@ -481,6 +506,33 @@ extern "C" int tlie_sigmoid_gate(void* values, int act_dtype, const void* pre, i
     hipLaunchKernelGGL((sigmoid_gate_kernel<D, A>), dim3(blocks), dim3(256), 0, s, (A*)values, (const D*)pre, nsplit, \
                        (size_t)split_stride, col, row_width, total, cols);                                       \
     return launch_status();                                                                                      \
+  }
+  TLIE_CASE(kF32, float, kF32, float)
+  TLIE_CASE(kF32, float, kBF16, bf16)
+  TLIE_CASE(kBF16, bf16, kBF16, bf16)
+#undef TLIE_CASE
+  return kBadArgument;
+}
+
+// values: [rows, heads * dv] of act_dtype, changed in place; pre: a product [nsplit][rows][row_width] whose columns
+// col .. col + heads - 1 are the heads' gates' pre-activations.
+extern "C" int tlie_head_gate(void* values, int act_dtype, const void* pre, int pre_dtype, int nsplit, long long split_stride,
+                              int col, int row_width, int rows, int heads, int dv, void* stream) {
+  if (rows <= 0 || heads <= 0 || dv <= 0 || col < 0 || col + heads > row_width || nsplit < 1) return kBadArgument;
+  const int cols = heads * dv;
+  const bool wide = dv % 8 == 0 && (reinterpret_cast<uintptr_t>(values) & 31) == 0;
+  const size_t groups = static_cast<size_t>(rows) * cols / (wide ? 8 : 1);
+  const int blocks = static_cast<int>((groups + 255) / 256 < 16384 ? (groups + 255) / 256 : 16384);
+  hipStream_t s = (hipStream_t)stream;
+#define TLIE_CASE(DC, D, AC, A)                                                                                       \
+  if (pre_dtype == DC && act_dtype == AC) {                                                                           \
+    if (wide)                                                                                                         \
+      hipLaunchKernelGGL((head_gate_kernel<D, A, 8>), dim3(blocks), dim3(256), 0, s, (A*)values, (const D*)pre, nsplit, \
+                         (size_t)split_stride, col, row_width, groups, cols, dv);                                     \
+    else                                                                                                              \
+      hipLaunchKernelGGL((head_gate_kernel<D, A, 1>), dim3(blocks), dim3(256), 0, s, (A*)values, (const D*)pre, nsplit, \
+                         (size_t)split_stride, col, row_width, groups, cols, dv);                                     \
+    return launch_status();                                                                                           \
   }
   TLIE_CASE(kF32, float, kF32, float)
   TLIE_CASE(kF32, float, kBF16, bf16)

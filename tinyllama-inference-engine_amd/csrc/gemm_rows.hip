@@ -23,6 +23,8 @@
 //   * store: float32 [M, N] (qkv for the rotation kernel; logits).
 //   * SiLU gate: W's rows alternate gate and up (g0, u0, g1, u1, ...); out[m, i] = silu(g) * u,
 //     bfloat16 [M, N / 2].
+//   * squared ReLU, for feed-forwards without a gate: out[m, n] = s * max(y, 0)^2, bfloat16 [M, N], s = 1 or a number
+//     of the row's own for every block of columns (a routed feed-forward's weights of its experts).
 //   * residual: residual[m, n] += y (float32, in place: every element has one owner), and for the
 //     norm that reads the residual next: xg[m, n] = bfloat16(residual * g_next[n]) and the partial
 //     sums of squares per row and 16 columns.
@@ -43,7 +45,7 @@ union RowPack {
   bf16x8 v;
 };
 
-constexpr int kEpilogueStore = 0, kEpilogueSilu = 1, kEpilogueResidual = 2, kEpilogueRope = 3;
+constexpr int kEpilogueStore = 0, kEpilogueSilu = 1, kEpilogueResidual = 2, kEpilogueRope = 3, kEpilogueRelu2 = 4;
 
 struct RowsArgs {
   const uint16_t* x;          // [M, K] bfloat16
@@ -60,17 +62,22 @@ struct RowsArgs {
   float gate_alpha;
   // outputs
   float* y;                   // store: [M, N]
-  uint16_t* act;              // SiLU: [M, N / 2]
+  uint16_t* act;              // SiLU: [M, N / 2]; squared ReLU: [M, N]
   float* residual;            // residual: [M, N], updated in place
   const uint16_t* next_weight;  // residual: [N] bfloat16 weight of the next norm, or null
-  const float* next_weight_f32; // the same when that weight is kept in float32
+  union {
+    const float* next_weight_f32; // the same when that weight is kept in float32
+    const float* act_scale;     // squared ReLU: [M, act_scale_cols], a number for every act_block columns, or null
+  };
   uint16_t* xg;               // residual: [M, N] bfloat16(residual * next weight), or null
   float* ssq_out;             // residual: [ceil(N / rows_per_block), 16], or null
   // rotation and cache write: N = (nq + 2 nkv) * d, heads in the order q | k | v
   const int* positions;       // [M]
   const int* slot_map;        // [M] cache row of each token (page * page_size + row), or -1
   const float* inv_freq;      // [rot_dim / 2], or null: no rotation
-  int rot_dim, nq, nkv, d, page_size;
+  union { int rot_dim, act_scale_cols; };
+  union { int nq, act_block; };
+  int nkv, d, page_size;
   float gate_limit;
   uint16_t* q_out;            // [M, nq * d]
   uint16_t* cache;            // [pages, 2, nkv, page_size * d]: keys [row][dim], values [dim][row]
@@ -202,6 +209,8 @@ gemm_rows_kernel(const RowsArgs a) {
         pre_old[st][turn] = a.residual[static_cast<size_t>(token) * a.N + n];
         if (a.xg != nullptr) pre_g[st][turn] = a.next_weight != nullptr ? bf16_bits_to_float(a.next_weight[n]) : a.next_weight_f32[n];
       }
+      if (EPILOGUE == kEpilogueRelu2)
+        pre_g[st][turn] = live && a.act_scale != nullptr ? a.act_scale[static_cast<size_t>(token) * a.act_scale_cols + n / a.act_block] : 1.f;
       if (EPILOGUE == kEpilogueRope && live) {
         const int head = n / a.d, p = n % a.d;
         if (a.inv_freq != nullptr && head < a.nq + a.nkv && p < a.rot_dim)
@@ -278,6 +287,10 @@ gemm_rows_kernel(const RowsArgs a) {
           const float gated = gated_value(value, up, a.gate_kind, a.gate_alpha, a.gate_limit);
           a.act[static_cast<size_t>(token) * (a.N / 2) + (n >> 1)] = __bfloat16_as_ushort(__float2bfloat16(gated));
         }
+      } else if (EPILOGUE == kEpilogueRelu2) {
+        const float positive = fmaxf(value, 0.f), weight = pre_g[st][turn];
+        if (live)                                            // (an expert that the token does not use: zero, whatever its sums are)
+          a.act[static_cast<size_t>(token) * a.N + n] = __bfloat16_as_ushort(__float2bfloat16(weight != 0.f ? weight * positive * positive : 0.f));
       } else if (EPILOGUE == kEpilogueRope) {
         const float other = __shfl_xor(value, 1, 64);        // the pair's other element, when this one is rotated
         if (live) {
@@ -387,6 +400,8 @@ using namespace tlie;
 // x [M, K], w [N, K], bias [N] or null: bfloat16; M <= 16, K % 8 == 0.
 // ssq_in [strips_in, 16] or null (then no row scale); width: the normed input's width.
 // epilogue 0: y float [M, N].  1: act bfloat16 [M, N / 2], N even, W's rows alternating gate, up.
+// 4: act bfloat16 [M, N] = s * max(y, 0)^2, s from act_scale float [M, act_scale_cols] (a number for every act_block
+// columns), or 1 when it is null.
 // 2: residual float [M, N] += y; if xg is given, next_weight [N] (bfloat16 if next_weight_dtype is 1,
 // else float) and xg bfloat16 [M, N]; if ssq_out is given, float [ceil(N / rows_per_block) * max(1, rows_per_block / 16), 16]
 // (all of it is written).
@@ -400,13 +415,17 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
                               const void* next_weight, int next_weight_dtype, void* xg, float* ssq_out,
                               const int* positions, const int* slot_map, const float* inv_freq, int rot_dim, int nq,
                               int nkv, int d, int page_size, void* q_out, void* cache, int waves, int rows_per_block,
-                              int gate_kind, float gate_alpha, float gate_limit, void* stream) {
+                              int gate_kind, float gate_alpha, float gate_limit, const float* act_scale, int act_scale_cols,
+                              int act_block, void* stream) {
   if (gate_kind != kGateSilu && gate_kind != kGateClampedSwish) return kBadArgument;
   if (M <= 0 || M > 16 || N <= 0 || K <= 0 || (K & 7) != 0 || (waves != 2 && waves != 4 && waves != 8 && waves != 16)) return kBadArgument;
   if (!(rows_per_block >= 2 && rows_per_block <= 16 && rows_per_block % 2 == 0) && !(rows_per_block == 32 && waves <= 8)) return kBadArgument;
   if (ssq_in != nullptr && (strips_in <= 0 || width <= 0)) return kBadArgument;
   if (epilogue == kEpilogueStore && y == nullptr) return kBadArgument;
   if (epilogue == kEpilogueSilu && (act == nullptr || (N & 1) != 0)) return kBadArgument;
+  if (epilogue == kEpilogueRelu2 &&
+      (act == nullptr || (act_scale != nullptr && (act_block <= 0 || act_scale_cols < (N + act_block - 1) / act_block))))
+    return kBadArgument;
   if (epilogue == kEpilogueResidual && (residual == nullptr || (xg != nullptr && next_weight == nullptr))) return kBadArgument;
   if (epilogue == kEpilogueRope &&
       (positions == nullptr || slot_map == nullptr || q_out == nullptr || cache == nullptr || nq <= 0 || nkv <= 0 || d <= 0 ||
@@ -421,9 +440,11 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
   a.next_weight = next_weight_dtype == kBF16 ? (const uint16_t*)next_weight : nullptr;
   a.next_weight_f32 = next_weight_dtype == kBF16 ? nullptr : (const float*)next_weight;
   a.xg = (uint16_t*)xg, a.ssq_out = ssq_out;
+  if (epilogue == kEpilogueRelu2) a.act_scale = act_scale;
   a.positions = positions, a.slot_map = slot_map, a.inv_freq = inv_freq, a.rot_dim = rot_dim;
   a.gate_kind = gate_kind, a.gate_alpha = gate_alpha, a.gate_limit = gate_limit;
   a.nq = nq, a.nkv = nkv, a.d = d, a.page_size = page_size, a.q_out = (uint16_t*)q_out, a.cache = (uint16_t*)cache;
+  if (epilogue == kEpilogueRelu2) a.act_scale_cols = act_scale_cols, a.act_block = act_block;
   const dim3 grid((N + rows_per_block - 1) / rows_per_block);
   hipStream_t s = (hipStream_t)stream;
 #define TLIE_CASE(E)                                                                                  \
@@ -448,6 +469,7 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
   TLIE_CASE(kEpilogueSilu)
   TLIE_CASE(kEpilogueResidual)
   TLIE_CASE(kEpilogueRope)
+  TLIE_CASE(kEpilogueRelu2)
 #undef TLIE_CASE
   return kBadArgument;
 }

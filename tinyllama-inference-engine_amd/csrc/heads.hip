@@ -71,6 +71,74 @@ head_combine_kernel(const float* __restrict__ a, int heads, int dv, int pair_gro
   for (int e = lane; e < dv; e += 64) emit(e, value(e) * r);
 }
 
+// The same for one result a head that is too wide for a wave (more than 512 dims: all heads of a mixer normed together
+// are one head here): a workgroup a head, eight dims a thread and access, a thread's first kKept groups kept between the
+// sum of squares and the output.  dv a multiple of 8, rows of `a`, weight, gate and out at multiples of 32 bytes, the
+// gate's parts a multiple of 8 apart.
+template <typename D, typename W, typename A>
+__global__ void __launch_bounds__(256)
+head_combine_wide_kernel(const float* __restrict__ a, int heads, int dv, float eps, const W* __restrict__ weight, float mult,
+                         const D* __restrict__ gate, int gate_nsplit, size_t gate_split_stride, int gate_row, int gate_col,
+                         int gate_kind, A* __restrict__ out) {
+  __shared__ float scratch[16];
+  constexpr int kKept = 2;
+  const int t = blockIdx.x, h = blockIdx.y;
+  const size_t base = (static_cast<size_t>(t) * heads + h) * dv;
+  float kept[kKept][8];
+  float squares = 0.f;
+#pragma unroll
+  for (int i = 0; i < kKept; ++i) {
+    const int e = (threadIdx.x + i * blockDim.x) * 8;
+    if (e < dv) {
+      load8(a + base + e, kept[i]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) squares += kept[i][j] * kept[i][j];
+    }
+  }
+  for (int e = (threadIdx.x + kKept * blockDim.x) * 8; e < dv; e += blockDim.x * 8) {
+    float v[8];
+    load8(a + base + e, v);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) squares += v[j] * v[j];
+  }
+  const float r = mult / sqrtf(block_sum(squares, scratch) / static_cast<float>(dv) + eps);
+  auto emit = [&](int e, float (&v)[8]) {
+    const int c = h * dv + e;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] *= r;
+    if (weight != nullptr) {
+      float w[8];
+      load8(weight + c, w);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] *= w[j];
+    }
+    if (gate != nullptr) {
+      float z[8];
+      const D* from = gate + static_cast<size_t>(t) * gate_row + gate_col + c;
+      load8(from, z);
+      for (int s = 1; s < gate_nsplit; ++s) {
+        float more[8];
+        load8(from + s * gate_split_stride, more);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) z[j] += more[j];
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] *= (gate_kind == 1 ? z[j] : 1.f) / (1.f + expf(-z[j]));
+    }
+    store8(out + base + e, v);
+  };
+#pragma unroll
+  for (int i = 0; i < kKept; ++i) {
+    const int e = (threadIdx.x + i * blockDim.x) * 8;
+    if (e < dv) emit(e, kept[i]);
+  }
+  for (int e = (threadIdx.x + kKept * blockDim.x) * 8; e < dv; e += blockDim.x * 8) {
+    float v[8];
+    load8(a + base + e, v);
+    emit(e, v);
+  }
+}
+
 }  // namespace tlie
 
 using namespace tlie;
@@ -87,8 +155,18 @@ extern "C" int tlie_head_combine(const float* a, int tokens, int heads, int dv, 
   if (heads > 4 * 65535) return kBadArgument;
   const dim3 grid(tokens, (heads + 3) / 4);
   hipStream_t s = (hipStream_t)stream;
+  const bool wide = pair_group == 0 && dv > 512 && dv % 8 == 0 && heads <= 65535 && gate_row % 8 == 0 && gate_col % 8 == 0 &&
+                    (gate_nsplit <= 1 || gate_split_stride % 8 == 0) &&
+                    ((reinterpret_cast<uintptr_t>(a) | reinterpret_cast<uintptr_t>(weight) | reinterpret_cast<uintptr_t>(gate) |
+                      reinterpret_cast<uintptr_t>(out)) & 31) == 0;
 #define TLIE_CASE(GC, D, WC, W, AC, A)                                                                                   \
   if (gate_dtype == GC && weight_dtype == WC && out_dtype == AC) {                                                       \
+    if (wide) {                                                                                                          \
+      hipLaunchKernelGGL((head_combine_wide_kernel<D, W, A>), dim3(tokens, heads), dim3(256), 0, s, a, heads, dv, eps,    \
+                         (const W*)weight, mult, (const D*)gate, gate_nsplit, (size_t)gate_split_stride, gate_row,       \
+                         gate_col, gate_kind, (A*)out);                                                                  \
+      return launch_status();                                                                                            \
+    }                                                                                                                    \
     hipLaunchKernelGGL((head_combine_kernel<D, W, A>), grid, dim3(256), 0, s, a, heads, dv, pair_group, parts, lambda, eps,     \
                        (const W*)weight, mult, (const D*)gate, gate_nsplit, (size_t)gate_split_stride, gate_row, gate_col, \
                        gate_kind, (A*)out);                                                                                          \

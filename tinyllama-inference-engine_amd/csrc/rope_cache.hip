@@ -149,6 +149,7 @@ __global__ void rope_cache_wide_kernel(const D* __restrict__ qkv, const int* __r
 //                    the weight, before the rotation
 //   values_are_keys  the product has no value columns: a key head's columns as projected (before norm and rotation)
 //                    are also its value head (nv = nkv, dv = d)
+//   head_scale       float [nq]: query head h is multiplied by head_scale[h] (a factor of its scores)
 //   temp_coef, temp_every   a query at position p is multiplied by 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)
 struct PlaceOptions {
   const float* q_norm;
@@ -157,6 +158,7 @@ struct PlaceOptions {
   int values_are_keys;
   float temp_coef;
   float temp_every;
+  const float* head_scale;
   int stage;         // the launch gave LDS for the q and k columns (set by the entry point)
 };
 
@@ -201,7 +203,10 @@ __global__ void qkv_place_kernel(const D* __restrict__ qkv, int nsplit, size_t s
   // a column of q or k after its norm (and, for a query, its temperature), before the rotation
   auto normed = [&](int c) {
     const float v = raw(c);
-    if (c < nq * d) return options.q_norm != nullptr ? v * q_scale * options.q_norm[c] : v * q_scale;
+    if (c < nq * d) {
+      const float scaled = options.head_scale != nullptr ? v * q_scale * options.head_scale[c / d] : v * q_scale;
+      return options.q_norm != nullptr ? scaled * options.q_norm[c] : scaled;
+    }
     return options.k_norm != nullptr ? v * k_scale * options.k_norm[c - nq * d] : v;
   };
   const int slot = nkv > 0 ? slot_map[t] : -1;
@@ -243,7 +248,7 @@ extern "C" int tlie_qkv_place(const void* qkv, int in_dtype, int nsplit, long lo
                               const int* slot_map, const float* inv_freq, int rot_dim, void* q_out, void* cache,
                               int act_dtype, int tokens, int nq, int nkv, int nv, int d, int dv, int page_size, int row_width,
                               const float* q_norm, const float* k_norm, float norm_eps, int values_are_keys, float temp_coef,
-                              float temp_every, void* stream) {
+                              float temp_every, const float* head_scale, void* stream) {
   if (tokens <= 0 || nq <= 0 || nkv < 0 || d <= 0 || dv <= 0 || page_size <= 0 || nsplit < 1) return kBadArgument;
   if (rot_dim < 0 || rot_dim > d || rot_dim % 2 != 0 || (nkv > 0 && (cache == nullptr || slot_map == nullptr))) return kBadArgument;
   if (nv < 0 || nv > nkv || (nkv > 0 && (nv == 0 || nkv % nv != 0))) return kBadArgument;
@@ -260,7 +265,7 @@ extern "C" int tlie_qkv_place(const void* qkv, int in_dtype, int nsplit, long lo
   const size_t columns = static_cast<size_t>(nq + nkv) * d;
   const int stage = normed && columns <= 14000 ? 1 : 0;          // (beyond that a row does not fit beside the rest: every read goes to memory)
   const size_t lds = (static_cast<size_t>(rot_dim) + 16 + (stage ? columns : 0)) * sizeof(float);
-  const PlaceOptions options{q_norm, k_norm, norm_eps, values_are_keys, temp_coef, temp_every, stage};
+  const PlaceOptions options{q_norm, k_norm, norm_eps, values_are_keys, temp_coef, temp_every, head_scale, stage};
   hipStream_t s = (hipStream_t)stream;
 #define TLIE_CASE(DC, D, AC, A)                                                                                \
   if (in_dtype == DC && act_dtype == AC) {                                                                     \

@@ -4,6 +4,7 @@
 //                                                                      the new x in the activation type (for a product)
 //   side_gate         g[t, j] = gelu_tanh(pre[t, j]) * table[token[t], offset + j]
 //   residual_inject   x[t, :] = or += table[token[t], :] + vector      (table or vector optional)
+//   pass_input        out[t] = [x[t, :]; table[token[t], :]], side by side, in the activation type (for a product)
 //
 // The residual is float, and so are all sums here.
 #include "common.h"
@@ -66,6 +67,28 @@ residual_inject_kernel(float* __restrict__ residual, const int* __restrict__ tok
     if (row != nullptr) v += to_float(row[c]);
     if (vector != nullptr) v += to_float(vector[c]);
     x[c] = v;
+  }
+}
+
+template <typename W, typename A, int V>
+__global__ void __launch_bounds__(256)
+pass_input_kernel(const float* __restrict__ residual, const int* __restrict__ tokens, const W* __restrict__ table,
+                  A* __restrict__ out, int width) {
+  const int t = blockIdx.x;
+  const float* x = residual + static_cast<size_t>(t) * width;
+  const W* row = table + static_cast<size_t>(tokens[t]) * width;
+  A* to = out + static_cast<size_t>(t) * 2 * width;
+  for (int c = (blockIdx.y * 256 + threadIdx.x) * V; c < width; c += gridDim.y * 256 * V) {
+    if constexpr (V == 8) {
+      float v[8];
+      load8(x + c, v);
+      store8(to + c, v);
+      load8(row + c, v);
+      store8(to + width + c, v);
+    } else {
+      to[c] = from_float<A>(x[c]);
+      to[width + c] = from_float<A>(to_float(row[c]));
+    }
   }
 }
 
@@ -138,4 +161,33 @@ extern "C" int tlie_residual_inject(float* residual, const int* tokens, const vo
   else
     return kBadArgument;
   return launch_status();
+}
+
+// residual: float [count, width]; tokens int32 [count]; table [vocab, width] of w_dtype; out: [count, 2 * width] of out_dtype.
+extern "C" int tlie_pass_input(const float* residual, const int* tokens, const void* table, int w_dtype, void* out,
+                               int out_dtype, int count, int width, void* stream) {
+  if (count <= 0 || width <= 0 || residual == nullptr || tokens == nullptr || table == nullptr || out == nullptr) return kBadArgument;
+  hipStream_t s = (hipStream_t)stream;
+  const bool wide = (width & 7) == 0 && ((reinterpret_cast<uintptr_t>(residual) | reinterpret_cast<uintptr_t>(table) |
+                                          reinterpret_cast<uintptr_t>(out)) & 31) == 0;
+  const int per_block = wide ? 2048 : 256;
+  int across = (width + per_block - 1) / per_block;
+  if (across > 64) across = 64;
+  const dim3 grid(count, across);
+#define TLIE_CASE(WC, W, AC, A)                                                                                       \
+  if (w_dtype == WC && out_dtype == AC) {                                                                             \
+    if (wide)                                                                                                         \
+      hipLaunchKernelGGL((pass_input_kernel<W, A, 8>), grid, dim3(256), 0, s, residual, tokens, (const W*)table,       \
+                         (A*)out, width);                                                                             \
+    else                                                                                                              \
+      hipLaunchKernelGGL((pass_input_kernel<W, A, 1>), grid, dim3(256), 0, s, residual, tokens, (const W*)table,       \
+                         (A*)out, width);                                                                             \
+    return launch_status();                                                                                           \
+  }
+  TLIE_CASE(kF32, float, kF32, float)
+  TLIE_CASE(kBF16, bf16, kF32, float)
+  TLIE_CASE(kBF16, bf16, kBF16, bf16)
+  TLIE_CASE(kF32, float, kBF16, bf16)
+#undef TLIE_CASE
+  return kBadArgument;
 }

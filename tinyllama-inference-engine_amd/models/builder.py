@@ -2,6 +2,8 @@
 own parameters; nothing here names an architecture."""
 from __future__ import annotations
 
+from functools import partial
+
 import torch
 
 from .. import parts as _parts  # noqa: F401  (fills the part registries)
@@ -9,6 +11,7 @@ from ..cache.manager import RunNeed
 from ..config.spec import ModelSpec, TensorSpec
 from .. import ops
 from ..ops import ResidualUpdated
+from ..parts.linear import Linear
 from ..registry import lookup
 from ..weights.arena import keep_in
 
@@ -42,6 +45,7 @@ class DecoderModel:
         self.final_norm = lookup("norm", spec.final_norm.kind)(spec.final_norm, dtype, device)
         self.head = lookup("head", spec.head.kind)(spec.head, dtype, device)
         self.run_vectors: dict[str, torch.Tensor] = {}       # the tensors of which runs add a row to the residual, by name
+        self.pass_inputs: dict[str, Linear] = {}             # the products that form a run's first residual, by the tensor's name
 
     def load(self, weights) -> None:
         """weights: tensors on the device by name: a dict, or a `ResidentWeights`, which brings a
@@ -58,6 +62,8 @@ class DecoderModel:
             if run.add_vector is not None and run.add_vector[0] not in self.run_vectors:
                 name = run.add_vector[0]
                 self.run_vectors[name] = keep_in(weights, weights[name].to(self.embedding.table.dtype).contiguous())
+            if run.pass_input is not None and run.pass_input not in self.pass_inputs:
+                self.pass_inputs[run.pass_input] = Linear(weights[run.pass_input], None, self.dtype, keep=partial(keep_in, weights))
             if run.depth_mix is not None and run.depth_mix not in self.run_vectors:
                 self.run_vectors[run.depth_mix] = keep_in(weights, weights[run.depth_mix].to(self.embedding.table.dtype).contiguous())
         release()
@@ -96,7 +102,7 @@ class DecoderModel:
             # a block may say which norm reads the residual first (its writer can then leave that
             # norm's inputs); a block that does not is handed a plain residual
             return block.entry_norm() if hasattr(block, "entry_norm") else None
-        first_norm = entry_norm(self.blocks[runs[0].layer])
+        first_norm = entry_norm(self.blocks[runs[0].layer]) if runs[0].pass_input is None else None
         lazy = first_norm.lazy_params() if first_norm is not None else None
         if few and hasattr(self.embedding, "forward_rows") and lazy is not None:
             residual, normed = self.embedding.forward_rows(ctx.tokens, lazy)
@@ -109,7 +115,10 @@ class DecoderModel:
             # a residual of several streams: all start as the embedding's output; the layers work on all of them
             residual = ops.stream_spread(residual, self.spec.streams)
         for index, run in enumerate(runs):
-            next_norm = entry_norm(self.blocks[runs[index + 1].layer]) if index + 1 < len(runs) else self.final_norm
+            if index + 1 == len(runs):
+                next_norm = self.final_norm
+            else:                       # (what reads the residual next is a product, where the next run begins with one)
+                next_norm = entry_norm(self.blocks[runs[index + 1].layer]) if runs[index + 1].pass_input is None else None
             if trace is not None:
                 ctx.trace_prefix = f"layer{index}."
             if run.add_embedding or run.add_vector is not None:
@@ -119,6 +128,13 @@ class DecoderModel:
                     pending = None
                 vector = self.run_vectors[run.add_vector[0]][run.add_vector[1]] if run.add_vector is not None else None
                 ops.residual_inject(residual, ctx.tokens, self.embedding.table if run.add_embedding else None, vector)
+            if run.pass_input is not None:
+                # a pass begins with a residual of its own: a product of the residual so far and the embedding's output
+                if pending is not None:
+                    self._settle(residual, pending, self.dtype)
+                    pending = None
+                joined = ops.pass_input(residual, ctx.tokens, self.embedding.table, self.dtype)
+                residual = self.pass_inputs[run.pass_input](joined, out_dtype=torch.float32, whole=True).dense(torch.float32)
             pending = self.blocks[run.layer].forward(residual, pending, ctx, bindings[index], next_norm=next_norm)
         if ctx.num_wanted == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=self.device)
@@ -158,7 +174,7 @@ class DecoderModel:
         normed = None
         logits = None
         for index, run in enumerate(runs):
-            if run.add_embedding or run.add_vector is not None:
+            if run.add_embedding or run.add_vector is not None or run.pass_input is not None:
                 raise ops.invalid_argument("runs that take the embedding or a vector again do not go with the mix over results")
             block = self.blocks[run.layer]
             if trace is not None:
@@ -195,7 +211,9 @@ class DecoderModel:
         """Adds what a block handed on into the residual now (a block whose result waits for the next norm)."""
         if isinstance(pending, ops.NormedDelta):
             ops.norm_add_rmsnorm(residual, pending.product, pending.weight, pending.eps, None, pending.eps, dtype)
-        else:
+        elif isinstance(pending, ops.ScaledSum):
+            ops.layer_norm(residual, pending, None, None, 0.0, dtype, want_out=False)
+        elif not isinstance(pending, ResidualUpdated):
             residual += ops.as_product(pending).dense(torch.float32)
 
 

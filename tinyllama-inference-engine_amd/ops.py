@@ -379,7 +379,8 @@ def qkv_place(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor | No
               rot_dim: int, cache: torch.Tensor | None, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
               act_dtype: torch.dtype, value_heads: int | None = None, extra_cols: int = 0,
               q_norm: torch.Tensor | None = None, k_norm: torch.Tensor | None = None, norm_eps: float = 0.0,
-              values_are_keys: bool = False, q_temp: tuple[float, float] | None = None) -> torch.Tensor:
+              values_are_keys: bool = False, q_temp: tuple[float, float] | None = None,
+              head_scale: torch.Tensor | None = None) -> torch.Tensor:
     """`rope_cache` for any sizes: value heads of `value_dim` dims (a page is then nkv planes of keys and
     after them nkv planes of transposed values), and num_kv_heads 0 for a layer that reads another
     layer's cache: only its queries [T, nq * d] are rotated and returned, nothing is written.
@@ -389,7 +390,7 @@ def qkv_place(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor | No
     together, are RMS-normed (norm_eps inside the root) and multiplied by the weight before the rotation.
     values_are_keys: the product holds no value columns; a key head as projected, before norm and rotation, is also its
     value head (value_dim = head_dim).  q_temp (coef, every): a query at position p is multiplied by
-    1 + coef * ln(floor((p + 1) / every) + 1)."""
+    1 + coef * ln(floor((p + 1) / every) + 1).  head_scale (float32 [nq]): query head h is multiplied by head_scale[h]."""
     _check_product(qkv, "qkv")
     if values_are_keys and (value_dim != head_dim or (value_heads is not None and value_heads != num_kv_heads) or num_kv_heads == 0):
         raise invalid_shape("qkv_place: values that are the keys have the keys' heads and size")
@@ -400,6 +401,10 @@ def qkv_place(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor | No
                 raise invalid_shape(f"qkv_place: {name} needs {count} entries and a positive eps")
     if q_temp is not None and not float(q_temp[1]) > 0.0:
         raise invalid_argument("qkv_place: the query temperature's period must be positive")
+    if head_scale is not None:
+        _device_tensor(head_scale, "head_scale", torch.float32)
+        if head_scale.shape != (num_heads,):
+            raise invalid_shape("qkv_place: head_scale needs one number a query head")
     _device_tensor(positions, "positions", torch.int32)
     tokens = qkv.rows
     value_heads = num_kv_heads if value_heads is None else int(value_heads)
@@ -427,7 +432,7 @@ def qkv_place(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor | No
                                     num_heads, num_kv_heads, value_heads, head_dim, value_dim, page_size, qkv.cols,
                                     _ptr(q_norm), _ptr(k_norm), ctypes.c_float(norm_eps), 1 if values_are_keys else 0,
                                     ctypes.c_float(float(q_temp[0]) if q_temp else 0.0),
-                                    ctypes.c_float(float(q_temp[1]) if q_temp else 0.0), _stream()),
+                                    ctypes.c_float(float(q_temp[1]) if q_temp else 0.0), _ptr(head_scale), _stream()),
            "qkv_place")
     return q_out
 
@@ -701,24 +706,29 @@ def mlstm_scan(fused: Product, q_col: int, k_col: int, v_col: int, gates: torch.
 
 @dataclass
 class ScaledSum:
-    """What a mixer of two branches hands on: first * first_scale + second * second_scale, not added up yet.  A norm
-    that knows it (`layer_norm`) adds both into the residual in its own kernel; anyone else asks for `dense()`."""
+    """What a part of two branches hands on: first * first_scale + second * second_scale, not added up yet; with
+    `row_scale` (float32 [rows, n]) row t of the second is also multiplied by the last number of its row, row_scale[t, n - 1].
+    A norm that knows it (`layer_norm`) adds both into the residual in its own kernel; anyone else asks for `dense()`."""
     first: Product
     first_scale: float
     second: Product
     second_scale: float
+    row_scale: torch.Tensor | None = None
 
     def dense(self, dtype: torch.dtype | None = None) -> torch.Tensor:
-        out = self.first.dense(torch.float32) * self.first_scale + self.second.dense(torch.float32) * self.second_scale
+        second = self.second.dense(torch.float32) * self.second_scale
+        if self.row_scale is not None:
+            second = second * self.row_scale[:, -1:]
+        out = self.first.dense(torch.float32) * self.first_scale + second
         return out if dtype is None else out.to(dtype)
 
 
 def layer_norm(residual: torch.Tensor, delta, weight: torch.Tensor | None, bias: torch.Tensor | None, eps: float,
                out_dtype: torch.dtype, rows: torch.Tensor | None = None, history: torch.Tensor | None = None,
                history_count: int = 0, history_weight: torch.Tensor | None = None, mixed: torch.Tensor | None = None,
-               want_out: bool = True) -> torch.Tensor | None:
+               want_out: bool = True, centred: bool = True) -> torch.Tensor | None:
     """residual += delta (a Product, a ScaledSum or None; all rows, in place), then out = (x - mean) / sqrt(var + eps)
-    * weight + bias of every row, means and variances float.  With `history` (float32 [entries, tokens, hidden] of which
+    * weight + bias of every row, means and variances float (centred False: an RMS norm, x / sqrt(mean(x^2) + eps) * weight).  With `history` (float32 [entries, tokens, hidden] of which
     the first history_count are read, the last of them being `residual` itself) what is normed is the weighted sum
     sum_j history_weight[j] * history[j], which is also written to `mixed`.  With `rows` (int32 indices) only those
     rows are normed and nothing but the result is written.  want_out False: only the sums."""
@@ -728,17 +738,20 @@ def layer_norm(residual: torch.Tensor, delta, weight: torch.Tensor | None, bias:
     tokens, hidden = residual.shape
     if hidden > 16000:
         raise invalid_argument("layer_norm: rows of at most 16000 values")
-    w_code = F32
-    if want_out:
+    w_code = BF16                    # (without a norm: no weight is read; the kernel for both types of products)
+    if not want_out:
+        out_dtype = torch.float32
+    else:
         _device_tensor(weight, "norm weight", (torch.float32, torch.bfloat16))
         w_code = dtype_code(weight.dtype)
         if weight.shape != (hidden,) or (bias is not None and (bias.shape != (hidden,) or bias.dtype != weight.dtype)):
             raise invalid_shape("layer_norm: weight and bias need one entry per column, of one type")
         if not eps > 0.0:
             raise EngineError(ErrorCode.NUMERICAL, "a norm requires a positive epsilon")
-    parts = []
+    parts, row_scale = [], None
     if isinstance(delta, ScaledSum):
         parts = [(delta.first, delta.first_scale), (delta.second, delta.second_scale)]
+        row_scale = delta.row_scale
     elif delta is not None:
         parts = [(as_product(delta), 1.0)]
     for product, _ in parts:
@@ -747,6 +760,11 @@ def layer_norm(residual: torch.Tensor, delta, weight: torch.Tensor | None, bias:
             raise invalid_shape(f"layer_norm: delta [{product.rows}, {product.cols}] does not fit residual {list(residual.shape)}")
     while len(parts) < 2:
         parts.append((None, 0.0))
+    if row_scale is not None:
+        _device_tensor(row_scale, "row_scale", torch.float32)
+        if row_scale.dim() != 2 or row_scale.shape[0] != tokens:
+            raise invalid_shape("layer_norm: the second summand's numbers are [tokens, n], of which the last is read")
+        row_scale = row_scale[:, -1]                      # (a row's numbers lie side by side: the stride is their count)
     if history_count > 0:
         _device_tensor(history, "history", torch.float32)
         _device_tensor(history_weight, "history weight", (torch.float32, torch.bfloat16))
@@ -776,7 +794,8 @@ def layer_norm(residual: torch.Tensor, delta, weight: torch.Tensor | None, bias:
         _ptr(residual), _ptr(d1.data if d1 is not None else None), code(d1), d1.nsplit if d1 is not None else 1,
         ctypes.c_longlong(d1.split_stride if d1 is not None else 0), ctypes.c_float(s1),
         _ptr(d2.data if d2 is not None else None), code(d2), d2.nsplit if d2 is not None else 1,
-        ctypes.c_longlong(d2.split_stride if d2 is not None else 0), ctypes.c_float(s2),
+        ctypes.c_longlong(d2.split_stride if d2 is not None else 0), ctypes.c_float(s2), _ptr(row_scale),
+        row_scale.stride(0) if row_scale is not None else 0, 1 if centred else 0,
         _ptr(history if history_count > 0 else None), ctypes.c_longlong(tokens * hidden), int(history_count),
         _ptr(history_weight if history_count > 0 else None), _ptr(mixed if history_count > 0 and rows is None else None),
         _ptr(weight if want_out else None), _ptr(bias if want_out else None), w_code, ctypes.c_float(eps if want_out else 1.0),
@@ -921,14 +940,17 @@ def decay_scan_state_shape(heads: int, dim: int, value_dim: int) -> tuple[int, .
 def decay_scan(q: tuple[Product, int], k: tuple[Product, int], v: tuple[Product, int], state: torch.Tensor, seq_start: torch.Tensor,
                seq_slot: torch.Tensor, heads: int, dim: int, value_dim: int, decay: torch.Tensor | None = None,
                head_decay: torch.Tensor | None = None, bonus: torch.Tensor | None = None, q_scale: float = 1.0,
-               k_scale: float = 1.0, max_new: int = 1) -> torch.Tensor:
+               k_scale: float = 1.0, max_new: int = 1, activation: str | None = None) -> torch.Tensor:
     """Linear attention with a decaying matrix state over the step's tokens, sequence by sequence (see
     csrc/decay_scan.hip): S' = diag(w) S + k v^T, o = S'^T q per head; with `bonus` (float32 [heads * dim]) the result is
     read before the token joins the state, o = (S + diag(bonus) k v^T)^T q.  q, k, v: (product, first column), of one
     type; the decays w either `head_decay` (float32 [heads], one a head) or `decay` (float32 [tokens, heads * dim], one a
     token and key channel).  Carries `state` (float32 [slots, *decay_scan_state_shape]) for sequences whose slot is not
     negative (or [slots, floats] rows that begin with that shape's floats); returns float32 [tokens, heads * value_dim].  max_new: the most tokens any sequence brings in this step;
-    from SCAN_SLICED_FROM on the tokens are taken in slices of SCAN_SLICE that run side by side."""
+    from SCAN_SLICED_FROM on the tokens are taken in slices of SCAN_SLICE that run side by side.  activation "silu": q, k
+    and v are z * sigmoid(z) of their columns (before the scales)."""
+    if activation not in (None, "silu"):
+        raise invalid_argument(f"decay_scan: unknown activation {activation!r}")
     for name, (product, _) in (("q", q), ("k", k), ("v", v)):
         _check_product(product, name)
     _device_tensor(state, "state", torch.float32)
@@ -981,7 +1003,7 @@ def decay_scan(q: tuple[Product, int], k: tuple[Product, int], v: tuple[Product,
         product, col = pair
         return (_ptr(product.data), product.nsplit, ctypes.c_longlong(product.split_stride), product.cols, int(col))
     _check(library().tlie_decay_scan(*columns(q), *columns(k), *columns(v), code, kind, _ptr(decay), _ptr(head_decay), _ptr(bonus),
-                                     ctypes.c_float(q_scale), ctypes.c_float(k_scale), _ptr(state), _ptr(seq_start),
+                                     1 if activation == "silu" else 0, ctypes.c_float(q_scale), ctypes.c_float(k_scale), _ptr(state), _ptr(seq_start),
                                      _ptr(seq_slot), _ptr(out), sequences, heads, dim, value_dim, slices, _ptr(parts),
                                      ctypes.c_longlong(state.stride(0)), _stream()), "decay_scan")
     return out
@@ -1020,6 +1042,60 @@ def few_outputs(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None
     _check(library().tlie_few_outputs(_ptr(x), dtype_code(x.dtype), _ptr(weight), _ptr(bias), dtype_code(weight.dtype),
                                       _ptr(out), x.shape[0], x.shape[1], outputs, int(top), ROUTER_SCORES[score], int(extra),
                                       _stream()), "few_outputs")
+    return out
+
+
+def grouped_router(x: torch.Tensor, weight: torch.Tensor, correction: torch.Tensor | None, top: int, identities: int = 0,
+                   groups: int = 1, keep: int = 1) -> torch.Tensor:
+    """A router over experts and, after them, `identities` outputs that stand for the identity.  s = softmax(x . weight^T)
+    over all outputs (float sums); the choice goes by s + correction (float32 [outputs]): of `groups` equal groups of
+    neighbours the `keep` with the largest best choice score stay, and of their outputs the `top` largest are picked (the
+    lower index on a tie).  Returns float32 [tokens, experts] (one column more with identities): a picked expert's s divided
+    by the sum of all picked ones' (+ 1e-20), 0 for an expert that is not picked, and last the identities' weights together."""
+    _device_tensor(x, "x", (torch.float32, torch.bfloat16))
+    _device_tensor(weight, "weight", (torch.float32, torch.bfloat16))
+    if x.dim() != 2 or weight.dim() != 2 or x.shape[1] != weight.shape[1]:
+        raise invalid_shape(f"grouped_router: x {list(x.shape)} does not fit weight {list(weight.shape)}")
+    outputs = weight.shape[0]
+    if outputs > 4096:
+        raise invalid_argument("grouped_router: at most 4096 outputs")
+    if correction is not None:
+        _device_tensor(correction, "correction", torch.float32)
+        if correction.shape != (outputs,):
+            raise invalid_shape("grouped_router: the correction needs one entry per output")
+    if not 0 <= identities < outputs or groups <= 0 or outputs % groups != 0 or not 0 < keep <= groups:
+        raise invalid_argument("grouped_router: identities leave experts over, and equal groups divide the outputs")
+    if not 0 < top <= keep * (outputs // groups):
+        raise invalid_argument("grouped_router: a token picks between 1 and all outputs of the groups that stay")
+    scale = torch.empty((x.shape[0], outputs - identities + (1 if identities else 0)), dtype=torch.float32, device=x.device)
+    if x.shape[0] == 0:
+        return scale
+    _check(library().tlie_grouped_router(_ptr(x), dtype_code(x.dtype), _ptr(weight), dtype_code(weight.dtype), _ptr(correction),
+                                         _ptr(scale), x.shape[0], x.shape[1], outputs, int(identities), int(top), int(groups),
+                                         int(keep), _stream()), "grouped_router")
+    return scale
+
+
+def _block_scale(scale: torch.Tensor | None, block: int, rows: int, cols: int) -> tuple[int, int]:
+    """(numbers a row, columns a number serves) of a scale matrix, checked against the columns it goes with."""
+    if scale is None:
+        return 0, 1
+    _device_tensor(scale, "scale", torch.float32)
+    if scale.dim() != 2 or scale.shape[0] != rows or block <= 0 or scale.shape[1] * block < cols:
+        raise invalid_shape("the scale matrix does not fit the columns")
+    return scale.shape[1], int(block)
+
+
+def relu_squared(pre: Product, out_dtype: torch.dtype, scale: torch.Tensor | None = None, block: int = 1) -> torch.Tensor:
+    """out[t, c] = s * max(pre[t, c], 0)^2, s = scale[t, c // block] (float32 [tokens, n]; 0 gives 0 whatever the sum is), or 1."""
+    _check_product(pre, "pre")
+    scale_cols, block = _block_scale(scale, block, pre.rows, pre.cols)
+    out = torch.empty((pre.rows, pre.cols), dtype=out_dtype, device=pre.data.device)
+    if out.numel() == 0:
+        return out
+    _check(library().tlie_relu_squared(_ptr(pre.data), dtype_code(pre.data.dtype), pre.nsplit, ctypes.c_longlong(pre.split_stride),
+                                       _ptr(scale), scale_cols, block, _ptr(out), dtype_code(out_dtype), pre.rows, pre.cols,
+                                       _stream()), "relu_squared")
     return out
 
 
@@ -1070,6 +1146,22 @@ def sigmoid_gate(values: torch.Tensor, pre: Product, col: int) -> torch.Tensor:
     _check(library().tlie_sigmoid_gate(_ptr(values), dtype_code(values.dtype), _ptr(pre.data), dtype_code(pre.data.dtype), pre.nsplit,
                                        ctypes.c_longlong(pre.split_stride), int(col), pre.cols, values.shape[0], values.shape[1],
                                        _stream()), "sigmoid_gate")
+    return values
+
+
+def head_gate(values: torch.Tensor, pre: Product, col: int, heads: int) -> torch.Tensor:
+    """values[t, h * dv + e] *= sigmoid(pre[t, col + h]), in place: one gate a head, whose pre-activations are columns of a
+    wider product; the sigmoid and the product are float."""
+    _device_tensor(values, "values", (torch.float32, torch.bfloat16))
+    _check_product(pre, "pre")
+    if (values.dim() != 2 or heads <= 0 or values.shape[1] % heads != 0 or values.shape[0] != pre.rows or col < 0
+            or col + heads > pre.cols):
+        raise invalid_shape(f"head_gate: {heads} columns from {col} of a product [{pre.rows}, {pre.cols}] do not fit values {list(values.shape)}")
+    if values.shape[0] == 0:
+        return values
+    _check(library().tlie_head_gate(_ptr(values), dtype_code(values.dtype), _ptr(pre.data), dtype_code(pre.data.dtype), pre.nsplit,
+                                    ctypes.c_longlong(pre.split_stride), int(col), pre.cols, values.shape[0], int(heads),
+                                    values.shape[1] // heads, _stream()), "head_gate")
     return values
 
 
@@ -1211,6 +1303,23 @@ def residual_inject(residual: torch.Tensor, tokens: torch.Tensor | None, table: 
         return
     _check(library().tlie_residual_inject(_ptr(residual), _ptr(tokens), _ptr(table), _ptr(vector), code, rows, width,
                                           1 if accumulate else 0, _stream()), "residual_inject")
+
+
+def pass_input(residual: torch.Tensor, tokens: torch.Tensor, table: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """[tokens, 2 * hidden] of out_dtype: the residual's row and the token's row of the embedding's table side by side, as
+    the product that forms a pass's first residual reads them."""
+    _device_tensor(residual, "residual", torch.float32)
+    _device_tensor(tokens, "tokens", torch.int32)
+    _device_tensor(table, "embedding table", (torch.float32, torch.bfloat16))
+    if residual.dim() != 2 or table.dim() != 2 or tokens.shape != (residual.shape[0],) or table.shape[1] != residual.shape[1]:
+        raise invalid_shape("pass_input: residual [T, hidden], tokens [T] and a table [vocab, hidden]")
+    count, hidden = residual.shape
+    out = torch.empty((count, 2 * hidden), dtype=out_dtype, device=residual.device)
+    if count == 0:
+        return out
+    _check(library().tlie_pass_input(_ptr(residual), _ptr(tokens), _ptr(table), dtype_code(table.dtype), _ptr(out),
+                                     dtype_code(out_dtype), count, hidden, _stream()), "pass_input")
+    return out
 
 
 def gemm_generic(x: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor | None, out_dtype: torch.dtype) -> Product:
@@ -1873,14 +1982,16 @@ class RopeTarget:
 
 def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str = "store",
               residual: torch.Tensor | None = None, next_norm: tuple | None = None, waves: int | None = None,
-              rows_per_block: int | None = None, rope: RopeTarget | None = None, gate=None):
+              rows_per_block: int | None = None, rope: RopeTarget | None = None, gate=None, act_scale: torch.Tensor | None = None,
+              act_block: int = 1):
     """y = x . W^T (+ bias) for at most 16 rows.  x: bfloat16 [M, K], or `NormedRows` (then the
     result's rows are scaled as the norm would have scaled the input).
     epilogue "store": float32 [M, N] as a `Product`.  "silu": W's rows alternate gate and up;
     returns bfloat16 silu(gate) * up [M, N / 2] (gate: (name, alpha, limit) of another gate, see `silu_mul`).  "residual": residual [M, N] += y in place, returns
     a `ResidualUpdated`, with the next norm's inputs when next_norm = (weight [N], eps) is given.
     "rope": W is a fused q/k/v weight with rows in the order of `paired_rows`; q and k are rotated,
-    k and v written to the cache (as `rope_cache` does), bfloat16 q [M, nq * d] is returned."""
+    k and v written to the cache (as `rope_cache` does), bfloat16 q [M, nq * d] is returned.
+    "relu2": bfloat16 s * max(y, 0)^2 [M, N] (act_scale, act_block: see `relu_squared`)."""
     scale = x if isinstance(x, NormedRows) else None
     data = scale.xg if scale is not None else x
     _device_tensor(data, "x", torch.bfloat16)
@@ -1915,6 +2026,9 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
         if out_features % 2 != 0:
             raise invalid_shape("gemm_rows: the gated product needs an even number of rows of W")
         act = torch.empty((rows, out_features // 2), dtype=torch.bfloat16, device=device)
+    elif epilogue == "relu2":
+        code = 4
+        act = torch.empty((rows, out_features), dtype=torch.bfloat16, device=device)
     elif epilogue == "residual":
         code = 2
         _device_tensor(residual, "residual", torch.float32)
@@ -1951,6 +2065,7 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
         q_out = torch.empty((rows, rope.num_heads * rope.head_dim), dtype=torch.bfloat16, device=device)
     else:
         raise invalid_argument(f"gemm_rows: unknown epilogue '{epilogue}'")
+    scale_cols, block = _block_scale(act_scale if epilogue == "relu2" else None, act_block, rows, out_features)
     if rope is None or epilogue != "rope":
         rope_args = (_ptr(None), _ptr(None), _ptr(None), 0, 0, 0, 0, 0, _ptr(None), _ptr(None))
     else:
@@ -1959,12 +2074,13 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
     _check(library().tlie_gemm_rows(_ptr(data), _ptr(weight), _ptr(bias), rows, out_features, in_features, _ptr(ssq_in),
                                     strips_in, in_features, ctypes.c_float(eps), code, _ptr(y), _ptr(act), _ptr(residual),
                                     _ptr(next_weight), next_code, _ptr(xg), _ptr(ssq_out), *rope_args, waves, rows_per_block,
-                                    *_gate_args(gate if epilogue == "silu" else None), _stream()), "gemm_rows")
+                                    *_gate_args(gate if epilogue == "silu" else None),
+                                    _ptr(act_scale if epilogue == "relu2" else None), scale_cols, block, _stream()), "gemm_rows")
     if epilogue == "rope":
         return q_out
     if epilogue == "store":
         return Product(y, 1)
-    if epilogue == "silu":
+    if epilogue in ("silu", "relu2"):
         return act
     return ResidualUpdated(NormedRows(xg, ssq_out, float(next_norm[1])) if next_norm is not None else None)
 

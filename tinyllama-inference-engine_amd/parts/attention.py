@@ -40,11 +40,16 @@ class Attention(Mixer):
                          its value head
       qk_norm            "whole": all of a token's query columns together, and all of its key columns together, are
                          RMS-normed (norm_eps) with a weight of that many entries (q_norm, k_norm), before the rotation
-      names              the tensors' names after the prefix, by role (q, k, v, o, q_bias .. o_bias, sink, q_norm, k_norm)
+      head_temp          a learned number per head (temp) that multiplies the head's scaled scores
+      head_gate          a head's result is multiplied by sigmoid(W_g x)_h, one number a head (W_g: head_gate), before the
+                         output projection
+      names              the tensors' names after the prefix, by role (q, k, v, o, q_bias .. o_bias, sink, q_norm, k_norm, temp,
+                         head_gate)
     Tensors: `<prefix>{q,k,v,o}_proj.weight` (and `.bias` when bias) unless `names` says otherwise."""
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
              "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
-             "sink": "sinks", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight"}
+             "sink": "sinks", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "temp": "temperature",
+             "head_gate": "gate.weight"}
 
     def __init__(self, spec: PartSpec, dtype, device):
         super().__init__(spec, dtype, device)
@@ -80,6 +85,9 @@ class Attention(Mixer):
         self.values_are_keys = bool(spec.get("values_are_keys", False))
         self.qk_norm = spec.get("qk_norm")
         self.norm_eps = float(spec.get("norm_eps", 0.0))
+        self.head_temp, self.head_gate = bool(spec.get("head_temp", False)), bool(spec.get("head_gate", False))
+        if self.head_gate and self.bias:
+            raise invalid_config("attention: a gate a head goes with projections without biases")
         if self.softcap is not None and not self.softcap > 0.0:
             raise invalid_config("attention: a cap of the scores must be positive")
         if self.q_temp is not None and (len(self.q_temp) != 2 or not self.q_temp[1] > 0.0):
@@ -90,11 +98,12 @@ class Attention(Mixer):
             raise invalid_config("attention: qk_norm is \"whole\" (with a positive norm_eps, on a layer with keys of its own) or absent")
         # what the kernels that are fused for the plain case (one head size, no sink, no chunks, own keys
         # and values, scores as they are) do not take goes through the kernels for any sizes
-        self.placed = self.q_temp is not None or self.values_are_keys or self.qk_norm is not None   # options of the placement kernel alone
+        self.placed = (self.q_temp is not None or self.values_are_keys or self.qk_norm is not None or self.head_temp
+                       or self.head_gate)                  # options of the placement kernel alone (or columns that it steps over)
         self.general = (self.dv != self.d or self.has_sink or self.chunk is not None or self.reads_other_cache
                         or self.softcap is not None or self.placed)
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
-        self.qkv = self.o = self.sink = self.q_norm = self.k_norm = None
+        self.qkv = self.o = self.sink = self.q_norm = self.k_norm = self.temp = None
 
     @classmethod
     def tensor_specs(cls, spec, prefix):
@@ -115,6 +124,10 @@ class Attention(Mixer):
             specs += [TensorSpec(prefix + names[role + "_bias"], (shape[0],)) for role, shape in shapes]
         if spec.get("sink", False):
             specs.append(TensorSpec(prefix + names["sink"], (nq,)))
+        if spec.get("head_temp", False):
+            specs.append(TensorSpec(prefix + names["temp"], (nq,), init="norm"))
+        if spec.get("head_gate", False):
+            specs.append(TensorSpec(prefix + names["head_gate"], (nq, hidden)))
         return specs
 
     def load(self, weights, prefix):
@@ -129,7 +142,9 @@ class Attention(Mixer):
         roles = ("q",) if self.reads_other_cache else (("q", "k") if self.values_are_keys else ("q", "k", "v"))
 
         def cat(suffix):
-            joined = torch.cat([weights[prefix + names[role + suffix]] for role in roles], dim=0)
+            # (the heads' gates are columns of the same product, after q, k and v)
+            last = ("head_gate",) if self.head_gate and not suffix else ()
+            joined = torch.cat([weights[prefix + names[role + suffix]] for role in (*roles, *last)], dim=0)
             return joined[order].contiguous() if order is not None else joined
         keep = partial(keep_in, weights)
         self.qkv = Linear(cat(""), cat("_bias") if self.bias else None, self.dtype, keep=keep)
@@ -137,6 +152,8 @@ class Attention(Mixer):
                         self.dtype, keep=keep)
         if self.has_sink:
             self.sink = keep(weights[prefix + names["sink"]].float().contiguous())     # (it enters the softmax, which is float)
+        if self.head_temp:                                 # (it enters the scores, which are float)
+            self.temp = keep(weights[prefix + names["temp"]].float().contiguous())
         if self.qk_norm is not None:                       # (norms are float)
             self.q_norm = keep(weights[prefix + names["q_norm"]].float().contiguous())
             self.k_norm = keep(weights[prefix + names["k_norm"]].float().contiguous())
@@ -178,17 +195,18 @@ class Attention(Mixer):
             raise invalid_config("attention: a position encoding that is no rotation table goes with the plain options only")
         inv_freq, rot_dim = table if table is not None else (None, 0)
         writes = binding.writes and not self.reads_other_cache
-        q = None
+        q = fused = None
         if (table is None and self.dv == self.d and self.d % 2 == 0 and not self.reads_other_cache and not self.placed
                 and self.qkv.takes_rows(x.shape[0])):
             # a step of few rows, one head size, own keys and values: the product places q and writes the cache itself
             q = self.qkv(x, rope=ops.RopeTarget(ctx.positions, pages.slot_map if writes else ctx.no_slots, None, 0, binding.cache,
                                                 self.nq, self.nkv, self.d))
         if q is None or isinstance(q, ops.Product):
-            q = ops.qkv_place(ops.as_product(q if q is not None else self.qkv(x)), ctx.positions, pages.slot_map if writes else ctx.no_slots, inv_freq,
+            fused = ops.as_product(q if q is not None else self.qkv(x))
+            q = ops.qkv_place(fused, ctx.positions, pages.slot_map if writes else ctx.no_slots, inv_freq,
                           rot_dim, binding.cache, self.nq, 0 if self.reads_other_cache else self.nkv, self.d, self.dv, self.dtype,
                           q_norm=self.q_norm, k_norm=self.k_norm, norm_eps=self.norm_eps, values_are_keys=self.values_are_keys,
-                          q_temp=self.q_temp)
+                          q_temp=self.q_temp, head_scale=self.temp, extra_cols=self.nq if self.head_gate else 0)
         if self.dv == self.d and ops.attention_mfma_takes(self.dtype, self.d, binding.cache.shape[3] // self.d):
             # bfloat16, one head size: the kernel on the matrix cores (scores, softmax and sink float)
             tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d)
@@ -200,6 +218,8 @@ class Attention(Mixer):
                                              self.d, self.window, self.scale, tiled=ops.attention_generic_plan(ctx, self.d, self.dv),
                                              seq_start=ctx.seq_start, value_dim=self.dv, chunk=self.chunk, sink=self.sink,
                                              softcap=self.softcap)
+        if self.head_gate:
+            attended = ops.head_gate(attended, fused, fused.cols - self.nq, self.nq)
         return self.o(attended)
 
     def forward(self, x, ctx, binding: Binding, into=None):

@@ -20,8 +20,8 @@ from .base import ResidualTarget
 @register("block", "pre_norm")
 class PreNormBlock:
     """x += mixer(norm(x)), then, if the layer has a feed-forward, x += feed_forward(norm(x)).  With
-    `LayerSpec.sublayer_input` a part of the "sublayer_input" table stands between each norm and its sublayer (built
-    once for each); what such parts keep per request is this block's state, one row of it each."""
+    `LayerSpec.sublayer_input` a part of the "sublayer_input" table stands between the norm and the sublayer (built
+    once for each of `LayerSpec.sublayer_input_of`); what such parts keep per request is this block's state, one row of it each."""
 
     def __init__(self, layer: LayerSpec, dtype, device):
         from ..config.spec import PartSpec
@@ -30,35 +30,41 @@ class PreNormBlock:
         self.dtype = dtype
         between = layer.sublayer_input
 
-        def norm(spec):
-            if between is not None:         # what stands behind the norm reads floats
+        def norm(spec, sublayer):
+            before_part = self._has_input(layer, sublayer)
+            if before_part:                 # what stands behind the norm reads floats
                 spec = PartSpec(spec.kind, {**dict(spec.params), "out": "float32"})
             built = lookup("norm", spec.kind)(spec, dtype, device)
-            if between is not None and getattr(built, "out_dtype", None) != torch.float32:
+            if before_part and getattr(built, "out_dtype", None) != torch.float32:
                 raise invalid_config(f"a norm '{spec.kind}' cannot leave floats for what stands between it and its sublayer")
             return built
-        self.mixer_norm = norm(layer.mixer_norm)
+        self.mixer_norm = norm(layer.mixer_norm, "mixer")
         self.mixer = lookup("mixer", layer.mixer.kind)(layer.mixer, dtype, device)
         self.feed_forward_norm = self.feed_forward = self.mixer_input = self.feed_forward_input = None
         if layer.feed_forward is not None:
-            self.feed_forward_norm = norm(layer.feed_forward_norm)
+            self.feed_forward_norm = norm(layer.feed_forward_norm, "feed_forward")
             self.feed_forward = lookup("feed_forward", layer.feed_forward.kind)(layer.feed_forward, dtype, device)
-        if between is not None:
-            self.mixer_input = lookup("sublayer_input", between.kind)(between, dtype, device)
-            if self.feed_forward is not None:
-                self.feed_forward_input = lookup("sublayer_input", between.kind)(between, dtype, device)
+        for sublayer in ("mixer", "feed_forward"):
+            if self._has_input(layer, sublayer):
+                setattr(self, sublayer + "_input", lookup("sublayer_input", between.kind)(between, dtype, device))
         # the route on which norms are folded into products and products add into the residual is for the plain layer
         self.plain = between is None and self.feed_forward is not None
+
+    @staticmethod
+    def _has_input(layer: LayerSpec, sublayer: str) -> bool:
+        """Whether a part stands between the norm and this sublayer ("mixer" or "feed_forward")."""
+        return (layer.sublayer_input is not None and sublayer in layer.sublayer_input_of
+                and getattr(layer, sublayer) is not None)
 
     @classmethod
     def _parts(cls, layer: LayerSpec):
         """(attribute, registry table, the layer's spec of it) of the parts this layer has."""
         parts = [("mixer_norm", "norm", layer.mixer_norm), ("mixer", "mixer", layer.mixer)]
-        if layer.sublayer_input is not None:
+        if cls._has_input(layer, "mixer"):
             parts.append(("mixer_input", "sublayer_input", layer.sublayer_input))
         if layer.feed_forward is not None:
             parts += [("feed_forward_norm", "norm", layer.feed_forward_norm), ("feed_forward", "feed_forward", layer.feed_forward)]
-            if layer.sublayer_input is not None:
+            if cls._has_input(layer, "feed_forward"):
                 parts.append(("feed_forward_input", "sublayer_input", layer.sublayer_input))
         return parts
 
@@ -159,7 +165,7 @@ class PreNormBlock:
         if self.feed_forward is not None:
             normed = self.feed_forward_norm.add_forward(residual, out)
             if self.feed_forward_input is not None:
-                normed = self.feed_forward_input.forward(normed, ctx, binding.block_state[:, 1])
+                normed = self.feed_forward_input.forward(normed, ctx, binding.block_state[:, -1])
             keep("post_attention_norm", normed)
             out = self.feed_forward.forward(normed, ctx)
             if trace is not None:

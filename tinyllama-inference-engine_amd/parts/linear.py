@@ -39,6 +39,13 @@ class Linear:
         ask for the gate, or for the add into the residual)."""
         return ops.gemm_rows_takes(rows, self.weight, self.dtype)
 
+    def relu_squared(self, x, scale: torch.Tensor | None = None, block: int = 1) -> torch.Tensor:
+        """s * max(y, 0)^2 in the activation type, y the product with x: applied by the product's own kernel for a step of few
+        rows, else by the kernel that adds its parts up.  scale, block: see `ops.relu_squared`."""
+        if self.takes_rows(x.shape[0]) and not isinstance(x, ops.NormedRows) and x.dtype == torch.bfloat16:
+            return ops.gemm_rows(x, self.weight, self.bias, "relu2", act_scale=scale, act_block=block)
+        return ops.relu_squared(ops.as_product(self(x)), self.dtype, scale, block)
+
     def __call__(self, x, out_dtype: torch.dtype | None = None, whole: bool = False, into=None, gated: bool = False,
                  rope=None, gate=None):
         """out_dtype: what a dense result is stored in (the skinny kernel's partial sums are float32

@@ -5,7 +5,7 @@ Per token and head, with a query q and a key k (dim values each), a value v (vdi
 There is no softmax and no denominator.  What a request carries from token to token is S of every head: a row of
 floats in the cache manager's state area, zero when the request is admitted.  The projections are the framework's
 products; positions and angles, decays and what they are made of, the state, the scan's sums and the heads' norms are
-float whatever the activation type.  The three mixers differ in where the decay comes from and in what stands around
+float whatever the activation type.  The mixers differ in where the decay comes from and in what stands around
 the scan (`ops.decay_scan`, csrc/decay_scan.hip):
 
     retention                  one fixed decay a head; q and k turned by their positions, k scaled by dim^(-1/2) after
@@ -13,6 +13,8 @@ the scan (`ops.decay_scan`, csrc/decay_scan.hip):
     gated_linear_attention     a decay per token and key channel, sigmoid(z)^(1/tau) with z from a low-rank product with
                                a bias; q scaled by dim^(-1/2); each head's result RMS-normed with a weight the heads
                                share, times silu(gate), output product
+    lightning_attention        one fixed decay a head; q, k and v are silu of their products; the heads' results together
+                               RMS-normed with a weight, times sigmoid(gate), output product
     token_shift_mixing         every projection reads its own blend of a token's input and the input of the token before
                                it (part of the state); a decay per token and key channel, exp(-exp(z)) with z from a
                                low-rank product through tanh plus a vector; the result is read before the token joins
@@ -97,6 +99,60 @@ class Retention(Mixer):
                                  self.heads, self.d, self.dv, head_decay=self.head_decay, max_new=ctx.max_new)
         normed = ops.head_combine(scanned, self.heads, self.dv, self.eps, self.dtype, gate=fused, gate_col=2 * keys + values,
                                   gate_kind="silu")
+        return self.o(normed)
+
+
+@register("mixer", "lightning_attention")
+class LightningAttention(Mixer):
+    """spec: hidden_size, num_heads, head_dim, value_dim, decay (one number a head), norm_eps, names (the tensors' names
+    after the prefix, by role).
+    Tensors: q and k [heads * head_dim, hidden]; v and gate [heads * value_dim, hidden]; norm [heads * value_dim] (the norm
+    is over all heads together); o [hidden, heads * value_dim]."""
+    graph_safe = True
+    NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "gate": "g_proj.weight", "o": "o_proj.weight",
+             "norm": "norm.weight"}
+
+    def __init__(self, spec: PartSpec, dtype, device):
+        super().__init__(spec, dtype, device)
+        self.hidden = int(spec["hidden_size"])
+        self.heads, self.d, self.dv = int(spec["num_heads"]), int(spec["head_dim"]), int(spec["value_dim"])
+        _check_sizes("lightning_attention", self.heads, self.d, self.dv)
+        decay = [float(value) for value in spec["decay"]]
+        if len(decay) != self.heads or not all(0.0 <= value <= 1.0 for value in decay):
+            raise invalid_config("lightning_attention: one decay between 0 and 1 a head")
+        self.head_decay = torch.tensor(decay, dtype=torch.float32, device=device)
+        self.eps = float(spec["norm_eps"])
+        self.names = {**self.NAMES, **dict(spec.get("names") or {})}
+        self.fused = self.o = self.norm = None
+
+    @classmethod
+    def tensor_specs(cls, spec, prefix):
+        names = {**cls.NAMES, **dict(spec.get("names") or {})}
+        hidden, heads, d, dv = int(spec["hidden_size"]), int(spec["num_heads"]), int(spec["head_dim"]), int(spec["value_dim"])
+        shapes = (("q", (heads * d, hidden)), ("k", (heads * d, hidden)), ("v", (heads * dv, hidden)),
+                  ("gate", (heads * dv, hidden)), ("o", (hidden, heads * dv)))
+        specs = [TensorSpec(prefix + names[role], shape) for role, shape in shapes]
+        specs.append(TensorSpec(prefix + names["norm"], (heads * dv,), init="norm"))
+        return specs
+
+    def load(self, weights, prefix):
+        keep = partial(keep_in, weights)
+        get = lambda role: weights[prefix + self.names[role]]        # noqa: E731
+        self.fused = Linear(torch.cat([get("q"), get("k"), get("v"), get("gate")], dim=0).contiguous(), None, self.dtype, keep=keep)
+        self.norm = keep(get("norm").contiguous())
+        self.o = Linear(get("o"), None, self.dtype, keep=keep)
+
+    def state_need(self):
+        return StateNeed(ops.decay_scan_state_shape(self.heads, self.d, self.dv), torch.float32)
+
+    def forward(self, x, ctx, binding: Binding, into=None):
+        fused = ops.as_product(self.fused(x))
+        keys, values = self.heads * self.d, self.heads * self.dv
+        scanned = ops.decay_scan((fused, 0), (fused, keys), (fused, 2 * keys), binding.state, ctx.seq_start, ctx.seq_slot,
+                                 self.heads, self.d, self.dv, head_decay=self.head_decay, max_new=ctx.max_new, activation="silu")
+        # (all heads are one row of the norm)
+        normed = ops.head_combine(scanned, 1, values, self.eps, self.dtype, weight=self.norm, gate=fused,
+                                  gate_col=2 * keys + values, gate_kind="sigmoid")
         return self.o(normed)
 
 

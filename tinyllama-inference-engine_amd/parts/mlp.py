@@ -81,9 +81,9 @@ class GatedMLP(FeedForward):
 @register("feed_forward", "mlp")
 class PlainMLP(FeedForward):
     """down(act(up(x))), no gate.  spec: hidden_size, intermediate_size, activation: "xielu", which has two learned numbers
-    (p, q): for z > 0 softplus(p) z^2 + z / 2, otherwise (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2; names (the tensors'
-    names after the prefix, by role: up, down, act).
-    Tensors: `<prefix>{up,down}_proj.weight`, `<prefix>act` [2] unless `names` says otherwise."""
+    (p, q): for z > 0 softplus(p) z^2 + z / 2, otherwise (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2; or "relu_squared",
+    max(z, 0)^2; names (the tensors' names after the prefix, by role: up, down, act).
+    Tensors: `<prefix>{up,down}_proj.weight`, and for xielu `<prefix>act` [2], unless `names` says otherwise."""
     graph_safe = True
     NAMES = {"up": "up_proj.weight", "down": "down_proj.weight", "act": "act"}
 
@@ -91,7 +91,7 @@ class PlainMLP(FeedForward):
         super().__init__(spec, dtype, device)
         self.hidden, self.inter = int(spec["hidden_size"]), int(spec["intermediate_size"])
         self.activation = spec.get("activation", "xielu")
-        if self.activation != "xielu":
+        if self.activation not in ("xielu", "relu_squared"):
             raise invalid_config(f"mlp: activation '{self.activation}' is not implemented")
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
         self.up = self.down = self.numbers = None
@@ -100,14 +100,19 @@ class PlainMLP(FeedForward):
     def tensor_specs(cls, spec, prefix):
         names = {**cls.NAMES, **dict(spec.get("names") or {})}
         hidden, inter = int(spec["hidden_size"]), int(spec["intermediate_size"])
-        return [TensorSpec(prefix + names["up"], (inter, hidden)), TensorSpec(prefix + names["down"], (hidden, inter)),
-                TensorSpec(prefix + names["act"], (2,), init="offset")]
+        specs = [TensorSpec(prefix + names["up"], (inter, hidden)), TensorSpec(prefix + names["down"], (hidden, inter))]
+        if spec.get("activation", "xielu") == "xielu":
+            specs.append(TensorSpec(prefix + names["act"], (2,), init="offset"))
+        return specs
 
     def load(self, weights, prefix):
         keep = partial(keep_in, weights)
         self.up = Linear(weights[prefix + self.names["up"]], None, self.dtype, keep=keep)
         self.down = Linear(weights[prefix + self.names["down"]], None, self.dtype, keep=keep)
-        self.numbers = keep(weights[prefix + self.names["act"]].contiguous())
+        if self.activation == "xielu":
+            self.numbers = keep(weights[prefix + self.names["act"]].contiguous())
 
     def forward(self, x, ctx, into=None):
+        if self.activation == "relu_squared":
+            return self.down(self.up.relu_squared(x))
         return self.down(ops.xielu(ops.as_product(self.up(x)), self.numbers, self.dtype))

@@ -14,8 +14,10 @@ from .base import Norm, NormedDelta, ResidualUpdated, as_product
 
 @register("norm", "rms_norm")
 class RMSNorm(Norm):
-    """spec: size, eps; optionally offset (the stored weight w lies around zero and acts as 1 + w) and
-    tensor (the tensor's name after the prefix; default "weight").  Tensor: `<prefix><tensor>` [size]."""
+    """spec: size, eps; optionally offset (the stored weight w lies around zero and acts as 1 + w),
+    tensor (the tensor's name after the prefix; default "weight") and out (the type of the result: "float32" for a reader
+    that wants floats; default: the activation type).  Tensor: `<prefix><tensor>` [size].
+    What the residual still lacks it adds in its own kernel, the two summands of an `ops.ScaledSum` too."""
     graph_safe = True
 
     def __init__(self, spec: PartSpec, dtype, device):
@@ -23,6 +25,7 @@ class RMSNorm(Norm):
         self.size = int(spec["size"])
         self.eps = float(spec["eps"])
         self.offset = bool(spec.get("offset", False))
+        self.out_dtype = torch.float32 if spec.get("out") == "float32" else dtype
         self.weight = None
 
     @classmethod
@@ -39,10 +42,11 @@ class RMSNorm(Norm):
             self.weight = keep_in(weights, stored.contiguous())
 
     def forward(self, residual):
-        return ops.add_rmsnorm(residual, None, self.weight, self.eps, self.dtype)
+        return self.add_forward(residual, None)
 
     def lazy_params(self):
-        return self.weight, self.eps
+        # (a reader that wants floats reads no product's input: the norm is then formed by its own kernel)
+        return (self.weight, self.eps) if self.out_dtype == self.dtype else None
 
     def add_forward(self, residual, delta, rows=None, lazy=False):
         if isinstance(delta, ResidualUpdated):
@@ -51,6 +55,10 @@ class RMSNorm(Norm):
             if lazy and rows is None and delta.normed is not None:
                 return delta.normed
             delta = None
+        if self.out_dtype != self.dtype or isinstance(delta, ops.ScaledSum):
+            if isinstance(delta, NormedDelta):
+                return super().add_forward(residual, delta, rows=rows)
+            return ops.layer_norm(residual, delta, self.weight, None, self.eps, self.out_dtype, rows=rows, centred=False)
         if isinstance(delta, NormedDelta):
             if delta.weight.dtype == self.weight.dtype:
                 return ops.norm_add_rmsnorm(residual, delta.product, delta.weight, delta.eps, self.weight, self.eps,

@@ -12,6 +12,12 @@ Other designs of the same shape, as options:
     weigh "output"              out = sum of w_e * expert_e(x): the weight multiplies what the expert gives
     activation "clamped_swish"  g = min(gate, limit), u = clamp(up, -limit, limit), g * sigmoid(alpha g) * (u + 1), with a
                                 limit for the experts and one for the shared expert
+    score "softmax_grouped"     s = softmax(z) over all outputs; the choice goes by s + a correction [outputs], among the
+                                experts of the `keep` of `groups` groups of neighbours whose best such number is largest;
+                                the weights are the chosen s divided by their sum
+    identity                    so many outputs of the router after the experts stand for the identity: their "result" is x
+                                itself, times the weight
+    activation "relu_squared"   experts without a gate, down_e(max(up_e(x), 0)^2)
     shared_gate                 the shared expert's result is multiplied by sigmoid(w_sg . x), one number a token
 
 All experts' gate and up matrices are one matrix, their rows side by side expert by expert (g0 u0 g1 u1 ...), the
@@ -20,7 +26,8 @@ products around a gate kernel that multiplies an expert's columns by the token's
 expert that the token does not use (silu(0) * 0 adds nothing to the second product, exactly).  Since the products
 are linear, s (W x) stands for W (s x); a weight on an expert's result multiplies the columns of the second product's
 input in the result's place; and the shared expert's gate is one more row of the router's matrix, which stands outside
-the choice.
+the choice.  An expert without a gate has its up rows alone in the first matrix.  The identities' weights together
+multiply the row x, which whoever adds the feed-forward's result into the residual adds beside it (`ops.ScaledSum`).
 """
 from __future__ import annotations
 
@@ -39,14 +46,16 @@ from .linear import Linear
 
 @register("feed_forward", "routed_mlp")
 class RoutedMLP(FeedForward):
-    """spec: hidden_size, experts, top, expert_size, shared_size (0: no shared expert), score ("sigmoid" or
-    "softmax_of_chosen"), renormalize (False), weigh ("input" or "output"), router_bias (False), activation ("silu" or
-    "clamped_swish" with alpha, limit, shared_limit), shared_gate (False), names (router, router_bias, expert: a pattern
+    """spec: hidden_size, experts, top, expert_size, shared_size (0: no shared expert), score ("sigmoid",
+    "softmax_of_chosen", or "softmax_grouped" with groups, keep and identity), renormalize (the last score's weights are,
+    the others' are not), weigh ("input" or "output"), router_bias (False), activation ("silu", "clamped_swish" with alpha,
+    limit, shared_limit, or "relu_squared"), shared_gate (False), names (router, router_bias, correction, expert: a pattern
     with {} for the expert's number, shared, shared_gate, gate, up, down).
-    Tensors: router [experts, hidden] (and its bias [experts]); per expert and for the shared one gate, up [size, hidden],
-    down [hidden, size]; the shared expert's gate [1, hidden]."""
+    Tensors: router [experts + identity, hidden] (and its bias [experts], or its correction [experts + identity]); per expert
+    and for the shared one gate (if the activation has one), up [size, hidden], down [hidden, size]; the shared expert's
+    gate [1, hidden]."""
     graph_safe = True
-    NAMES = {"router": "router.weight", "router_bias": "router.bias", "expert": "experts.{}.", "shared": "shared_expert.",
+    NAMES = {"router": "router.weight", "router_bias": "router.bias", "correction": "router.correction", "expert": "experts.{}.", "shared": "shared_expert.",
              "shared_gate": "shared_expert_gate.weight", "gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
 
     def __init__(self, spec: PartSpec, dtype, device):
@@ -54,17 +63,34 @@ class RoutedMLP(FeedForward):
         self.hidden = int(spec["hidden_size"])
         self.experts, self.top = int(spec["experts"]), int(spec["top"])
         self.expert_size, self.shared_size = int(spec["expert_size"]), int(spec.get("shared_size", 0))
-        if min(self.experts, self.top, self.expert_size) <= 0 or self.top > self.experts or self.shared_size < 0:
-            raise invalid_config("routed_mlp: experts, top (at most experts) and expert_size must be positive")
+        if min(self.experts, self.top, self.expert_size) <= 0 or self.top > self.experts + int(spec.get("identity", 0)) or self.shared_size < 0:
+            raise invalid_config("routed_mlp: experts, top (at most all outputs) and expert_size must be positive")
         self.score, self.weigh = spec.get("score", "sigmoid"), spec.get("weigh", "input")
         self.activation = spec.get("activation", "silu")
         self.alpha, self.limit = float(spec.get("alpha", 1.0)), float(spec.get("limit", 0.0))
         self.shared_limit = float(spec.get("shared_limit", self.limit))
         self.router_bias, self.shared_gate = bool(spec.get("router_bias", False)), bool(spec.get("shared_gate", False))
-        if self.score not in ops.ROUTER_SCORES or self.weigh not in ("input", "output") or spec.get("renormalize", False):
-            raise invalid_config("routed_mlp: scores are sigmoids or the softmax over the chosen logits, not renormalized, and weigh "
-                                 "the expert's input or its output")
-        if self.activation not in ops.GATES or (self.weigh == "input" and self.activation != "silu"):
+        self.grouped = self.score == "softmax_grouped"
+        self.identity = int(spec.get("identity", 0))
+        self.groups, self.keep_groups = int(spec.get("groups", 1)), int(spec.get("keep", 1))
+        if ((not self.grouped and self.score not in ops.ROUTER_SCORES) or self.weigh not in ("input", "output")
+                or bool(spec.get("renormalize", False)) != self.grouped):
+            raise invalid_config("routed_mlp: scores are sigmoids, the softmax over the chosen logits (both not renormalized) or the "
+                                 "softmax over all of them with a choice among groups (renormalized), and weigh the expert's input "
+                                 "or its output")
+        if self.identity < 0 or (not self.grouped and (self.identity, self.groups, self.keep_groups) != (0, 1, 1)):
+            raise invalid_config("routed_mlp: identities and groups go with the softmax over all logits")
+        if self.grouped:
+            outputs = self.experts + self.identity
+            if self.groups <= 0 or outputs % self.groups != 0 or not 0 < self.keep_groups <= self.groups:
+                raise invalid_config(f"routed_mlp: {self.groups} equal groups, of which {self.keep_groups} stay, do not divide {outputs} outputs")
+            if self.top > self.keep_groups * (outputs // self.groups):
+                raise invalid_config(f"routed_mlp: a token cannot use {self.top} of the outputs of {self.keep_groups} groups")
+            if self.activation != "relu_squared" or self.shared_size > 0 or spec.get("router_bias", False):
+                raise invalid_config("routed_mlp: a choice among groups goes with experts without gates, no shared expert and no router bias")
+        if self.activation == "relu_squared" and (self.weigh != "output" or self.shared_size > 0):
+            raise invalid_config("routed_mlp: experts without gates take weights on their results, and have no shared one beside them")
+        if (self.activation not in ops.GATES and self.activation != "relu_squared") or (self.weigh == "input" and self.activation != "silu"):
             raise invalid_config("routed_mlp: a score that weighs the expert's input goes with the SiLU gate only")
         if self.activation == "clamped_swish" and not (self.limit > 0.0 and self.shared_limit > 0.0):
             raise invalid_config("routed_mlp: the clamped gate needs positive limits")
@@ -73,7 +99,7 @@ class RoutedMLP(FeedForward):
         if self.score == "softmax_of_chosen" and self.top > 64:
             raise invalid_config("routed_mlp: the softmax over the chosen logits takes at most 64 of them")
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
-        self.router = self.router_b = self.gate_up = self.down = None
+        self.router = self.router_b = self.correction = self.gate_up = self.down = None
 
     @classmethod
     def _prefixes(cls, spec, prefix, names):
@@ -88,14 +114,18 @@ class RoutedMLP(FeedForward):
     def tensor_specs(cls, spec, prefix):
         names = {**cls.NAMES, **dict(spec.get("names") or {})}
         hidden = int(spec["hidden_size"])
-        specs = [TensorSpec(prefix + names["router"], (int(spec["experts"]), hidden))]
+        outputs, gated = int(spec["experts"]) + int(spec.get("identity", 0)), spec.get("activation", "silu") != "relu_squared"
+        specs = [TensorSpec(prefix + names["router"], (outputs, hidden))]
+        if spec.get("score", "sigmoid") == "softmax_grouped":
+            specs.append(TensorSpec(prefix + names["correction"], (outputs,), init="offset"))
         if spec.get("router_bias", False):
             specs.append(TensorSpec(prefix + names["router_bias"], (int(spec["experts"]),), init="spread"))
         if spec.get("shared_gate", False):
             specs.append(TensorSpec(prefix + names["shared_gate"], (1, hidden)))
         for place, size in cls._prefixes(spec, prefix, names):
-            specs += [TensorSpec(place + names["gate"], (size, hidden)), TensorSpec(place + names["up"], (size, hidden)),
-                      TensorSpec(place + names["down"], (hidden, size))]
+            if gated:
+                specs.append(TensorSpec(place + names["gate"], (size, hidden)))
+            specs += [TensorSpec(place + names["up"], (size, hidden)), TensorSpec(place + names["down"], (hidden, size))]
         return specs
 
     def load(self, weights, prefix):
@@ -109,17 +139,36 @@ class RoutedMLP(FeedForward):
                 bias = torch.cat([bias, torch.zeros(1, dtype=bias.dtype, device=bias.device)])
         self.router = keep(router.contiguous())
         self.router_b = keep(bias.contiguous()) if bias is not None else None
+        if self.grouped:                                   # (it enters the router's choice, which is float)
+            self.correction = keep(weights[prefix + names["correction"]].float().contiguous())
         rows, columns = [], []
         for place, size in self._prefixes(self.spec, prefix, names):
-            gate, up = weights[place + names["gate"]], weights[place + names["up"]]
-            rows.append(torch.stack([gate, up], dim=1).reshape(2 * size, self.hidden))
+            up = weights[place + names["up"]]
+            if self.activation == "relu_squared":
+                rows.append(up)
+            else:
+                rows.append(torch.stack([weights[place + names["gate"]], up], dim=1).reshape(2 * size, self.hidden))
             columns.append(weights[place + names["down"]])
         self.gate_up = Linear(torch.cat(rows, dim=0).contiguous(), None, self.dtype, keep=keep)
         self.down = Linear(torch.cat(columns, dim=1).contiguous(), None, self.dtype, keep=keep)
 
     def forward(self, x, ctx, into=None):
+        if self.activation == "relu_squared":
+            return self._forward_ungated(x)
         scale = ops.few_outputs(x, self.router, self.router_b, top=self.top, score=self.score, extra=1 if self.shared_gate else 0)
         hidden = ops.routed_gate(ops.as_product(self.gate_up(x)), scale, self.expert_size, self.dtype, weigh=self.weigh,
                                  shared_scaled=self.shared_gate, gate=self.activation, alpha=self.alpha, limit=self.limit,
                                  shared_limit=self.shared_limit)
         return self.down(hidden)
+
+    def _forward_ungated(self, x):
+        if self.grouped:
+            scale = ops.grouped_router(x, self.router, self.correction, self.top, self.identity, self.groups, self.keep_groups)
+        else:
+            scale = ops.few_outputs(x, self.router, self.router_b, top=self.top, score=self.score)
+        hidden = self.gate_up.relu_squared(x, scale, self.expert_size)
+        out = self.down(hidden)
+        if self.identity == 0:
+            return out
+        # the identities' weights together are the scale matrix's last column: x times it joins beside the experts' sum
+        return ops.ScaledSum(ops.as_product(out), 1.0, ops.as_product(x), 1.0, row_scale=scale)
