@@ -13,6 +13,29 @@ import math
 import torch
 
 F64 = torch.float64
+NOISE = None          # a torch.Generator while `noisy` runs: every product's input and result are then moved by a rounding
+
+
+def product(x, w):
+    """x W^T, W stored [out, in]."""
+    if NOISE is None:
+        return x @ w.T
+    return moved(moved(x) @ w.T)
+
+
+def moved(x):
+    """x, each element moved by as much as rounding to bfloat16 may move it (2^-9 of itself), at random."""
+    return x * (1.0 + 2.0 ** -9 * (2.0 * torch.rand(x.shape, generator=NOISE, dtype=F64) - 1.0))
+
+
+def noisy(seed, run):
+    """run() with every product's input and result moved at random: what 16-bit storage alone does to a result."""
+    global NOISE
+    NOISE = torch.Generator().manual_seed(seed)
+    try:
+        return run()
+    finally:
+        NOISE = None
 
 
 def silu(z):
@@ -66,23 +89,23 @@ def windowed_attention(mixer, w, prefix, h, positions):
     """Grouped softmax attention over a sliding window; a factor of the scores and a gate on the result, one a head."""
     H, G, dim, vdim = mixer["heads"], mixer["kv_heads"], mixer["dim"], mixer["vdim"]
     T = h.shape[0]
-    q = (h @ w[prefix + "q"].T).reshape(T, H, dim)
-    k = (h @ w[prefix + "k"].T).reshape(T, G, dim)
-    v = (h @ w[prefix + "v"].T).reshape(T, G, vdim)
+    q = product(h, w[prefix + "q"]).reshape(T, H, dim)
+    k = product(h, w[prefix + "k"]).reshape(T, G, dim)
+    v = product(h, w[prefix + "v"]).reshape(T, G, vdim)
     rot = mixer.get("rot")
     if rot is not None:
         q = rotate_halves(q, positions, int(rot["dims"]), float(rot["base"]))
         k = rotate_halves(k, positions, int(rot["dims"]), float(rot["base"]))
     size = (mixer.get("mask") or {}).get("size")
     mask = window_mask(T, size)
-    gate = torch.sigmoid(h @ w[prefix + "g"].T)                       # [T, H]
+    gate = torch.sigmoid(product(h, w[prefix + "g"]))                       # [T, H]
     heads = []
     for head in range(H):
         group = head // (H // G)
         scores = q[:, head] @ k[:, group].T * float(mixer["scale"]) * w[prefix + "temp"][head]
         weights = torch.softmax(scores.masked_fill(~mask, -math.inf), dim=-1)
         heads.append(weights @ v[:, group] * gate[:, head:head + 1])
-    return torch.cat(heads, dim=-1) @ w[prefix + "o"].T
+    return product(torch.cat(heads, dim=-1), w[prefix + "o"])
 
 
 def decayed_state_walk(q, k, v, decay, bonus=None):
@@ -108,13 +131,13 @@ def time_mixing(mixer, w, prefix, h, eps):
     H, dim = mixer["heads"], mixer["dim"]
     T = h.shape[0]
     mixed = {name: blend(h, w[prefix + "mu." + name]) for name in "rkvgw"}
-    r, k, v = ((mixed[name] @ w[prefix + name].T).reshape(T, H, dim) for name in "rkv")
-    gate = silu(mixed["g"] @ w[prefix + "g"].T)
-    z = torch.tanh(mixed["w"] @ w[prefix + "w1"].T) @ w[prefix + "w2"].T + w[prefix + "w0"]
+    r, k, v = (product(mixed[name], w[prefix + name]).reshape(T, H, dim) for name in "rkv")
+    gate = silu(product(mixed["g"], w[prefix + "g"]))
+    z = torch.tanh(product(mixed["w"], w[prefix + "w1"])) @ w[prefix + "w2"].T + w[prefix + "w0"]
     decay = torch.exp(-torch.exp(z)).reshape(T, H, dim)
     heads = [unit_rms(decayed_state_walk(r[:, head], k[:, head], v[:, head], decay[:, head], bonus=w[prefix + "u"][head]), eps)
              for head in range(H)]
-    return (torch.cat(heads, dim=-1) * w[prefix + "norm"] * gate) @ w[prefix + "o"].T
+    return product(torch.cat(heads, dim=-1) * w[prefix + "norm"] * gate, w[prefix + "o"])
 
 
 def parallel(mixer, w, prefix, h, positions, eps):
@@ -127,15 +150,15 @@ def parallel(mixer, w, prefix, h, positions, eps):
 def lightning(mixer, w, prefix, h, positions, eps):
     H, dim, vdim = mixer["heads"], mixer["dim"], mixer["vdim"]
     T = h.shape[0]
-    q = silu(h @ w[prefix + "q"].T).reshape(T, H, dim)
-    k = silu(h @ w[prefix + "k"].T).reshape(T, H, dim)
-    v = silu(h @ w[prefix + "v"].T).reshape(T, H, vdim)
+    q = silu(product(h, w[prefix + "q"])).reshape(T, H, dim)
+    k = silu(product(h, w[prefix + "k"])).reshape(T, H, dim)
+    v = silu(product(h, w[prefix + "v"])).reshape(T, H, vdim)
     heads = []
     for head in range(H):
         decay = torch.full((T, dim), float(mixer["decay"][head]), dtype=F64)
         heads.append(decayed_state_walk(q[:, head], k[:, head], v[:, head], decay))
     joined = rms_norm(torch.cat(heads, dim=-1), w[prefix + "norm"], eps)       # all heads together
-    return (joined * torch.sigmoid(h @ w[prefix + "g"].T)) @ w[prefix + "o"].T
+    return product(joined * torch.sigmoid(product(h, w[prefix + "g"])), w[prefix + "o"])
 
 
 MIXERS = {"parallel": parallel, "lightning": lightning}
@@ -147,7 +170,7 @@ def relu_squared(z):
 
 
 def dense(w, prefix, h):
-    return relu_squared(h @ w[prefix + "up"].T) @ w[prefix + "down"].T
+    return product(relu_squared(product(h, w[prefix + "up"])), w[prefix + "down"])
 
 
 def router_choice(z, correction, top, groups=None):
@@ -192,7 +215,7 @@ def mixture(mlp, w, prefix, h, margins=None):
     """margins: a list that takes, per call, every token's `router_margin`."""
     router = mlp["router"]
     experts, top = int(router["experts"]), int(router["top"])
-    z = h @ w[prefix + "router"].T
+    z = product(h, w[prefix + "router"])
     correction = w[prefix + "correction"]
     _, chosen, weights = router_choice(z, correction, top, router.get("groups"))
     if margins is not None:
@@ -233,13 +256,13 @@ def forward(config, weights, tokens, margins=None):
         layer = config["layers"][index]
         prefix = f"l{index}."
         if enters:
-            x = torch.cat([x, first], dim=-1) @ w["loop.in"].T
+            x = product(torch.cat([x, first], dim=-1), w["loop.in"])
         h = blend(rms_norm(x, w[prefix + "norm1"], eps), w[prefix + "shift"])
         x = x + MIXERS[layer["type"]](layer["mixer"], w, prefix + "mix.", h, positions, eps)
         if layer.get("mlp") is not None:
             x = x + feed_forward(layer["mlp"], w, prefix + "mlp.", rms_norm(x, w[prefix + "norm2"], eps), margins)
         residuals.append(x)
-    logits = rms_norm(x, w["final.norm"], eps) @ w["embed"].T
+    logits = product(rms_norm(x, w["final.norm"], eps), w["embed"])
     cap = config.get("logit_softcap")
     if cap is not None:
         logits = float(cap) * torch.tanh(logits / float(cap))
