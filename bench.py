@@ -299,12 +299,48 @@ def narolorn_configs(sizes):
     return narolorn, llama
 
 
+# layer sizes for `--design paluzen`: the same widths and vocabulary; attention with Llama's heads over a window of 1024 beside
+# heads of 64 dims as many as the width has; lightning attention with heads of 128 x 128 over the width; experts without a
+# gate of which four in use have as many weights as Llama's feed-forward (two matrices of 1.5 times its inner size together),
+# 14 of them beside 2 identities in 4 groups of which 3 stay; a dense feed-forward of the same weights; four layers of which
+# the first two run twice (six runs)
+PALUZEN_SIZES = {
+    "w2048": dict(width=2048, ff=8448, llama_ff=5632, vocab=32000, heads=32, kv_heads=4, dim=64, window=1024, shift_heads=32, shift_dim=64,
+                  light_heads=16, light_dim=128, light_vdim=128, experts=14, identity=2, groups=4, keep=3, top=4, expert_ff=2112, rank=16),
+    "w4096": dict(width=4096, ff=21504, llama_ff=14336, vocab=32000, heads=32, kv_heads=8, dim=128, window=1024, shift_heads=64, shift_dim=64,
+                  light_heads=32, light_dim=128, light_vdim=128, experts=14, identity=2, groups=4, keep=3, top=4, expert_ff=5376, rank=16),
+}
+
+
+def paluzen_configs(sizes):
+    """(the Paluzen configuration, the Llama configuration of equal sizes): attention beside token-shift mixing with a dense
+    feed-forward, lightning attention with a routed one, the two mixers again with routed ones; the first two run twice,
+    each pass after its product with the embedding's output.  Beside as many Llama layers as that makes runs."""
+    s = sizes
+    dense = {"kind": "dense", "ff": s["ff"]}
+    routed = {"kind": "moe", "expert": {"ff": s["expert_ff"]},
+              "router": {"experts": s["experts"], "top": s["top"], "identity": s["identity"], "groups": {"count": s["groups"], "keep": s["keep"]}}}
+    side = {"left": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5,
+                     "mask": {"size": s["window"]}, "rot": {"base": 10000.0, "dims": s["dim"] // 2}},
+            "right": {"heads": s["shift_heads"], "dim": s["shift_dim"]}, "left_scale": 1.0, "right_scale": 1.0}
+    light = {"heads": s["light_heads"], "dim": s["light_dim"], "vdim": s["light_vdim"],
+             "decay": [1.0 - 2.0 ** (-5 - 3 * head / max(s["light_heads"] - 1, 1)) for head in range(s["light_heads"])]}
+    layers = [{"type": "parallel", "mixer": side, "mlp": dense}, {"type": "lightning", "mixer": light, "mlp": routed},
+              {"type": "parallel", "mixer": side, "mlp": routed}, {"type": "lightning", "mixer": light, "mlp": routed}]
+    paluzen = {"architecture": "Paluzen", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-5}, "logit_softcap": 30.0,
+               "loop": {"start": 0, "stop": 2, "times": 2}, "layers": layers}
+    llama = dict(TINYLLAMA, hidden_size=s["width"], intermediate_size=s["llama_ff"], num_hidden_layers=6,
+                 num_attention_heads=s["heads"], num_key_value_heads=s["kv_heads"], vocab_size=s["vocab"], max_position_embeddings=4096)
+    return paluzen, llama
+
+
 def bench_design(args, torch) -> int:
-    """`--design fadutar|raketar|tugalix|narolorn`: one JSON line.  Per size: tokens a second of a prompt step of 2048 tokens and of decode steps
+    """`--design fadutar|raketar|tugalix|narolorn|paluzen`: one JSON line.  Per size: tokens a second of a prompt step of 2048 tokens and of decode steps
     at the record's batch and context, for that decoder and for the Llama decoder of equal sizes (random
     weights, bfloat16, through the engine's own loop), and every kernel the design adds alone, beside the like kernel."""
     from tlie_amd import Engine, ops
-    from tlie_amd.kernel_bench import bench_design_kernels, bench_narolorn_kernels, bench_raketar_kernels, bench_tugalix_kernels
+    from tlie_amd.kernel_bench import (bench_design_kernels, bench_narolorn_kernels, bench_paluzen_kernels, bench_raketar_kernels,
+                                       bench_tugalix_kernels)
     peaks = ops.measured_peaks("cuda:0")
     record = {"metric": f"{args.design}: prefill and decode tok/s beside the Llama decoder of equal sizes", "unit": "tokens/s",
               "n_gpus": 1, "dtype": "bf16", "data": "synthetic: uniform random token ids, random weights",
@@ -313,9 +349,10 @@ def bench_design(args, torch) -> int:
     all_sizes, configs, kernels = {"fadutar": (DESIGN_SIZES, design_configs, bench_design_kernels),
                                    "raketar": (RAKETAR_SIZES, raketar_configs, bench_raketar_kernels),
                                    "tugalix": (TUGALIX_SIZES, tugalix_configs, bench_tugalix_kernels),
-                                   "narolorn": (NAROLORN_SIZES, narolorn_configs, bench_narolorn_kernels)}[args.design]
+                                   "narolorn": (NAROLORN_SIZES, narolorn_configs, bench_narolorn_kernels),
+                                   "paluzen": (PALUZEN_SIZES, paluzen_configs, bench_paluzen_kernels)}[args.design]
     for name, sizes in all_sizes.items():
-        entry = {"layers": {"fadutar": 4 * sizes.get("groups", 0), "raketar": 6, "tugalix": 4, "narolorn": 6}[args.design], "sizes": sizes}
+        entry = {"layers": {"fadutar": 4 * sizes.get("groups", 0), "raketar": 6, "tugalix": 4, "narolorn": 6, "paluzen": 6}[args.design], "sizes": sizes}
         for model, config in zip((args.design, "llama"), configs(sizes)):
             engine = Engine(None, dtype="bfloat16", config=config, random_seed=0, max_tokens=args.batch * args.context + 4096,
                             page_size=16, max_requests=args.batch + 1)
@@ -361,7 +398,7 @@ def main() -> int:
                         help="time the kernels of a decode step (--batch, --context) and of a prompt step one by one at the "
                              "shape's layer sizes, each inside a replayed recording that walks through copies of its weights; "
                              "NAME keeps the kernels whose name holds it; prints one JSON line per kernel")
-    parser.add_argument("--design", default=None, choices=["fadutar", "raketar", "tugalix", "narolorn"],
+    parser.add_argument("--design", default=None, choices=["fadutar", "raketar", "tugalix", "narolorn", "paluzen"],
                         help="prefill and decode throughput of that decoder design at layer sizes of real models, beside the Llama "
                              "decoder at equal sizes, and its own kernels alone beside the like kernels (one JSON line of its own)")
     parser.add_argument("--shape", default="tinyllama", choices=["tinyllama", *OTHER_SHAPES],

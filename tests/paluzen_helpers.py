@@ -63,11 +63,11 @@ CONFIG_V = {        # no loop, logits as they are, no windows and no turning key
         {"type": "parallel", "mixer": parallel((2, 1, 40, 40, 0.2), (1, 33), (1.0, 0.4), window=1), "mlp": moe(3, 1, 20, groups=(3, 1))},
     ],
 }
-CONFIG_W = {        # a loop of the first layer alone; head sizes the matrix cores take
+CONFIG_W = {        # a loop of the first layer alone; head sizes the matrix cores take, experts whose products run over pairs of experts and tokens
     "architecture": "Paluzen", "vocab": 96, "width": 128, "norm": {"eps": 1e-5}, "logit_softcap": 25.0,
     "loop": {"start": 0, "stop": 1, "times": 2},
     "layers": [
-        {"type": "parallel", "mixer": parallel((4, 2, 64, 64, 0.13), (4, 32), (1.0, 1.0), window=24, rot=(30000.0, 32)), "mlp": moe(7, 2, 32, groups=(4, 3), identity=1)},
+        {"type": "parallel", "mixer": parallel((4, 2, 64, 64, 0.13), (4, 32), (1.0, 1.0), window=24, rot=(30000.0, 32)), "mlp": moe(7, 2, 64, groups=(4, 3), identity=1)},
         {"type": "lightning", "mixer": lightning(160, 64, [0.999, 0.8]), "mlp": dense(264)},
         {"type": "parallel", "mixer": parallel((2, 2, 48, 48, 0.15), (2, 64), (0.9, 0.3), window=80, rot=(100.0, 48)), "mlp": moe(8, 8, 16, identity=4)},
     ],

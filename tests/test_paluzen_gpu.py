@@ -210,6 +210,96 @@ def test_the_placement_multiplies_every_query_head_by_its_number(heads, groups, 
     assert float((got.cpu().double().reshape(tokens, heads, d) - turned * numbers.double()[None, :, None]).abs().max()) < 1e-3
 
 
+@pytest.mark.parametrize("heads,groups,d,rot,extra", [(4, 2, 16, 8, 8), (3, 1, 32, 32, 5), (6, 3, 64, 0, 0), (2, 2, 48, 16, 3)])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_rotation_and_cache_write_with_a_number_a_head_and_columns_beside(heads, groups, d, rot, extra, dtype):
+    """The kernel for any step, and for few rows the product that does the same itself: against the placement of any sizes,
+    with the weight's rows in paired order."""
+    from tlie_amd import ops
+    activation = torch.float32 if dtype == "float32" else torch.bfloat16
+    generator = torch.Generator().manual_seed(d + extra)
+    tokens, page_size, inner = 6, 16, 128
+    placed = (heads + 2 * groups) * d
+    x, w = torch.randn(tokens, inner, generator=generator).to(activation), (torch.randn(placed + extra, inner, generator=generator) / 11.0).to(activation)
+    numbers = torch.randn(heads, generator=generator).to(DEVICE)
+    positions = torch.tensor([0, 1, 2, 7, 8, 500], dtype=torch.int32, device=DEVICE)
+    slots = torch.tensor([5, 6, 7, 0, 1, -1], dtype=torch.int32, device=DEVICE)
+    inv = (100.0 ** (-2.0 * torch.arange(rot // 2, dtype=F64) / rot)).float().to(DEVICE) if rot else None
+    order = torch.cat([ops.paired_rows(heads, groups, d, rot), torch.arange(placed, placed + extra)]) if rot else torch.arange(placed + extra)
+    caches = [torch.zeros(2, 2, groups, page_size * d, dtype=activation, device=DEVICE) for _ in range(3)]
+    full = (x.double() @ w.double().T).float()
+    want = ops.qkv_place(ops.Product(full.to(DEVICE), 1), positions, slots, inv, rot, caches[0], heads, groups, d, d, activation, extra_cols=extra,
+                         head_scale=numbers)
+    got = ops.rope_cache(ops.Product(full[:, order].to(DEVICE).contiguous(), 1), positions, slots, inv, rot, caches[1], heads, groups, d, activation,
+                         paired=rot > 0, extra_cols=extra, head_scale=numbers)
+    assert float((got.float() - want.float()).abs().max()) <= (2e-6 if dtype == "float32" else 1e-2) * float(want.abs().max())
+    assert float((caches[0].float() - caches[1].float()).abs().max()) <= (2e-6 if dtype == "float32" else 1e-2) * float(caches[0].abs().max())
+    if dtype == "bfloat16":
+        target = ops.RopeTarget(positions, slots, inv, rot, caches[2], heads, groups, d, extra_cols=extra, head_scale=numbers)
+        got = ops.gemm_rows(x.to(DEVICE), w[order].to(DEVICE).contiguous(), None, "rope", rope=target)
+        if extra:
+            got, beside = got
+            assert float((beside.dense().cpu() - full[:, placed:]).abs().max()) < 1e-4
+        assert float((got.float() - want.float()).abs().max()) <= 1e-2 * float(want.abs().max())
+        assert float((caches[0].float() - caches[2].float()).abs().max()) <= 1e-2 * float(caches[0].abs().max())
+
+
+def _scale_matrix(tokens, experts, columns, top, generator, unused=()):
+    scale = torch.zeros(tokens, columns)
+    for t in range(tokens):
+        count = int(torch.randint(0, top + 1, (1,), generator=generator))
+        usable = [e for e in torch.randperm(experts, generator=generator).tolist() if e not in unused][:count]
+        scale[t, usable] = torch.rand(len(usable), generator=generator) + 0.1
+    scale[:, experts:] = 9.0                                                # (columns after the experts' are someone else's)
+    return scale
+
+
+@pytest.mark.parametrize("tokens,experts,columns,top,unused", [(300, 7, 8, 3, (2,)), (1, 3, 3, 1, ()), (1500, 70, 71, 5, (0, 69)), (65, 130, 130, 2, ()),
+                                                               (40, 4, 4, 4, (0, 1, 2, 3)), (2048, 2, 2, 1, (0,))])
+def test_the_plan_of_pairs(tokens, experts, columns, top, unused):
+    from tlie_amd import ops
+    generator = torch.Generator().manual_seed(tokens + experts)
+    scale = _scale_matrix(tokens, experts, columns, top, generator, unused)
+    plan = ops.route_plan(scale.to(DEVICE), experts, top)
+    for e in range(experts):
+        users = scale[:, e].nonzero().flatten()
+        assert int(plan.counts[e]) == len(users)
+        assert torch.equal(plan.lists[e, :len(users)].cpu().long(), users)
+        assert torch.equal(plan.ranks[users.to(DEVICE), e].cpu().long(), torch.arange(len(users)))
+
+
+@pytest.mark.parametrize("tokens,experts,columns,top,width,size,unused", [
+    (300, 7, 8, 3, 128, 64, (2,)), (1, 3, 4, 1, 64, 192, ()), (700, 5, 5, 2, 192, 128, (0, 4)), (150, 70, 70, 4, 64, 64, (3,)), (500, 2, 3, 1, 320, 64, ()),
+    (20, 4, 4, 4, 64, 64, (0, 1, 2, 3))])
+def test_products_over_the_pairs_of_experts_and_tokens(tokens, experts, columns, top, width, size, unused):
+    """Experts that no token uses, that few and that many use (more and less than a tile, no multiple of one), tokens that
+    use none, against each expert alone; the pairs of one token alone give the same bits as among all."""
+    from tlie_amd import ops
+    generator = torch.Generator().manual_seed(tokens)
+    scale = _scale_matrix(tokens, experts, columns, top, generator, unused)
+    x = torch.randn(tokens, width, generator=generator).bfloat16()
+    up = (torch.randn(experts * size, width, generator=generator) / math.sqrt(width)).bfloat16()
+    down = (torch.randn(width, experts * size, generator=generator) / math.sqrt(size)).bfloat16()
+    assert ops.routed_tiles_take(up, down, experts)
+
+    def run(rows):
+        plan = ops.route_plan(scale[rows].to(DEVICE).contiguous(), experts, top)
+        hidden = ops.routed_relu_squared(x[rows].to(DEVICE).contiguous(), up.to(DEVICE), plan)
+        return hidden, ops.routed_sum(ops.routed_down(hidden, down.to(DEVICE), plan), plan)
+    hidden, got = run(list(range(tokens)))
+    want, at = torch.zeros(tokens, width, dtype=F64), 0
+    for e in range(experts):
+        users = scale[:, e].nonzero().flatten()
+        act = plain.relu_squared(x[users].double() @ up[e * size:(e + 1) * size].double().T) * scale[users, e:e + 1].double()
+        if len(users):
+            assert float((hidden[at:at + len(users)].cpu().double() - act).abs().max()) < 1e-2 * float(act.abs().max())
+            want[users] += hidden[at:at + len(users)].cpu().double() @ down[:, e * size:(e + 1) * size].double().T
+        at += len(users)
+    assert float((got.cpu().double() - want).abs().max()) <= 1e-2 * max(float(want.abs().max()), 1e-30)
+    for t in {0, tokens // 2, tokens - 1}:
+        assert torch.equal(run([t])[1][0], got[t])
+
+
 @pytest.mark.parametrize("heads,dv,col,nsplit,dtype", [(4, 24, 7, 1, torch.float32), (3, 5, 0, 2, torch.float32), (8, 64, 16, 1, torch.bfloat16),
                                                        (2, 256, 3, 3, torch.bfloat16)])
 def test_a_gate_a_head(heads, dv, col, nsplit, dtype):
@@ -410,11 +500,12 @@ def test_lightning_attention_alone(tmp_path, mixer, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("mlp", [dense(40), dense(264), moe(6, 3, 16, groups=(4, 2), identity=2), moe(5, 1, 13, identity=1), moe(4, 4, 24)])
-def test_feed_forwards_alone(tmp_path, mlp, dtype):
+@pytest.mark.parametrize("mlp,width", [(dense(40), 48), (dense(264), 48), (moe(6, 3, 16, groups=(4, 2), identity=2), 48), (moe(5, 1, 13, identity=1), 48),
+                                       (moe(4, 4, 24), 48), (moe(9, 3, 64, groups=(4, 3), identity=3), 64), (moe(4, 2, 128), 128)])
+def test_feed_forwards_alone(tmp_path, mlp, width, dtype):
     """A layer's second sublayer from its input, and what the mixer reads: the shift's result does not depend on the cut."""
     layer = {"type": "lightning", "mixer": lightning(8, 8, [0.9, 0.5]), "mlp": mlp}
-    folder, config, weights = _single_layer(tmp_path, layer, seed=15)
+    folder, config, weights = _single_layer(tmp_path, layer, seed=15, width=width)
     tokens = tokens_of(16, 100, 97)
     first = None
     for cuts in ([100], [2], [1], [9, 1, 30]):

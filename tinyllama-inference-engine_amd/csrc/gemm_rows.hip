@@ -61,17 +61,20 @@ struct RowsArgs {
   float inv_width, eps;       // 1 / width of the normed input
   float gate_alpha;
   // outputs
-  float* y;                   // store: [M, N]
+  float* y;                   // store: [M, N]; rotation: [M, N - (nq + 2 nkv) * d], the columns after q, k and v
   uint16_t* act;              // SiLU: [M, N / 2]; squared ReLU: [M, N]
   float* residual;            // residual: [M, N], updated in place
-  const uint16_t* next_weight;  // residual: [N] bfloat16 weight of the next norm, or null
+  union {
+    const uint16_t* next_weight;  // residual: [N] bfloat16 weight of the next norm, or null
+    const float* head_scale;    // rotation: [nq], query head h is multiplied by head_scale[h], or null
+  };
   union {
     const float* next_weight_f32; // the same when that weight is kept in float32
     const float* act_scale;     // squared ReLU: [M, act_scale_cols], a number for every act_block columns, or null
   };
   uint16_t* xg;               // residual: [M, N] bfloat16(residual * next weight), or null
   float* ssq_out;             // residual: [ceil(N / rows_per_block), 16], or null
-  // rotation and cache write: N = (nq + 2 nkv) * d, heads in the order q | k | v
+  // rotation and cache write: the first (nq + 2 nkv) * d of the N rows of W, heads in the order q | k | v
   const int* positions;       // [M]
   const int* slot_map;        // [M] cache row of each token (page * page_size + row), or -1
   const float* inv_freq;      // [rot_dim / 2], or null: no rotation
@@ -215,6 +218,7 @@ gemm_rows_kernel(const RowsArgs a) {
         const int head = n / a.d, p = n % a.d;
         if (a.inv_freq != nullptr && head < a.nq + a.nkv && p < a.rot_dim)
           sincosf(static_cast<float>(a.positions[token]) * a.inv_freq[p >> 1], &pre_sine[st][turn], &pre_cosine[st][turn]);
+        pre_g[st][turn] = a.head_scale != nullptr && head < a.nq ? a.head_scale[head] : 1.f;
         if (head >= a.nq) pre_slot[st][turn] = a.slot_map[token];
       }
     }
@@ -293,7 +297,10 @@ gemm_rows_kernel(const RowsArgs a) {
           a.act[static_cast<size_t>(token) * a.N + n] = __bfloat16_as_ushort(__float2bfloat16(weight != 0.f ? weight * positive * positive : 0.f));
       } else if (EPILOGUE == kEpilogueRope) {
         const float other = __shfl_xor(value, 1, 64);        // the pair's other element, when this one is rotated
-        if (live) {
+        const int placed = (a.nq + 2 * a.nkv) * a.d;         // columns of q, k and v; those after them are stored as they are
+        if (live && n >= placed) {
+          a.y[static_cast<size_t>(token) * (a.N - placed) + n - placed] = value;
+        } else if (live) {
           const int head = n / a.d, p = n % a.d;
           float result = value;
           int e = p;
@@ -308,7 +315,7 @@ gemm_rows_kernel(const RowsArgs a) {
               result = value * cosine - other * sine;        // first' = first cos - second sin
             }
           }
-          const uint16_t bits = __bfloat16_as_ushort(__float2bfloat16(result));
+          const uint16_t bits = __bfloat16_as_ushort(__float2bfloat16(a.head_scale != nullptr ? result * pre_g[st][turn] : result));
           if (head < a.nq) {
             a.q_out[(static_cast<size_t>(token) * a.nq + head) * a.d + e] = bits;
           } else {
@@ -409,14 +416,14 @@ using namespace tlie;
 // strip of 16 is idle), or 32 (two strips, with at most 8 waves).
 // 3: the rotation and cache write of rope_cache.hip on W's rows in paired order (see above): positions, slot_map [M],
 // inv_freq [rot_dim / 2] or null, q_out bfloat16 [M, nq * d], cache bfloat16 [pages, 2, nkv, page_size * d];
-// N = (nq + 2 nkv) * d.
+// N >= (nq + 2 nkv) * d, the rows of W after those give y float [M, N - (nq + 2 nkv) * d]; head_scale float [nq] or null.
 extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, int M, int N, int K, const float* ssq_in,
                               int strips_in, int width, float eps, int epilogue, float* y, void* act, float* residual,
                               const void* next_weight, int next_weight_dtype, void* xg, float* ssq_out,
                               const int* positions, const int* slot_map, const float* inv_freq, int rot_dim, int nq,
                               int nkv, int d, int page_size, void* q_out, void* cache, int waves, int rows_per_block,
                               int gate_kind, float gate_alpha, float gate_limit, const float* act_scale, int act_scale_cols,
-                              int act_block, void* stream) {
+                              int act_block, const float* head_scale, void* stream) {
   if (gate_kind != kGateSilu && gate_kind != kGateClampedSwish) return kBadArgument;
   if (M <= 0 || M > 16 || N <= 0 || K <= 0 || (K & 7) != 0 || (waves != 2 && waves != 4 && waves != 8 && waves != 16)) return kBadArgument;
   if (!(rows_per_block >= 2 && rows_per_block <= 16 && rows_per_block % 2 == 0) && !(rows_per_block == 32 && waves <= 8)) return kBadArgument;
@@ -429,7 +436,7 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
   if (epilogue == kEpilogueResidual && (residual == nullptr || (xg != nullptr && next_weight == nullptr))) return kBadArgument;
   if (epilogue == kEpilogueRope &&
       (positions == nullptr || slot_map == nullptr || q_out == nullptr || cache == nullptr || nq <= 0 || nkv <= 0 || d <= 0 ||
-       page_size <= 0 || N != (nq + 2 * nkv) * d || rot_dim < 0 || rot_dim > d || (rot_dim & 1) != 0 || (d & 1) != 0))
+       page_size <= 0 || N < (nq + 2 * nkv) * d || (N > (nq + 2 * nkv) * d && y == nullptr) || rot_dim < 0 || rot_dim > d || (rot_dim & 1) != 0 || (d & 1) != 0))
     return kBadArgument;
   RowsArgs a;
   a.x = (const uint16_t*)x, a.w = (const uint16_t*)w, a.bias = (const uint16_t*)bias;
@@ -441,6 +448,7 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
   a.next_weight_f32 = next_weight_dtype == kBF16 ? nullptr : (const float*)next_weight;
   a.xg = (uint16_t*)xg, a.ssq_out = ssq_out;
   if (epilogue == kEpilogueRelu2) a.act_scale = act_scale;
+  if (epilogue == kEpilogueRope) a.head_scale = head_scale;
   a.positions = positions, a.slot_map = slot_map, a.inv_freq = inv_freq, a.rot_dim = rot_dim;
   a.gate_kind = gate_kind, a.gate_alpha = gate_alpha, a.gate_limit = gate_limit;
   a.nq = nq, a.nkv = nkv, a.d = d, a.page_size = page_size, a.q_out = (uint16_t*)q_out, a.cache = (uint16_t*)cache;

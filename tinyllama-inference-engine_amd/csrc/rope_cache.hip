@@ -21,19 +21,21 @@ namespace tlie {
 // (no rotation at all).  paired: within a q or k head the input's columns are stored with the two
 // elements of a rotation pair side by side (element i at 2i, element i + rot_dim/2 at 2i + 1), as
 // the product of few rows wants its weight's rows; outputs are in natural order either way.
+// row_width: columns of a row of the product, of which q, k and v are the first.  head_scale (or null): float [nq], query head
+// h is multiplied by head_scale[h].
 // blockDim.x = heads_per_block * d; grid = (tokens, ceil(heads / heads_per_block)).
 template <typename D, typename A>
 __global__ void rope_cache_kernel(const D* __restrict__ qkv, int nsplit, size_t split_stride,
                                   const int* __restrict__ positions, const int* __restrict__ slot_map,
                                   const float* __restrict__ inv_freq, int rot_dim, A* __restrict__ q_out,
-                                  A* __restrict__ cache, int nq, int nkv, int d, int page_size, int paired) {
+                                  A* __restrict__ cache, int nq, int nkv, int d, int page_size, int paired, int row_width,
+                                  const float* __restrict__ head_scale) {
   extern __shared__ float lds[];
   float* cosines = lds;                  // rot_dim / 2
   float* sines = cosines + rot_dim / 2;  // rot_dim / 2
   float* values = sines + rot_dim / 2;   // blockDim.x
   const int t = blockIdx.x;
   const int heads = nq + 2 * nkv;
-  const int width = heads * d;
   const int half = rot_dim / 2;
   if (inv_freq != nullptr) {
     const float pos = static_cast<float>(positions[t]);
@@ -45,7 +47,8 @@ __global__ void rope_cache_kernel(const D* __restrict__ qkv, int nsplit, size_t 
   float mine = 0.f;
   int column = e;
   if (paired && head < nq + nkv && e < rot_dim) column = e < half ? 2 * e : 2 * (e - half) + 1;
-  if (live) mine = sum_splits(qkv + static_cast<size_t>(t) * width + head * d + column, nsplit, split_stride);
+  if (live) mine = sum_splits(qkv + static_cast<size_t>(t) * row_width + head * d + column, nsplit, split_stride);
+  if (head_scale != nullptr && head < nq) mine *= head_scale[head];
   values[threadIdx.x] = mine;
   __syncthreads();
   if (!live) return;
@@ -81,7 +84,7 @@ template <typename D, typename A>
 __global__ void rope_cache_wide_kernel(const D* __restrict__ qkv, const int* __restrict__ positions,
                                        const int* __restrict__ slot_map, const float* __restrict__ inv_freq,
                                        int rot_dim, A* __restrict__ q_out, A* __restrict__ cache, int nq, int nkv,
-                                       int d, int page_size) {
+                                       int d, int page_size, int row_width, const float* __restrict__ head_scale) {
   extern __shared__ float lds[];
   const int half = rot_dim / 2;
   float* cosines = lds;                  // half
@@ -94,7 +97,7 @@ __global__ void rope_cache_wide_kernel(const D* __restrict__ qkv, const int* __r
   float first_v[8];
   const bool first_live = static_cast<int>(threadIdx.x) < heads * per_head;
   if (first_live)
-    load8(qkv + (static_cast<size_t>(t) * heads + threadIdx.x / per_head) * d + (threadIdx.x % per_head) * 8, first_v);
+    load8(qkv + static_cast<size_t>(t) * row_width + threadIdx.x * 8, first_v);
   if (inv_freq != nullptr) {
     const float pos = static_cast<float>(positions[t]);
     for (int i = threadIdx.x; i < half; i += blockDim.x) sincosf(pos * inv_freq[i], &sines[i], &cosines[i]);
@@ -111,7 +114,12 @@ __global__ void rope_cache_wide_kernel(const D* __restrict__ qkv, const int* __r
 #pragma unroll
       for (int j = 0; j < 8; ++j) v[j] = first_v[j];
     } else {
-      load8(qkv + (static_cast<size_t>(t) * heads + head) * d + c, v);
+      load8(qkv + static_cast<size_t>(t) * row_width + g * 8, v);
+    }
+    if (head_scale != nullptr && head < nq) {
+      const float scale = head_scale[head];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) v[j] *= scale;
     }
     if (head >= nq + nkv) {
       // a value head: after the nkv key heads of the page, transposed
@@ -284,21 +292,23 @@ extern "C" int tlie_qkv_place(const void* qkv, int in_dtype, int nsplit, long lo
 extern "C" int tlie_rope_cache(const void* qkv, int in_dtype, int nsplit, long long split_stride,
                                const int* positions, const int* slot_map, const float* inv_freq, int rot_dim,
                                void* q_out, void* cache, int act_dtype, int tokens, int nq, int nkv, int d,
-                               int page_size, int paired, void* stream) {
+                               int page_size, int paired, int row_width, const float* head_scale, void* stream) {
+  if (row_width < (nq + 2 * nkv) * d) return kBadArgument;
   if (tokens <= 0 || nq <= 0 || nkv <= 0 || d <= 0 || d > 1024 || page_size <= 0 || nsplit < 1) return kBadArgument;
   if (rot_dim < 0 || rot_dim > d || rot_dim % 2 != 0) return kBadArgument;
   const int heads = nq + 2 * nkv;
   hipStream_t s = (hipStream_t)stream;
   const bool aligned = ((reinterpret_cast<uintptr_t>(qkv) | reinterpret_cast<uintptr_t>(q_out) |
                          reinterpret_cast<uintptr_t>(cache)) & 31) == 0;
-  if (nsplit == 1 && (d & 7) == 0 && aligned && (inv_freq == nullptr || (paired && (rot_dim & 7) == 0))) {
+  if (nsplit == 1 && (d & 7) == 0 && (row_width & 7) == 0 && aligned && (inv_freq == nullptr || (paired && (rot_dim & 7) == 0))) {
     const int groups = heads * d / 8;
     const int wide = groups >= 1024 ? 1024 : (groups + 63) / 64 * 64;
     const size_t wide_lds = static_cast<size_t>(rot_dim) * sizeof(float);
 #define TLIE_WIDE(DC, D, AC, A)                                                                              \
   if (in_dtype == DC && act_dtype == AC) {                                                                   \
     hipLaunchKernelGGL((rope_cache_wide_kernel<D, A>), dim3(tokens), dim3(wide), wide_lds, s, (const D*)qkv,   \
-                       positions, slot_map, inv_freq, rot_dim, (A*)q_out, (A*)cache, nq, nkv, d, page_size);  \
+                       positions, slot_map, inv_freq, rot_dim, (A*)q_out, (A*)cache, nq, nkv, d, page_size,   \
+                       row_width, head_scale);                                                               \
     return launch_status();                                                                                  \
   }
     TLIE_WIDE(kF32, float, kF32, float)
@@ -318,7 +328,7 @@ extern "C" int tlie_rope_cache(const void* qkv, int in_dtype, int nsplit, long l
   if (in_dtype == DC && act_dtype == AC) {                                                                   \
     hipLaunchKernelGGL((rope_cache_kernel<D, A>), grid, dim3(threads), lds, s, (const D*)qkv, nsplit,         \
                        (size_t)split_stride, positions, slot_map, inv_freq, rot_dim, (A*)q_out, (A*)cache, nq, \
-                       nkv, d, page_size, paired);                                                           \
+                       nkv, d, page_size, paired, row_width, head_scale);                                    \
     return launch_status();                                                                                  \
   }
   TLIE_CASE(kF32, float, kF32, float)

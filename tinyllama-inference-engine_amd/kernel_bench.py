@@ -746,3 +746,185 @@ def bench_tugalix_kernels(sizes: dict, batch: int = 8, context: int = 2048, prom
         times = _timed(lambda i: ops.silu_mul(dense_up, bf, interleaved=True), 4, samples)
         row(f"{label}: SiLU gate (Llama's)", times, tokens * lff * 6)
     return rows
+
+
+def bench_paluzen_kernels(sizes: dict, batch: int = 8, context: int = 2048, prompt: int = 2048, samples: int = 10, device="cuda:0",
+                          hbm_gbs: float = 8000.0, mfma_tflops: float = 2500.0) -> list[dict]:
+    """The kernels that the Paluzen decoder adds or runs in a new form, each alone at a layer's sizes, for a decode step of
+    `batch` requests at `context` positions and a prompt step of `prompt` tokens, each beside the like kernel of the closest
+    model (retention's scan, Llama's attention, rotation, add + norm, gate and dense products); every row carries the
+    fraction of the roofline its bytes or flops reach (`frac`: of `hbm_gbs` for rows with bytes, of `mfma_tflops` for rows
+    with flops).
+    sizes: width, ff, llama_ff, heads, kv_heads, dim, window (the attention side); shift_heads, shift_dim, rank (the side
+    beside it); light_heads, light_dim, light_vdim; experts, identity, groups, keep, top, expert_ff; vocab."""
+    device = torch.device(device)
+    torch.cuda.set_device(device)
+    bf, f32 = torch.bfloat16, torch.float32
+    width, ff, lff, vocab = sizes["width"], sizes["ff"], sizes["llama_ff"], sizes["vocab"]
+    H, G, d, window = sizes["heads"], sizes["kv_heads"], sizes["dim"], sizes["window"]
+    experts, identity, top, eff = sizes["experts"], sizes["identity"], sizes["top"], sizes["expert_ff"]
+    page_size, rows = 16, []
+
+    def rand(*shape, scale=0.02, dtype=bf):
+        return (torch.randn(shape, device=device, dtype=f32) * scale).to(dtype)
+
+    def row(name, times, read_bytes=0, flops=0):
+        entry = _row(name, times, read_bytes, flops)
+        if read_bytes:
+            entry["frac"] = round(entry["gbs"] / hbm_gbs, 3)
+        elif flops:
+            entry["frac"] = round(entry["tflops"] / mfma_tflops, 4)
+        rows.append(entry)
+
+    def ints(values):
+        return torch.tensor(values, dtype=torch.int32, device=device)
+
+    for label, tokens, seqs, keys in ((f"decode b{batch}", batch, batch, context), (f"prompt {prompt}", prompt, 1, prompt)):
+        if tokens <= 0:
+            continue
+        decode = seqs == tokens
+        blocks = (keys + page_size - 1) // page_size
+        pages = seqs * blocks
+        table = torch.arange(pages, dtype=torch.int32, device=device).view(seqs, blocks).contiguous()
+        if decode:
+            positions = torch.full((tokens,), keys - 1, dtype=torch.int32, device=device)
+            token_seq, seq_start = ints(list(range(tokens))), ints(list(range(tokens + 1)))
+            slot_map = (table[:, -1] * page_size + (keys - 1) % page_size).to(torch.int32).contiguous()
+            host = {}
+        else:
+            positions = torch.arange(tokens, dtype=torch.int32, device=device)
+            token_seq, seq_start = torch.zeros(tokens, dtype=torch.int32, device=device), ints([0, tokens])
+            slot_map = positions.clone()
+            host = {"seq_start": np.asarray([0, tokens], dtype=np.int32), "seq_len": np.asarray([keys], dtype=np.int32)}
+        seq_slot = ints(list(range(seqs)))
+        ctx = SimpleNamespace(max_new=1 if decode else tokens, num_seqs=seqs, num_tokens=tokens, max_context=keys, scratch={}, tile_owner=None,
+                              compute_units=int(torch.cuda.get_device_properties(device).multi_processor_count), host=host, tokens=positions,
+                              token_seq=token_seq, token_slot=seq_slot[token_seq.long()].contiguous(), seq_start=seq_start, seq_slot=seq_slot)
+        # ---- attention over a window (flops: the keys a token sees) ---------------------------------------------------
+        cache = rand(pages, 2, G, page_size * d, scale=0.5)
+        q = rand(tokens, H * d, scale=1.0)
+        plan = ops.attention_plan(ctx, H // G, G, d)
+        tiles, col_tiles, nsplit, split_len, waves, shared = plan
+        for name, reach in (("causal (Llama's)", None), (f"window of {window}", window)):
+            times = _timed(lambda i: ops.attention_mfma(q, cache, table, tiles, positions, H, G, d, reach, d ** -0.5, nsplit, split_len, col_tiles,
+                                                        waves, shared), 8, samples)
+            seen = min(keys, reach or keys)
+            flops = 4.0 * H * d * sum(min(p + 1, seen) for p in range(tokens)) if not decode else 0
+            row(f"{label}: attention, {name}, {H} heads of {d} on {G}", times, seqs * seen * 2 * G * d * 2 if decode else 0, flops)
+        qkv = ops.Product(rand(tokens, (H + 2 * G) * d, scale=1.0), 1)
+        inv_freq = torch.ones(d // 2, device=device)
+        times = _timed(lambda i: ops.rope_cache(qkv, positions, slot_map, inv_freq, d, cache, H, G, d, bf, paired=True), 8, samples)
+        row(f"{label}: rotation + cache write (Llama's)", times, tokens * (H * 2 + 2 * G) * d * 2 * 2)
+        gated = ops.Product(rand(tokens, (H + 2 * G) * d + H, scale=1.0), 1)       # (H is a multiple of 8: no column between)
+        temp, part_freq = rand(H, scale=1.0, dtype=f32), torch.ones(d // 4, device=device)
+        times = _timed(lambda i: ops.rope_cache(gated, positions, slot_map, part_freq, d // 2, cache, H, G, d, bf, paired=True, extra_cols=H,
+                                                head_scale=temp), 8, samples)
+        row(f"{label}: rotation + cache write with a number a head, gates' columns beside", times, tokens * (H * 2 + 2 * G) * d * 2 * 2)
+        values = rand(tokens, H * d, scale=1.0)
+        times = _timed(lambda i: ops.head_gate(values, gated, (H + 2 * G) * d, H), 8, samples)
+        row(f"{label}: a gate a head on the heads' results", times, tokens * H * d * 4)
+        # ---- the scans: a token costs 4 flops an element of S -----------------------------------------------------------
+        lh, ld, lv = sizes["light_heads"], sizes["light_dim"], sizes["light_vdim"]
+        fused = ops.Product(rand(tokens, 2 * lh * ld + 2 * lh * lv, scale=1.0), 1)
+        state = torch.zeros((seqs, *ops.decay_scan_state_shape(lh, ld, lv)), dtype=f32, device=device)
+        decay = torch.full((lh,), 0.97, dtype=f32, device=device)
+        for name, activation in (("retention's at these sizes", None), ("lightning, silu on the way in", "silu")):
+            times = _timed(lambda i: ops.decay_scan((fused, 0), (fused, lh * ld), (fused, 2 * lh * ld), state, seq_start, seq_slot, lh, ld, lv,
+                                                    head_decay=decay, max_new=ctx.max_new, activation=activation), 8, samples)
+            row(f"{label}: scan ({name}), {lh} heads of {ld} x {lv}", times, seqs * lh * ld * lv * 8 if decode else 0,
+                0 if decode else 4.0 * tokens * lh * ld * lv)
+        scanned, weight = rand(tokens, lh * lv, scale=1.0, dtype=f32), rand(lh * lv, scale=1.0)
+        times = _timed(lambda i: ops.head_combine(scanned, lh, lv, 1e-5, bf, weight=weight, gate=fused, gate_col=2 * lh * ld + lh * lv), 8, samples)
+        row(f"{label}: norm and gate, head by head (retention's)", times, tokens * lh * lv * (4 + 2 + 2))
+        times = _timed(lambda i: ops.head_combine(scanned, 1, lh * lv, 1e-5, bf, weight=weight, gate=fused, gate_col=2 * lh * ld + lh * lv), 8, samples)
+        row(f"{label}: norm and gate over all heads together", times, tokens * lh * lv * (4 + 2 + 2))
+        sh, sd = sizes["shift_heads"], sizes["shift_dim"]
+        shifted = ops.Product(rand(tokens, 3 * sh * sd, scale=1.0), 1)
+        shift_state = torch.zeros((seqs, *ops.decay_scan_state_shape(sh, sd, sd)), dtype=f32, device=device)
+        decays, bonus = torch.rand(tokens, sh * sd, device=device) * 0.1 + 0.9, rand(sh * sd, scale=1.0, dtype=f32)
+        times = _timed(lambda i: ops.decay_scan((shifted, 0), (shifted, sh * sd), (shifted, 2 * sh * sd), shift_state, seq_start, seq_slot, sh, sd, sd,
+                                                decay=decays, bonus=bonus, max_new=ctx.max_new), 8, samples)
+        row(f"{label}: scan of token-shift mixing (Tugalix's), {sh} heads of {sd} x {sd}", times, seqs * sh * sd * sd * 8 if decode else 0,
+            0 if decode else 4.0 * tokens * sh * sd * sd)
+        # ---- around a sublayer --------------------------------------------------------------------------------------------
+        residual = rand(tokens, width, scale=1.0, dtype=f32)
+        first, second = ops.Product(rand(tokens, width, scale=1.0), 1), ops.Product(rand(tokens, width, scale=1.0), 1)
+        norm_w, numbers = rand(width, scale=1.0), rand(tokens, 4, scale=1.0, dtype=f32)
+        times = _timed(lambda i: ops.add_rmsnorm(residual, first, norm_w, 1e-5, bf), 8, samples)
+        row(f"{label}: add + norm (Llama's)", times, tokens * width * (4 + 4 + 2 + 2))
+        times = _timed(lambda i: ops.layer_norm(residual, ops.ScaledSum(first, 1.0, second, 1.0), norm_w, None, 1e-5, bf, centred=False), 8, samples)
+        row(f"{label}: add of both sides + norm", times, tokens * width * (4 + 4 + 2 + 2 + 2))
+        times = _timed(lambda i: ops.layer_norm(residual, ops.ScaledSum(first, 1.0, second, 1.0, row_scale=numbers), norm_w, None, 1e-5, f32,
+                                                centred=False), 8, samples)
+        row(f"{label}: add of experts and identities + norm, floats out", times, tokens * width * (4 + 4 + 2 + 2 + 4))
+        normed, taps = rand(tokens, width, scale=1.0, dtype=f32), rand(width, 2, scale=0.3)
+        conv_state = torch.zeros(seqs, 1, width, dtype=f32, device=device)
+        times = _timed(lambda i: ops.input_conv(normed, taps, conv_state, ctx, bf), 8, samples)
+        row(f"{label}: token shift", times, tokens * width * (4 + 2) + (seqs * width * 8 if decode else 0))
+        mu, blend_state = torch.rand(5, width, device=device).to(bf), torch.zeros(seqs, width, dtype=f32, device=device)
+        x = rand(tokens, width, scale=1.0)
+        times = _timed(lambda i: ops.token_shift(x, mu, blend_state, ctx), 8, samples)
+        row(f"{label}: five blends with the token before (Tugalix's)", times, tokens * width * (2 + 5 * 2))
+        embed = rand(vocab, width)
+        ids = torch.randint(0, vocab, (tokens,), dtype=torch.int32, device=device)
+        times = _timed(lambda i: ops.pass_input(residual, ids, embed, bf), 8, samples)
+        row(f"{label}: what a pass begins with, side by side", times, tokens * width * (4 + 2 + 4))
+        del embed
+        # ---- feed-forwards --------------------------------------------------------------------------------------------------
+        router, correction = rand(experts + identity, width), rand(experts + identity, scale=0.01, dtype=f32)
+        groups = (sizes["groups"], sizes["keep"])
+        times = _timed(lambda i: ops.few_outputs(x, router, None, top=top, score="softmax_of_chosen"), 8, samples)
+        row(f"{label}: router, softmax over the chosen {top} of {experts + identity} (Narolorn's)", times, (tokens + experts + identity) * width * 2)
+        times = _timed(lambda i: ops.grouped_router(x, router, correction, top, identity, *groups), 8, samples)
+        row(f"{label}: router, {top} of {experts} and {identity} identities, {groups[1]} of {groups[0]} groups", times,
+            (tokens + experts + identity) * width * 2)
+        scale = ops.grouped_router(x, router, correction, top, identity, *groups)
+        pairs = float((scale[:, :experts] > 0).sum())
+        used = float((scale[:, :experts] > 0).any(dim=0).sum())
+        from .parts.linear import Linear
+        for name, inner in (("dense", ff), ("Llama's", lff)):
+            count = 2 if not decode else _copies(width * inner * 2)
+            ups = [Linear(rand(inner * (2 if name == "Llama's" else 1), width), None, bf) for _ in range(count)]
+            downs = [Linear(rand(width, inner), None, bf) for _ in range(count)]
+            if name == "Llama's":
+                times = _timed(lambda i: ops.silu_mul(ups[i](x), bf, interleaved=True) if not decode else ups[i](x, gated=True), count, samples)
+            else:
+                times = _timed(lambda i: ups[i].relu_squared(x), count, samples)
+            cols = ups[0].out_features
+            row(f"{label}: {name} feed-forward's first product and activation [{cols} x {width}]", times,
+                width * cols * 2 if decode else 0, 0 if decode else 2.0 * tokens * width * cols)
+            hidden = rand(tokens, inner, scale=1.0)
+            times = _timed(lambda i: downs[i](hidden), count, samples)
+            row(f"{label}: {name} feed-forward's second product [{width} x {inner}]", times,
+                width * inner * 2 if decode else 0, 0 if decode else 2.0 * tokens * width * inner)
+            del ups, downs
+        total = experts * eff
+        up, down = Linear(rand(total, width), None, bf), Linear(rand(width, total), None, bf)
+        times = _timed(lambda i: up.relu_squared(x, scale, eff), 2, samples)
+        row(f"{label}: experts' first product and activation over all columns ({experts} of {eff}, {pairs / tokens:.2f} in use a token)", times,
+            width * eff * used * 2 if decode else 0, 0 if decode else 2.0 * pairs * width * eff)
+        hidden = up.relu_squared(x, scale, eff)
+        times = _timed(lambda i: down(hidden), 2, samples)
+        row(f"{label}: experts' second product over all columns", times, width * eff * used * 2 if decode else 0,
+            0 if decode else 2.0 * pairs * width * eff)
+        if ops.routed_products_pay(tokens, up.weight, down.weight, experts, top):
+            plan = ops.route_plan(scale, experts, top)
+            times = _timed(lambda i: ops.route_plan(scale, experts, top), 8, samples)
+            row(f"{label}: plan of the pairs of experts and tokens", times, tokens * experts * 8)
+            times = _timed(lambda i: ops.routed_relu_squared(x, up.weight, plan), 2, samples)
+            row(f"{label}: experts' first product and activation over the pairs", times, 0, 2.0 * pairs * width * eff)
+            paired = ops.routed_relu_squared(x, up.weight, plan)
+            times = _timed(lambda i: ops.routed_down(paired, down.weight, plan), 2, samples)
+            row(f"{label}: experts' second product over the pairs", times, 0, 2.0 * pairs * width * eff)
+            apart = ops.routed_down(paired, down.weight, plan)
+            times = _timed(lambda i: ops.routed_sum(apart, plan), 4, samples)
+            row(f"{label}: sum of a token's pairs", times, int((pairs + tokens) * width * 2))
+            del paired, apart
+        pre = ops.Product(rand(tokens, ff, scale=1.0), 1)
+        times = _timed(lambda i: ops.relu_squared(pre, bf), 4, samples)
+        row(f"{label}: squared ReLU", times, tokens * ff * 4)
+        gate_up = ops.Product(rand(tokens, 2 * lff, scale=1.0), 1)
+        times = _timed(lambda i: ops.silu_mul(gate_up, bf, interleaved=True), 4, samples)
+        row(f"{label}: SiLU gate (Llama's)", times, tokens * lff * 6)
+        del up, down, hidden
+    return rows

@@ -212,6 +212,13 @@ def _check_cache(cache: torch.Tensor, num_kv_heads: int, head_dim: int, what: st
     return cache.shape[2] // (head_dim + value_dim)
 
 
+def _check_head_scale(head_scale: torch.Tensor | None, num_heads: int) -> None:
+    if head_scale is not None:
+        _device_tensor(head_scale, "head_scale", torch.float32)
+        if head_scale.shape != (num_heads,):
+            raise invalid_shape("head_scale needs one number a query head")
+
+
 def paired_rows(num_heads: int, num_kv_heads: int, head_dim: int, rot_dim: int) -> torch.Tensor:
     """The order in which the rows of a fused q/k/v weight are stored when rotation pairs are to sit
     side by side: within each q and k head, element i of the rotated part goes to 2i and element
@@ -230,9 +237,11 @@ def paired_rows(num_heads: int, num_kv_heads: int, head_dim: int, rot_dim: int) 
 
 def rope_cache(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor, inv_freq: torch.Tensor | None,
                rot_dim: int, cache: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
-               act_dtype: torch.dtype, paired: bool = False) -> torch.Tensor:
+               act_dtype: torch.dtype, paired: bool = False, extra_cols: int = 0,
+               head_scale: torch.Tensor | None = None) -> torch.Tensor:
     """Rotates q and k, returns q [T, nq * d], writes k and v into the cache rows of `slot_map`.
-    paired: qkv's columns are in the order of `paired_rows`.
+    paired: qkv's columns are in the order of `paired_rows`.  extra_cols: columns that the product has after q, k and v, which
+    are someone else's to read.  head_scale (float32 [nq]): query head h is multiplied by head_scale[h].
 
     slot_map[t] = page * page_size + row, or -1 to skip.  The slot map comes from the cache
     manager, which hands out only rows of pages it owns."""
@@ -241,8 +250,9 @@ def rope_cache(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor, in
     _device_tensor(slot_map, "slot_map", torch.int32)
     _device_tensor(cache, "cache", act_dtype)
     tokens = qkv.rows
-    if qkv.cols != (num_heads + 2 * num_kv_heads) * head_dim:
-        raise invalid_shape(f"rope_cache: qkv width {qkv.cols} is not (nq + 2 nkv) * d")
+    if extra_cols < 0 or qkv.cols != (num_heads + 2 * num_kv_heads) * head_dim + extra_cols:
+        raise invalid_shape(f"rope_cache: qkv width {qkv.cols} is not (nq + 2 nkv) * d + {extra_cols}")
+    _check_head_scale(head_scale, num_heads)
     if positions.shape != (tokens,) or slot_map.shape != (tokens,):
         raise invalid_shape("rope_cache: positions and slot_map need one entry per token")
     page_size = _check_cache(cache, num_kv_heads, head_dim, "rope_cache")
@@ -256,7 +266,8 @@ def rope_cache(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor, in
     _check(library().tlie_rope_cache(_ptr(qkv.data), dtype_code(qkv.data.dtype), qkv.nsplit,
                                      ctypes.c_longlong(qkv.split_stride), _ptr(positions), _ptr(slot_map), _ptr(inv_freq),
                                      rot_dim, _ptr(q_out), _ptr(cache), dtype_code(act_dtype), tokens, num_heads,
-                                     num_kv_heads, head_dim, page_size, 1 if paired else 0, _stream()), "rope_cache")
+                                     num_kv_heads, head_dim, page_size, 1 if paired else 0, qkv.cols, _ptr(head_scale),
+                                     _stream()), "rope_cache")
     return q_out
 
 
@@ -401,10 +412,7 @@ def qkv_place(qkv: Product, positions: torch.Tensor, slot_map: torch.Tensor | No
                 raise invalid_shape(f"qkv_place: {name} needs {count} entries and a positive eps")
     if q_temp is not None and not float(q_temp[1]) > 0.0:
         raise invalid_argument("qkv_place: the query temperature's period must be positive")
-    if head_scale is not None:
-        _device_tensor(head_scale, "head_scale", torch.float32)
-        if head_scale.shape != (num_heads,):
-            raise invalid_shape("qkv_place: head_scale needs one number a query head")
+    _check_head_scale(head_scale, num_heads)
     _device_tensor(positions, "positions", torch.int32)
     tokens = qkv.rows
     value_heads = num_kv_heads if value_heads is None else int(value_heads)
@@ -1451,6 +1459,100 @@ def gemm_tiles(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype = t
     return out
 
 
+# ---- products of a routed feed-forward over the pairs of experts and tokens ------------------------------
+
+
+@dataclass
+class RoutePlan:
+    """Which tokens use which expert, on the device: counts int32 [experts], lists int32 [experts, tokens] (an expert's
+    tokens in order), ranks int32 [tokens, experts] (a token's place in the expert's list), from the router's scale matrix
+    (float32 [tokens, at least experts]; 0: not used).  most: the most experts a token uses."""
+    scale: torch.Tensor
+    counts: torch.Tensor
+    lists: torch.Tensor
+    ranks: torch.Tensor
+    most: int
+
+    @property
+    def tokens(self) -> int:
+        return self.lists.shape[1]
+
+    @property
+    def experts(self) -> int:
+        return self.lists.shape[0]
+
+
+def route_plan(scale: torch.Tensor, experts: int, most: int) -> RoutePlan:
+    _device_tensor(scale, "scale", torch.float32)
+    if scale.dim() != 2 or not 0 < experts <= scale.shape[1] or not 0 < most <= experts:
+        raise invalid_shape("route_plan: a scale matrix [tokens, experts (or more)], and 1 to all experts a token")
+    tokens, device = scale.shape[0], scale.device
+    plan = RoutePlan(scale, torch.empty(experts, dtype=torch.int32, device=device), torch.empty((experts, tokens), dtype=torch.int32, device=device),
+                     torch.empty((tokens, experts), dtype=torch.int32, device=device), int(most))
+    if tokens > 0:
+        _check(library().tlie_route_plan(_ptr(scale), scale.shape[1], tokens, experts, _ptr(plan.counts), _ptr(plan.lists), _ptr(plan.ranks),
+                                         _stream()), "route_plan")
+    return plan
+
+
+def routed_tiles_take(up: torch.Tensor, down: torch.Tensor, experts: int) -> bool:
+    """Whether the tiles take these matrices: up [experts * size, width], down [width, experts * size]."""
+    return (up.dtype == torch.bfloat16 and down.dtype == torch.bfloat16 and up.shape[1] % 64 == 0
+            and (up.shape[0] // experts) % 64 == 0)
+
+
+def routed_products_pay(rows: int, up: torch.Tensor, down: torch.Tensor, experts: int, most: int) -> bool:
+    """Whether a step of `rows` tokens takes the products over pairs of experts and tokens rather than over all experts' columns:
+    where the tiles take the matrices, in steps of more tokens than the products of few rows serve, when a token leaves at
+    least half of the experts unused.  Measured with 4 of 14 experts of 2112 at width 2048 (of 5376 at 4096), both products
+    and all around them: 96 tokens 79 us against 106 (327 against 547), 512 tokens 107 against 225 (430 against 815), 2048
+    tokens 204 against 471 (978 against 2211)."""
+    return rows > SKINNY_MAX_ROWS and experts >= 2 * most and down.shape[0] % 8 == 0 and routed_tiles_take(up, down, experts)
+
+
+def routed_relu_squared(x: torch.Tensor, up: torch.Tensor, plan: RoutePlan) -> torch.Tensor:
+    """bfloat16 [tokens * most, size]: s * max(W_up[e] x, 0)^2 of every pair of an expert and a token that uses it, an
+    expert's pairs side by side, the experts in order (what lies beyond the last pair is not written).  up: bfloat16
+    [experts * size, width]; s: the token's number for the expert."""
+    _device_tensor(x, "x", torch.bfloat16)
+    _device_tensor(up, "up", torch.bfloat16)
+    if x.dim() != 2 or up.dim() != 2 or x.shape != (plan.tokens, up.shape[1]) or up.shape[0] % plan.experts != 0:
+        raise invalid_shape(f"routed_relu_squared: x {list(x.shape)} and up {list(up.shape)} do not fit {plan.tokens} tokens and {plan.experts} experts")
+    size = up.shape[0] // plan.experts
+    out = torch.empty((plan.tokens * plan.most, size), dtype=torch.bfloat16, device=x.device)
+    if plan.tokens > 0:
+        _check(library().tlie_routed_tiles(_ptr(x), _ptr(up), _ptr(plan.counts), _ptr(plan.lists), _ptr(plan.scale), plan.scale.shape[1], _ptr(out),
+                                           plan.tokens, plan.experts, plan.most, size, up.shape[1], 1, _stream()), "routed_tiles")
+    return out
+
+
+def routed_down(hidden: torch.Tensor, down: torch.Tensor, plan: RoutePlan) -> torch.Tensor:
+    """bfloat16 [tokens * most, width]: W_down[e] hidden of every pair (see `routed_relu_squared`).  down: bfloat16
+    [width, experts * size], an expert's matrix the columns from e * size on."""
+    _device_tensor(hidden, "hidden", torch.bfloat16)
+    _device_tensor(down, "down", torch.bfloat16)
+    if (hidden.dim() != 2 or down.dim() != 2 or hidden.shape[0] != plan.tokens * plan.most
+            or down.shape[1] != plan.experts * hidden.shape[1]):
+        raise invalid_shape(f"routed_down: hidden {list(hidden.shape)} and down {list(down.shape)} do not fit the plan")
+    out = torch.empty((hidden.shape[0], down.shape[0]), dtype=torch.bfloat16, device=hidden.device)
+    if plan.tokens > 0:
+        _check(library().tlie_routed_tiles(_ptr(hidden), _ptr(down), _ptr(plan.counts), _ptr(plan.lists), _ptr(None), 0, _ptr(out), plan.tokens,
+                                           plan.experts, plan.most, down.shape[0], hidden.shape[1], 0, _stream()), "routed_tiles")
+    return out
+
+
+def routed_sum(y: torch.Tensor, plan: RoutePlan) -> torch.Tensor:
+    """bfloat16 [tokens, width]: the sum of the token's pairs' rows of y, in the order of the experts."""
+    _device_tensor(y, "y", torch.bfloat16)
+    if y.dim() != 2 or y.shape[0] != plan.tokens * plan.most or y.shape[1] % 8 != 0:
+        raise invalid_shape(f"routed_sum: y {list(y.shape)} does not fit the plan (a width that is a multiple of 8)")
+    out = torch.empty((plan.tokens, y.shape[1]), dtype=torch.bfloat16, device=y.device)
+    if plan.tokens > 0:
+        _check(library().tlie_routed_sum(_ptr(y), _ptr(plan.scale), plan.scale.shape[1], _ptr(plan.counts), _ptr(plan.ranks), _ptr(out), plan.tokens,
+                                         plan.experts, plan.most, y.shape[1], _stream()), "routed_sum")
+    return out
+
+
 def library_fallbacks() -> int:
     """How many products `library_mm` has made with this library's own kernels because the vendor's
     library was not there or offered nothing for the shape (each slower, some many times)."""
@@ -1969,7 +2071,8 @@ def gemm_rows_shape(out_features: int, in_features: int, epilogue: str = "store"
 
 @dataclass
 class RopeTarget:
-    """What the rotation and cache write need besides the q/k/v product: see `rope_cache`."""
+    """What the rotation and cache write need besides the q/k/v product: see `rope_cache`.  extra_cols: rows that the weight
+    has after those of q, k and v; with them the product comes back as (q, a `Product` of those columns)."""
     positions: torch.Tensor
     slot_map: torch.Tensor
     inv_freq: torch.Tensor | None
@@ -1978,6 +2081,8 @@ class RopeTarget:
     num_heads: int
     num_kv_heads: int
     head_dim: int
+    extra_cols: int = 0
+    head_scale: torch.Tensor | None = None
 
 
 def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str = "store",
@@ -2050,8 +2155,11 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
         _device_tensor(rope.positions, "positions", torch.int32)
         _device_tensor(rope.slot_map, "slot_map", torch.int32)
         _device_tensor(rope.cache, "cache", torch.bfloat16)
-        if out_features != (rope.num_heads + 2 * rope.num_kv_heads) * rope.head_dim:
-            raise invalid_shape(f"gemm_rows: {out_features} rows of W are not (nq + 2 nkv) * d")
+        if rope.extra_cols < 0 or out_features != (rope.num_heads + 2 * rope.num_kv_heads) * rope.head_dim + rope.extra_cols:
+            raise invalid_shape(f"gemm_rows: {out_features} rows of W are not (nq + 2 nkv) * d + {rope.extra_cols}")
+        _check_head_scale(rope.head_scale, rope.num_heads)
+        if rope.extra_cols:
+            y = torch.empty((rows, rope.extra_cols), dtype=torch.float32, device=device)
         if rope.positions.shape != (rows,) or rope.slot_map.shape != (rows,):
             raise invalid_shape("gemm_rows: positions and slot_map need one entry per token")
         page_size = _check_cache(rope.cache, rope.num_kv_heads, rope.head_dim, "gemm_rows")
@@ -2075,9 +2183,10 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
                                     strips_in, in_features, ctypes.c_float(eps), code, _ptr(y), _ptr(act), _ptr(residual),
                                     _ptr(next_weight), next_code, _ptr(xg), _ptr(ssq_out), *rope_args, waves, rows_per_block,
                                     *_gate_args(gate if epilogue == "silu" else None),
-                                    _ptr(act_scale if epilogue == "relu2" else None), scale_cols, block, _stream()), "gemm_rows")
+                                    _ptr(act_scale if epilogue == "relu2" else None), scale_cols, block,
+                                    _ptr(rope.head_scale if epilogue == "rope" else None), _stream()), "gemm_rows")
     if epilogue == "rope":
-        return q_out
+        return (q_out, Product(y, 1)) if rope.extra_cols else q_out
     if epilogue == "store":
         return Product(y, 1)
     if epilogue in ("silu", "relu2"):

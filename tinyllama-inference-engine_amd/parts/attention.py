@@ -86,6 +86,8 @@ class Attention(Mixer):
         self.qk_norm = spec.get("qk_norm")
         self.norm_eps = float(spec.get("norm_eps", 0.0))
         self.head_temp, self.head_gate = bool(spec.get("head_temp", False)), bool(spec.get("head_gate", False))
+        if (self.head_temp or self.head_gate) and self.position.rotary_table() is None and type(self.position).apply_qk is not PositionEncoding.apply_qk:
+            raise invalid_config("attention: numbers a head go with a rotation table or no positions")
         if self.head_gate and self.bias:
             raise invalid_config("attention: a gate a head goes with projections without biases")
         if self.softcap is not None and not self.softcap > 0.0:
@@ -98,11 +100,12 @@ class Attention(Mixer):
             raise invalid_config("attention: qk_norm is \"whole\" (with a positive norm_eps, on a layer with keys of its own) or absent")
         # what the kernels that are fused for the plain case (one head size, no sink, no chunks, own keys
         # and values, scores as they are) do not take goes through the kernels for any sizes
-        self.placed = (self.q_temp is not None or self.values_are_keys or self.qk_norm is not None or self.head_temp
-                       or self.head_gate)                  # options of the placement kernel alone (or columns that it steps over)
+        self.placed = self.q_temp is not None or self.values_are_keys or self.qk_norm is not None   # options of the placement kernel alone
         self.general = (self.dv != self.d or self.has_sink or self.chunk is not None or self.reads_other_cache
                         or self.softcap is not None or self.placed)
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
+        # the heads' gates are columns of the q/k/v product, after those (as many as keep its rows' starts aligned)
+        self.gate_cols = (self.nq + 7) // 8 * 8 if self.head_gate else 0
         self.qkv = self.o = self.sink = self.q_norm = self.k_norm = self.temp = None
 
     @classmethod
@@ -142,10 +145,12 @@ class Attention(Mixer):
         roles = ("q",) if self.reads_other_cache else (("q", "k") if self.values_are_keys else ("q", "k", "v"))
 
         def cat(suffix):
-            # (the heads' gates are columns of the same product, after q, k and v)
-            last = ("head_gate",) if self.head_gate and not suffix else ()
-            joined = torch.cat([weights[prefix + names[role + suffix]] for role in (*roles, *last)], dim=0)
-            return joined[order].contiguous() if order is not None else joined
+            joined = torch.cat([weights[prefix + names[role + suffix]] for role in roles], dim=0)
+            joined = joined[order].contiguous() if order is not None else joined
+            if not self.head_gate:
+                return joined
+            gate = weights[prefix + names["head_gate"]].to(joined.dtype)
+            return torch.cat([joined, gate, gate.new_zeros(self.gate_cols - self.nq, self.hidden)], dim=0)
         keep = partial(keep_in, weights)
         self.qkv = Linear(cat(""), cat("_bias") if self.bias else None, self.dtype, keep=keep)
         self.o = Linear(weights[prefix + names["o"]], weights.get(prefix + names["o_bias"]) if self.bias else None,
@@ -196,17 +201,17 @@ class Attention(Mixer):
         inv_freq, rot_dim = table if table is not None else (None, 0)
         writes = binding.writes and not self.reads_other_cache
         q = fused = None
-        if (table is None and self.dv == self.d and self.d % 2 == 0 and not self.reads_other_cache and not self.placed
+        if (table is None and self.dv == self.d and self.d % 2 == 0 and not self.reads_other_cache and not self.placed and not self.head_gate
                 and self.qkv.takes_rows(x.shape[0])):
             # a step of few rows, one head size, own keys and values: the product places q and writes the cache itself
             q = self.qkv(x, rope=ops.RopeTarget(ctx.positions, pages.slot_map if writes else ctx.no_slots, None, 0, binding.cache,
-                                                self.nq, self.nkv, self.d))
+                                                self.nq, self.nkv, self.d, head_scale=self.temp))
         if q is None or isinstance(q, ops.Product):
             fused = ops.as_product(q if q is not None else self.qkv(x))
             q = ops.qkv_place(fused, ctx.positions, pages.slot_map if writes else ctx.no_slots, inv_freq,
                           rot_dim, binding.cache, self.nq, 0 if self.reads_other_cache else self.nkv, self.d, self.dv, self.dtype,
                           q_norm=self.q_norm, k_norm=self.k_norm, norm_eps=self.norm_eps, values_are_keys=self.values_are_keys,
-                          q_temp=self.q_temp, head_scale=self.temp, extra_cols=self.nq if self.head_gate else 0)
+                          q_temp=self.q_temp, head_scale=self.temp, extra_cols=self.gate_cols)
         if self.dv == self.d and ops.attention_mfma_takes(self.dtype, self.d, binding.cache.shape[3] // self.d):
             # bfloat16, one head size: the kernel on the matrix cores (scores, softmax and sink float)
             tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d)
@@ -219,7 +224,7 @@ class Attention(Mixer):
                                              seq_start=ctx.seq_start, value_dim=self.dv, chunk=self.chunk, sink=self.sink,
                                              softcap=self.softcap)
         if self.head_gate:
-            attended = ops.head_gate(attended, fused, fused.cols - self.nq, self.nq)
+            attended = ops.head_gate(attended, fused, fused.cols - self.gate_cols, self.nq)
         return self.o(attended)
 
     def forward(self, x, ctx, binding: Binding, into=None):
@@ -231,14 +236,19 @@ class Attention(Mixer):
         inv_freq, rot_dim = table if table is not None else (None, 0)
         other_positions = table is None and type(self.position).apply_qk is not PositionEncoding.apply_qk
         target = None
-        if not other_positions:
-            target = ops.RopeTarget(ctx.positions, slot_map, inv_freq, rot_dim, binding.cache, self.nq, self.nkv, self.d)
+        if not other_positions and self.d % 2 == 0:
+            target = ops.RopeTarget(ctx.positions, slot_map, inv_freq, rot_dim, binding.cache, self.nq, self.nkv, self.d,
+                                    extra_cols=self.gate_cols, head_scale=self.temp)
         q = self.qkv(x, rope=target)
+        gates = None
+        if isinstance(q, tuple):
+            q, gates = q
         if isinstance(q, ops.Product):              # the product did not rotate: a kernel of its own does
+            gates = q
             if other_positions:
                 q = self._apply_other_positions(q, ctx)
             q = ops.rope_cache(q, ctx.positions, slot_map, inv_freq, rot_dim, binding.cache, self.nq, self.nkv, self.d,
-                               self.dtype, paired=self.paired)
+                               self.dtype, paired=self.paired, extra_cols=self.gate_cols, head_scale=self.temp)
         page_size = binding.cache.shape[3] // self.d
         if ops.attention_mfma_takes(self.dtype, self.d, page_size):
             tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d)
@@ -248,6 +258,8 @@ class Attention(Mixer):
             attended = ops.attention_generic(q, binding.cache, pages.block_table, ctx.token_seq, ctx.positions, self.nq,
                                              self.nkv, self.d, self.window, self.scale,
                                              tiled=ops.attention_generic_plan(ctx, self.d), seq_start=ctx.seq_start)
+        if self.head_gate:
+            attended = ops.head_gate(attended, gates, gates.cols - self.gate_cols, self.nq)
         return self.o(attended, into=into)
 
     def _apply_other_positions(self, qkv, ctx):

@@ -26,8 +26,9 @@ products around a gate kernel that multiplies an expert's columns by the token's
 expert that the token does not use (silu(0) * 0 adds nothing to the second product, exactly).  Since the products
 are linear, s (W x) stands for W (s x); a weight on an expert's result multiplies the columns of the second product's
 input in the result's place; and the shared expert's gate is one more row of the router's matrix, which stands outside
-the choice.  An expert without a gate has its up rows alone in the first matrix.  The identities' weights together
-multiply the row x, which whoever adds the feed-forward's result into the residual adds beside it (`ops.ScaledSum`).
+the choice.  An expert without a gate has its up rows alone in the first matrix.  In a step of many tokens the
+products of such experts run over the pairs of an expert and a token that uses it (`ops.route_plan`), where that pays.  The
+identities' weights together multiply the row x, which whoever adds the feed-forward's result into the residual adds beside it (`ops.ScaledSum`).
 """
 from __future__ import annotations
 
@@ -166,8 +167,12 @@ class RoutedMLP(FeedForward):
             scale = ops.grouped_router(x, self.router, self.correction, self.top, self.identity, self.groups, self.keep_groups)
         else:
             scale = ops.few_outputs(x, self.router, self.router_b, top=self.top, score=self.score)
-        hidden = self.gate_up.relu_squared(x, scale, self.expert_size)
-        out = self.down(hidden)
+        most = min(self.top, self.experts)
+        if ops.routed_products_pay(x.shape[0], self.gate_up.weight, self.down.weight, self.experts, most) and x.dtype == torch.bfloat16:
+            plan = ops.route_plan(scale, self.experts, most)
+            out = ops.routed_sum(ops.routed_down(ops.routed_relu_squared(x, self.gate_up.weight, plan), self.down.weight, plan), plan)
+        else:
+            out = self.down(self.gate_up.relu_squared(x, scale, self.expert_size))
         if self.identity == 0:
             return out
         # the identities' weights together are the scale matrix's last column: x times it joins beside the experts' sum
