@@ -430,6 +430,57 @@ def test_products_of_few_rows_apply_the_squared_relu_themselves(rows, outputs, i
     assert float(got[0, :block].abs().max()) == 0.0
 
 
+@pytest.mark.parametrize("batch,rows,outputs,inner", [(4, 8, 96, 128), (1, 1, 40, 64), (3, 16, 2048, 72), (5, 3, 17, 1000)])
+def test_several_products_of_one_shape_in_one_launch(batch, rows, outputs, inner):
+    from tlie_amd import ops
+    generator = torch.Generator().manual_seed(outputs)
+    x = torch.randn(batch, rows, inner, generator=generator).bfloat16()
+    w = (torch.randn(batch, outputs, inner, generator=generator) / math.sqrt(inner)).bfloat16()
+    for index, got in enumerate(ops.gemm_rows_batch(x.to(DEVICE), w.to(DEVICE))):
+        want = x[index].double() @ w[index].double().T
+        assert float((got.dense().cpu().double() - want).abs().max()) < 1e-4
+
+
+@pytest.mark.parametrize("tokens,window,context", [(3, 20, 500), (8, 100, 3000), (2, 1024, 5000), (1, 40, 30)])
+def test_a_decode_step_over_a_window_shares_the_windows_keys(tokens, window, context):
+    """Long sequences and a short window: the parts of the keys lie in the window, wherever it begins, and no key is left
+    out or taken twice; one key at the window's edge, just inside or just outside, towers over the rest."""
+    from tlie_amd import ops
+    generator = torch.Generator().manual_seed(window)
+    heads, groups, d, page_size = 4, 2, 32, 16
+    blocks = -(-context // page_size)
+    lengths = [context - 37 * index for index in range(tokens)] if context > 400 else [context] * tokens
+    ctx = SimpleNamespace(max_new=1, num_seqs=tokens, num_tokens=tokens, max_context=context, scratch={}, tile_owner=None, compute_units=256, host={})
+    plan = ops.attention_plan(ctx, heads // groups, groups, d, window)
+    assert plan[2] == 1 or plan[2] * plan[3] < context or window + 31 >= context
+    tiles, col_tiles, nsplit, split_len, waves, shared = plan
+    k, v = (torch.randn(tokens, context, groups, d, generator=generator).bfloat16() for _ in range(2))
+    q = torch.randn(tokens, heads, d, generator=generator).bfloat16()
+    positions = torch.tensor([length - 1 for length in lengths], dtype=torch.int32, device=DEVICE)
+    table = torch.randperm(tokens * blocks, generator=generator).to(torch.int32).view(tokens, blocks)
+    for back in (window - 1, window, 0):                          # the towering key, so many positions before the token
+        keys = k.clone()
+        for t, length in enumerate(lengths):
+            if length - 1 - back >= 0:
+                keys[t, length - 1 - back] = 4.0 * q[t].float().reshape(groups, heads // groups, d).mean(dim=1).bfloat16()
+        cache = torch.zeros(tokens * blocks, 2, groups, page_size * d, dtype=torch.bfloat16)
+        for t in range(tokens):
+            for b in range(blocks):
+                rows = slice(b * page_size, min((b + 1) * page_size, context))
+                count = rows.stop - rows.start
+                page = cache[int(table[t, b])]
+                page[0].view(groups, page_size, d)[:, :count] = keys[t, rows].transpose(0, 1)
+                page[1].view(groups, d, page_size)[:, :, :count] = v[t, rows].permute(1, 2, 0)
+        got = ops.attention_mfma(q.reshape(tokens, -1).to(DEVICE), cache.to(DEVICE), table.to(DEVICE), tiles, positions, heads, groups, d, window, 0.3,
+                                 nsplit, split_len, col_tiles, waves, shared).float().cpu().reshape(tokens, heads, d)
+        for t, length in enumerate(lengths):
+            lo = max(0, length - window)
+            for h in range(heads):
+                weights = torch.softmax(0.3 * keys[t, lo:length, h // 2].double() @ q[t, h].double(), dim=0)
+                want = weights @ v[t, lo:length, h // 2].double()
+                assert float((got[t, h].double() - want).abs().max()) < 3e-2, f"token {t}, head {h}, key {back} back"
+
+
 @pytest.mark.parametrize("width,dtype", [(64, torch.float32), (50, torch.float32), (2056, torch.bfloat16), (30, torch.bfloat16)])
 def test_what_a_pass_begins_with(width, dtype):
     from tlie_amd import ops

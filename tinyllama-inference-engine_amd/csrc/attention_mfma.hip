@@ -187,7 +187,10 @@ attention_mfma_kernel(const uint16_t* __restrict__ q, const uint16_t* __restrict
   const int last_col = min(col0 + 16 * CT - 1, ncols - 1);
   const int tile_hi = pos0 + last_col / G + 1;
   const int tile_lo = bounded ? lower(pos0 + col0 / G) : 0;
-  const int split_lo = nsplit > 1 ? split * split_len : 0;
+  // (parts are counted from the first block that the workgroup's first column sees, so that with a window or chunks every
+  // part has keys to read however long the sequence is)
+  const int parts_lo = bounded && nsplit > 1 ? __builtin_amdgcn_readfirstlane(lower(pos0 + group_col0 / G) & ~31) : 0;
+  const int split_lo = nsplit > 1 ? parts_lo + split * split_len : 0;
   const int range_lo = __builtin_amdgcn_readfirstlane(wave_active ? max(tile_lo, split_lo) : 0);
   const int range_hi = __builtin_amdgcn_readfirstlane(wave_active ? (nsplit > 1 ? min(tile_hi, split_lo + split_len) : tile_hi) : 0);
 
@@ -744,7 +747,8 @@ using namespace tlie;
 // tiles: int32 [num_tiles, 4] with 16 * col_tiles columns each, or null for a decode step (then
 // col_tiles = 1 and num_tiles = tokens * ceil(G / 16)).
 // part_o: float [tokens * nq * nsplit * d], part_ml: float [tokens * nq * nsplit * 2] (both only when nsplit > 1);
-// split_len: positions per part, a multiple of 32, nsplit * split_len >= the longest sequence.
+// split_len: positions per part, a multiple of 32, nsplit * split_len >= the longest sequence, or (window or chunk > 0)
+// the most positions from the first block that a tile sees to its last token.
 // d % 16 == 0, d <= 256, page_size a power of two >= 16; col_tiles 1, or 4 for d <= 64, or 2 for d <= 128.
 // shared != 0 (prompt portions, col_tiles 1 or 2, d <= 128, 4 or 8 waves): tiles have 16 * col_tiles * waves columns, every wave
 // takes 16 * col_tiles of them, and keys and values reach the waves through LDS.  Otherwise:

@@ -169,12 +169,16 @@ gemm_rows_kernel(const RowsArgs a) {
   const int block_row = blockIdx.x * a.rows_per_block;
   const int strip_rows = STRIPS == 1 ? a.rows_per_block : 16;                 // with 8 rows a block, half the strip is idle
   const int k_begin = wave * a.k_per_wave, k_end = min(a.K, k_begin + a.k_per_wave);
+  // (store: product blockIdx.y of several of one shape that lie one after the other)
+  const size_t which = EPILOGUE == kEpilogueStore ? blockIdx.y : 0;
+  const uint16_t* const w_all = a.w + which * a.N * a.K;
+  const uint16_t* const x_all = a.x + which * a.M * a.K;
   // (a row beyond the matrix, in its last strip, becomes the last row: read again, never stored)
   const uint16_t* w_row[STRIPS];
 #pragma unroll
   for (int st = 0; st < STRIPS; ++st)
-    w_row[st] = a.w + static_cast<size_t>(min(block_row + st * 16 + col, a.N - 1)) * a.K;
-  const uint16_t* x_row = a.x + static_cast<size_t>(min(col, a.M - 1)) * a.K;
+    w_row[st] = w_all + static_cast<size_t>(min(block_row + st * 16 + col, a.N - 1)) * a.K;
+  const uint16_t* x_row = x_all + static_cast<size_t>(min(col, a.M - 1)) * a.K;
   const bool w_lane = col < strip_rows, x_lane = col < a.M;
 
   // the norm's partial sums of squares are asked for before the weights, and added up after the
@@ -284,7 +288,7 @@ gemm_rows_kernel(const RowsArgs a) {
       value += pre_bias[st][turn];
 
       if (EPILOGUE == kEpilogueStore) {
-        if (live) a.y[static_cast<size_t>(token) * a.N + n] = value;
+        if (live) a.y[(which * a.M + token) * a.N + n] = value;
       } else if (EPILOGUE == kEpilogueSilu) {
         const float up = __shfl_down(value, 1, 64);          // the odd row next to this even one
         if (live && (nn & 1) == 0) {
@@ -406,7 +410,8 @@ using namespace tlie;
 
 // x [M, K], w [N, K], bias [N] or null: bfloat16; M <= 16, K % 8 == 0.
 // ssq_in [strips_in, 16] or null (then no row scale); width: the normed input's width.
-// epilogue 0: y float [M, N].  1: act bfloat16 [M, N / 2], N even, W's rows alternating gate, up.
+// epilogue 0: y float [M, N]; batch > 1: so many products of one shape, x [batch, M, K], w [batch, N, K] and
+// y [batch, M, N] one after the other (no bias, no row scale).  1: act bfloat16 [M, N / 2], N even, W's rows alternating gate, up.
 // 4: act bfloat16 [M, N] = s * max(y, 0)^2, s from act_scale float [M, act_scale_cols] (a number for every act_block
 // columns), or 1 when it is null.
 // 2: residual float [M, N] += y; if xg is given, next_weight [N] (bfloat16 if next_weight_dtype is 1,
@@ -423,7 +428,8 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
                               const int* positions, const int* slot_map, const float* inv_freq, int rot_dim, int nq,
                               int nkv, int d, int page_size, void* q_out, void* cache, int waves, int rows_per_block,
                               int gate_kind, float gate_alpha, float gate_limit, const float* act_scale, int act_scale_cols,
-                              int act_block, const float* head_scale, void* stream) {
+                              int act_block, const float* head_scale, int batch, void* stream) {
+  if (batch < 1 || batch > 65535 || (batch > 1 && (epilogue != kEpilogueStore || bias != nullptr || ssq_in != nullptr))) return kBadArgument;
   if (gate_kind != kGateSilu && gate_kind != kGateClampedSwish) return kBadArgument;
   if (M <= 0 || M > 16 || N <= 0 || K <= 0 || (K & 7) != 0 || (waves != 2 && waves != 4 && waves != 8 && waves != 16)) return kBadArgument;
   if (!(rows_per_block >= 2 && rows_per_block <= 16 && rows_per_block % 2 == 0) && !(rows_per_block == 32 && waves <= 8)) return kBadArgument;
@@ -453,7 +459,7 @@ extern "C" int tlie_gemm_rows(const void* x, const void* w, const void* bias, in
   a.gate_kind = gate_kind, a.gate_alpha = gate_alpha, a.gate_limit = gate_limit;
   a.nq = nq, a.nkv = nkv, a.d = d, a.page_size = page_size, a.q_out = (uint16_t*)q_out, a.cache = (uint16_t*)cache;
   if (epilogue == kEpilogueRelu2) a.act_scale_cols = act_scale_cols, a.act_block = act_block;
-  const dim3 grid((N + rows_per_block - 1) / rows_per_block);
+  const dim3 grid((N + rows_per_block - 1) / rows_per_block, batch);
   hipStream_t s = (hipStream_t)stream;
 #define TLIE_CASE(E)                                                                                  \
   if (epilogue == E) {                                                                                \

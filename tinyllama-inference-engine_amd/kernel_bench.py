@@ -803,9 +803,8 @@ def bench_paluzen_kernels(sizes: dict, batch: int = 8, context: int = 2048, prom
         # ---- attention over a window (flops: the keys a token sees) ---------------------------------------------------
         cache = rand(pages, 2, G, page_size * d, scale=0.5)
         q = rand(tokens, H * d, scale=1.0)
-        plan = ops.attention_plan(ctx, H // G, G, d)
-        tiles, col_tiles, nsplit, split_len, waves, shared = plan
         for name, reach in (("causal (Llama's)", None), (f"window of {window}", window)):
+            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, H // G, G, d, reach)
             times = _timed(lambda i: ops.attention_mfma(q, cache, table, tiles, positions, H, G, d, reach, d ** -0.5, nsplit, split_len, col_tiles,
                                                         waves, shared), 8, samples)
             seen = min(keys, reach or keys)

@@ -1806,7 +1806,7 @@ def few_rows_route(rows: int, dtype: torch.dtype) -> bool:
     return dtype == torch.bfloat16 and 0 < rows <= ROWS_MAX
 
 
-def attention_plan(ctx, groups_per_kv: int, num_kv_heads: int, head_dim: int):
+def attention_plan(ctx, groups_per_kv: int, num_kv_heads: int, head_dim: int, reach: int | None = None):
     """How the tiled attention kernel is launched for the step `ctx` describes: its work list (made
     once per step and group size, kept in `ctx.scratch`; None for a decode step, whose tiles the
     kernel derives itself), and how the keys are cut: into as many parts as it takes to give a step
@@ -1814,12 +1814,17 @@ def attention_plan(ctx, groups_per_kv: int, num_kv_heads: int, head_dim: int):
     5 TB/s, 16 parts 4 TB/s, and merging more than 16 costs more than it gains), each part a
     multiple of 32 positions and at least 64.  The policy is this kernel's own and measured on the
     MI355X; the step's context only supplies the host arrays, the number of compute units, and, in a
-    recorded step, the owner of work lists at fixed addresses.
+    recorded step, the owner of work lists at fixed addresses.  reach: the most keys a token sees, itself
+    included (a window, a chunk): the parts of a decode step then share those keys (counted from the
+    block of 32 they begin in), not the whole sequence.
     Returns (tiles, col_tiles, nsplit, split_len, waves, shared): `waves` of a workgroup share a
     tile's keys, or with `shared` take columns of their own and get the keys through LDS."""
     decode = ctx.max_new == 1 and ctx.num_seqs == ctx.num_tokens
     col_tiles, shared = 1, False
+    context = ctx.max_context
     if decode:
+        if reach is not None:
+            context = min(context, int(reach) + 31)
         tiles, count = None, ctx.num_tokens * ((groups_per_kv + 15) // 16)
     else:
         col_tiles = attention_col_tiles(head_dim)
@@ -1870,20 +1875,20 @@ def attention_plan(ctx, groups_per_kv: int, num_kv_heads: int, head_dim: int):
         # launch, while a wave keeps 128 keys or more and the step has 2048 waves at most
         # (measured inside whole steps at 2048 positions: batch 1 16 parts x 1 wave, batch 8
         # 8 x 2, batch 64 1 x 8)
-        nsplit = max(1, min((256 + tiles_all - 1) // tiles_all, 16, (ctx.max_context + 63) // 64))
+        nsplit = max(1, min((256 + tiles_all - 1) // tiles_all, 16, (context + 63) // 64))
         waves = 1
         while (waves * 2 <= attention_max_waves(head_dim) and tiles_all * nsplit * waves * 2 <= 2048
-               and ctx.max_context >= nsplit * waves * 2 * 128):
+               and context >= nsplit * waves * 2 * 128):
             waves *= 2
-        if nsplit > 1 and ctx.max_context <= 256 and attention_max_waves(head_dim) >= 2:
+        if nsplit > 1 and context <= 256 and attention_max_waves(head_dim) >= 2:
             # up to 256 positions there is nothing to cut: two waves of one workgroup share the keys and the
             # merge launch goes (batch 1 at 200 positions 0.902 ms a step against 0.919, batch 8 0.998
             # against 1.017; at 450 positions the parts win again: 0.928 against 0.944 with 1 x 4)
             nsplit, waves = 1, 2
     if nsplit == 1:
         return tiles, col_tiles, 1, 0, waves, shared
-    split_len = ((ctx.max_context + nsplit - 1) // nsplit + 31) // 32 * 32
-    nsplit = (ctx.max_context + split_len - 1) // split_len
+    split_len = ((context + nsplit - 1) // nsplit + 31) // 32 * 32
+    nsplit = (context + split_len - 1) // split_len
     return tiles, col_tiles, nsplit, split_len, waves, shared
 
 
@@ -1904,7 +1909,8 @@ def attention_mfma(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tens
     positions: every tile's sequence is a row of block_table, its tokens are rows of q); None for
     a decode step, in which token i is the one token of sequence i.  nsplit > 1 cuts the keys into
     that many parts of split_len positions (a multiple of 32; nsplit * split_len must reach the
-    longest sequence) that run side by side and are merged.  col_tiles: the value the tiles were
+    longest sequence, or with a window or chunk, whose parts begin at the first block a tile sees, the
+    positions from there to the tile's last token) that run side by side and are merged.  col_tiles: the value the tiles were
     made with.  waves (a power of two up to `attention_max_waves`): so many waves of a
     workgroup share each tile's (or part's) keys and merge their results before writing.
     shared (prompt portions; col_tiles 1 or 2, head size up to 128, 4 or 8 waves): the tiles were made
@@ -2184,7 +2190,7 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
                                     _ptr(next_weight), next_code, _ptr(xg), _ptr(ssq_out), *rope_args, waves, rows_per_block,
                                     *_gate_args(gate if epilogue == "silu" else None),
                                     _ptr(act_scale if epilogue == "relu2" else None), scale_cols, block,
-                                    _ptr(rope.head_scale if epilogue == "rope" else None), _stream()), "gemm_rows")
+                                    _ptr(rope.head_scale if epilogue == "rope" else None), 1, _stream()), "gemm_rows")
     if epilogue == "rope":
         return (q_out, Product(y, 1)) if rope.extra_cols else q_out
     if epilogue == "store":
@@ -2192,6 +2198,27 @@ def gemm_rows(x, weight: torch.Tensor, bias: torch.Tensor | None, epilogue: str 
     if epilogue in ("silu", "relu2"):
         return act
     return ResidualUpdated(NormedRows(xg, ssq_out, float(next_norm[1])) if next_norm is not None else None)
+
+
+def gemm_rows_batch(x: torch.Tensor, weight: torch.Tensor) -> list[Product]:
+    """Several products of one shape for at most 16 rows in one launch: x bfloat16 [batch, M, K], weight bfloat16
+    [batch, N, K]; returns `batch` float32 products [M, N]."""
+    _device_tensor(x, "x", torch.bfloat16)
+    _device_tensor(weight, "weight", torch.bfloat16)
+    if x.dim() != 3 or weight.dim() != 3 or x.shape[0] != weight.shape[0] or x.shape[2] != weight.shape[2]:
+        raise invalid_shape(f"gemm_rows_batch: x {list(x.shape)} and weight {list(weight.shape)} do not fit")
+    batch, rows, in_features = x.shape
+    out_features = weight.shape[1]
+    if not gemm_rows_takes(rows, weight[0], x.dtype):
+        raise invalid_argument(f"gemm_rows_batch takes 1..{ROWS_MAX} rows of bfloat16 and an inner size that is a multiple of 8")
+    # (the launch has `batch` times the workgroups of one product: its shape is that of a product of as many rows of W)
+    waves, rows_per_block = gemm_rows_shape(batch * out_features, in_features, "store", _compute_units(x.device), rows)
+    y = torch.empty((batch, rows, out_features), dtype=torch.float32, device=x.device)
+    none = _ptr(None)
+    _check(library().tlie_gemm_rows(_ptr(x), _ptr(weight), none, rows, out_features, in_features, none, 0, in_features, ctypes.c_float(0.0), 0,
+                                    _ptr(y), none, none, none, BF16, none, none, none, none, none, 0, 0, 0, 0, 0, none, none, waves,
+                                    rows_per_block, *_gate_args(None), none, 0, 1, none, batch, _stream()), "gemm_rows_batch")
+    return [Product(y[index], 1) for index in range(batch)]
 
 
 def embed_rows(tokens: torch.Tensor, table: torch.Tensor, next_norm: tuple):

@@ -72,6 +72,7 @@ class Attention(Mixer):
         self.dv = int(spec.get("value_dim") or self.d)
         self.scale = float(spec["scale"]) if spec.get("scale") is not None else 1.0 / math.sqrt(float(self.d))
         self.chunk = spec.get("chunk")
+        self.reach = min((int(size) for size in (self.window, self.chunk) if size is not None), default=None)   # the most keys a token sees
         self.has_sink = bool(spec.get("sink", False))
         self.reads_other_cache = bool(spec.get("reads_other_cache", False))
         if not 0 < self.dv <= ops.ATTENTION_MAX_HEAD_DIM:
@@ -214,7 +215,7 @@ class Attention(Mixer):
                           q_temp=self.q_temp, head_scale=self.temp, extra_cols=self.gate_cols)
         if self.dv == self.d and ops.attention_mfma_takes(self.dtype, self.d, binding.cache.shape[3] // self.d):
             # bfloat16, one head size: the kernel on the matrix cores (scores, softmax and sink float)
-            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d)
+            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d, self.reach)
             attended = ops.attention_mfma(q, binding.cache, pages.block_table, tiles, ctx.positions, self.nq, self.nkv, self.d,
                                           self.window, self.scale, nsplit, split_len, col_tiles, waves, shared,
                                           chunk=self.chunk, sink=self.sink, softcap=self.softcap)
@@ -251,7 +252,7 @@ class Attention(Mixer):
                                self.dtype, paired=self.paired, extra_cols=self.gate_cols, head_scale=self.temp)
         page_size = binding.cache.shape[3] // self.d
         if ops.attention_mfma_takes(self.dtype, self.d, page_size):
-            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d)
+            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.nq // self.nkv, self.nkv, self.d, self.reach)
             attended = ops.attention_mfma(q, binding.cache, pages.block_table, tiles, ctx.positions, self.nq, self.nkv,
                                           self.d, self.window, self.scale, nsplit, split_len, col_tiles, waves, shared)
         else:

@@ -153,7 +153,7 @@ class LatentAttention(Mixer):
         q = ops.qkv_place(qkv, ctx.positions, pages.slot_map if binding.writes else ctx.no_slots, None, 0, binding.cache, self.heads,
                           self.heads, self.plain, self.dv, self.dtype)
         if self.dv == self.plain and ops.attention_mfma_takes(self.dtype, self.plain, binding.cache.shape[3] // self.plain):
-            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, 1, self.heads, self.plain)
+            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, 1, self.heads, self.plain, self.window)
             attended = ops.attention_mfma(q, binding.cache, pages.block_table, tiles, ctx.positions, self.heads, self.heads, self.plain,
                                           self.window, self.scale, nsplit, split_len, col_tiles, waves, shared, sink=self.sink)
         else:
@@ -179,7 +179,7 @@ class LatentAttention(Mixer):
                          q_wide, 0, self.heads * key, key, tokens, weight=self.up_keys_rows)
         value_dim = key if self.wide_values else self.rank
         if self.wide_values and ops.attention_mfma_takes(self.dtype, key, binding.cache.shape[-1] // key):
-            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.heads, 1, key)
+            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, self.heads, 1, key, self.window)
             attended = ops.attention_mfma(q_wide, binding.cache, pages.block_table, tiles, ctx.positions, self.heads, 1, key,
                                           self.window, self.scale, nsplit, split_len, col_tiles, waves, shared, sink=self.sink)
         else:

@@ -236,7 +236,7 @@ class TokenShiftMixing(Mixer):
         _check_sizes("token_shift_mixing", self.heads, self.d, self.d)
         self.eps = float(spec["norm_eps"])
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
-        self.blends = self.products = self.down = self.up = self.base = self.bonus = self.norm = self.o = None
+        self.blends = self.stacked = self.products = self.down = self.up = self.base = self.bonus = self.norm = self.o = None
 
     @classmethod
     def tensor_specs(cls, spec, prefix):
@@ -254,7 +254,9 @@ class TokenShiftMixing(Mixer):
         keep = partial(keep_in, weights)
         get = lambda role: weights[prefix + self.names[role]]        # noqa: E731
         self.blends = keep(torch.stack([get("shift_" + blend) for blend in self.BLENDS], dim=0).contiguous())
-        self.products = [Linear(get(role), None, self.dtype, keep=keep) for role in ("r", "k", "v", "gate")]
+        # four matrices of one shape, one after the other: a step of few rows takes their products in one launch
+        self.stacked = keep(torch.stack([get(role) for role in ("r", "k", "v", "gate")], dim=0).contiguous())
+        self.products = [Linear(matrix, None, self.dtype) for matrix in self.stacked]
         self.down = Linear(get("decay_down"), None, self.dtype, keep=keep)
         self.up = keep(get("decay_up").contiguous())
         if self.down.out_features != self.up.shape[1]:
@@ -274,7 +276,10 @@ class TokenShiftMixing(Mixer):
         scan_floats = shape[0] * shape[1] * shape[2]
         before = binding.state[:, scan_floats:]
         blended = ops.token_shift(x, self.blends, before, ctx)
-        r, k, v, gate = (ops.as_product(product(blended[index])) for index, product in enumerate(self.products))
+        if self.products[0].takes_rows(x.shape[0]):
+            r, k, v, gate = ops.gemm_rows_batch(blended[:4], self.stacked)
+        else:
+            r, k, v, gate = (ops.as_product(product(blended[index])) for index, product in enumerate(self.products))
         decay = ops.low_rank_decay(self.down(blended[4], out_dtype=torch.float32), self.up, self.base, "exp_neg_exp", inner_tanh=True)
         scanned = ops.decay_scan((r, 0), (k, 0), (v, 0), binding.state, ctx.seq_start, ctx.seq_slot, self.heads, self.d, self.d,
                                  decay=decay, bonus=self.bonus, max_new=ctx.max_new)
