@@ -143,9 +143,12 @@ class ModelSpec:
                     raise invalid_config(f"run {index} mixes the results so far with '{run.depth_mix}', which is no shared tensor [{index + 2}]")
             if run.pass_input is not None:
                 shapes = [tensor.shape for tensor in self.shared_tensors if tensor.name == run.pass_input]
-                if shapes != [(self.hidden_size, 2 * self.hidden_size)] or self.embedding.get("norm") is not None:
+                if (shapes != [(self.hidden_size, 2 * self.hidden_size)] or self.embedding.get("norm") is not None
+                        or self.embedding.get("scale", 1.0) != 1.0):
                     raise invalid_config(f"run {index} forms its residual with '{run.pass_input}', which is no shared tensor "
                                          "[hidden, 2 * hidden] (on an embedding whose output is its table's rows)")
+            if run.add_embedding and self.embedding.get("scale", 1.0) != 1.0:
+                raise invalid_config(f"run {index} takes the embedding's rows again, which goes with rows that are not scaled")
             if run.add_vector is not None:
                 name, row = run.add_vector
                 shapes = [tensor.shape for tensor in self.shared_tensors if tensor.name == name]
@@ -159,6 +162,7 @@ class TensorSpec:
     that the file gives and no configuration names (random weights draw `free_extent` there)."""
     name: str
     shape: tuple[int, ...]
-    init: str = "normal"        # how random weights draw it: "normal", "norm" (around 1), "offset" (a norm's weight stored around 0), "zeros", "forget_bias" (between 3 and 6), "fraction" (between 0 and 1), "mix" (weights of a sum: the last near 1, the others near 0), "near_identity" (a square matrix: 1 on the diagonal, small elsewhere), "share" (numbers around 1 / count), "spread" (of order 1 whatever the scale of the rest)
+    init: str = "normal"        # how random weights draw it: "normal", "norm" (around 1), "offset" (a norm's weight stored around 0), "zeros", "forget_bias" (between 3 and 6), "fraction" (between 0 and 1), "mix" (weights of a sum: the last near 1, the others near 0), "near_identity" (a square matrix: 1 on the diagonal, small elsewhere), "share" (numbers around 1 / count), "spread" (of order 1 whatever the scale of the rest), "taps" (of a short convolution), "log_rate" (the logarithm of a number between 1 and 16), "step_bias" (softplus of it lies between 0.001 and 0.1), "choice" (integers: a row's entries are distinct, below `choices`)
     free_extent: int = 16
+    choices: int = 0
     optional: bool = False       # absent is no error, present it is checked and not read (a tied head's matrix that some files still carry)

@@ -18,7 +18,8 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 SOURCES = ["elementwise.hip", "rope_cache.hip", "attention_generic.hip", "attention_mfma.hip", "gemm_generic.hip",
            "gemm_skinny.hip", "gemm_rows.hip", "gemm_tiles.hip", "sampling.hip", "library_gemm.hip", "probes.hip",
            "block_linear.hip", "latent.hip", "recurrence.hip", "heads.hip", "mlstm.hip", "routing.hip", "side.hip",
-           "decay_scan.hip", "canon.hip", "streams.hip"]
+           "decay_scan.hip", "canon.hip", "streams.hip", "short_conv.hip",
+           "gated_scan.hip", "post_norm.hip"]
 HEADERS = ["common.h", "no_alloc.h"]
 LIBRARY = "libtlie_hip.so"
 FLAGS = ["-O3", "--offload-arch=gfx950", "-std=c++17", "-fPIC", "-shared",

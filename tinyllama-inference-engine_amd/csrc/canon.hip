@@ -165,13 +165,6 @@ constexpr int kMaxTaps = 8, kConvTokens = 8;
 __device__ __forceinline__ void store1(float* p, float v) { *p = v; }
 __device__ __forceinline__ void store1(bf16* p, float v) { *p = __float2bfloat16(v); }
 
-// Four consecutive elements as floats (the address a multiple of 16 bytes for float, of 8 for bfloat16).
-__device__ __forceinline__ float4 load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
-__device__ __forceinline__ float4 load4(const bf16* p) {
-  const uint2 u = *reinterpret_cast<const uint2*>(p);
-  return make_float4(bf16_lo(u.x), bf16_hi(u.x), bf16_lo(u.y), bf16_hi(u.y));
-}
-
 // h: float [tokens, channels]; taps: [channels, ntaps], tap j weighs the input ntaps - 1 - j tokens back; state: float
 // [slots, ntaps - 1, channels] (a slot's rows `slot_stride` floats after the slot's before it), the last inputs, oldest
 // first.  Every thread owns V consecutive channels (V = 4 where the channels are a multiple of 4), blockIdx.y a stretch

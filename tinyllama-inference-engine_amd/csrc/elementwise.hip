@@ -7,15 +7,19 @@
 
 namespace tlie {
 
-// ---- embedding: residual[t, :] = table[token[t], :] as float -------------------------------
+// ---- embedding: residual[t, :] = scale * table[token[t], :] as float, and a bfloat16 copy if asked for ---------
 // reference: a row copy per token (src/model.cpp:94-97, src/cuda/model.cu:388-391)
 template <typename W>
-__global__ void embed_gather_kernel(const int* __restrict__ tokens, const W* __restrict__ table,
-                                    float* __restrict__ residual, int hidden) {
+__global__ void embed_gather_kernel(const int* __restrict__ tokens, const W* __restrict__ table, float scale,
+                                    float* __restrict__ residual, bf16* __restrict__ copy, int hidden) {
   const int t = blockIdx.x;
   const W* row = table + static_cast<size_t>(tokens[t]) * hidden;
   float* out = residual + static_cast<size_t>(t) * hidden;
-  for (int i = threadIdx.x; i < hidden; i += blockDim.x) out[i] = to_float(row[i]);
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) {
+    const float v = scale * to_float(row[i]);
+    out[i] = v;
+    if (copy != nullptr) copy[static_cast<size_t>(t) * hidden + i] = __float2bfloat16(v);
+  }
 }
 
 // ---- residual += delta (+ bias); out = RMSNorm(residual) * weight ----------------------------
@@ -322,16 +326,16 @@ __global__ void softcap_kernel(float* __restrict__ x, size_t total, float cap) {
 
 using namespace tlie;
 
-extern "C" int tlie_embed_gather(const int* tokens, const void* table, int table_dtype, float* residual,
+extern "C" int tlie_embed_gather(const int* tokens, const void* table, int table_dtype, float scale, float* residual, void* copy,
                                  int num_tokens, int hidden, void* stream) {
   if (num_tokens <= 0 || hidden <= 0) return kBadArgument;
   const int threads = hidden >= 1024 ? 256 : 64;
   if (table_dtype == kF32)
     hipLaunchKernelGGL(embed_gather_kernel<float>, dim3(num_tokens), dim3(threads), 0, (hipStream_t)stream,
-                       tokens, (const float*)table, residual, hidden);
+                       tokens, (const float*)table, scale, residual, (bf16*)copy, hidden);
   else if (table_dtype == kBF16)
     hipLaunchKernelGGL(embed_gather_kernel<bf16>, dim3(num_tokens), dim3(threads), 0, (hipStream_t)stream,
-                       tokens, (const bf16*)table, residual, hidden);
+                       tokens, (const bf16*)table, scale, residual, (bf16*)copy, hidden);
   else
     return kBadArgument;
   return launch_status();

@@ -248,13 +248,14 @@ __device__ __forceinline__ bool routed_tile(const int* __restrict__ counts, int 
 }
 
 // FIRST: the rows of x are the tokens of the expert's list, W_up[e] the rows e * N .. of w (K = w's row), and what is
-// stored is the weighed activation; else the rows of x are the pairs' own, and W_down[e] the columns e * K .. of w, whose
-// rows are experts * K long.  out: bfloat16 [pairs, N], room for `pairs` of them.  K % 64 == 0, N % 4 == 0.
+// stored is the weighed activation, s * max(y, 0)^2 or (gated: the rows of w alternate gate and up) s * silu(gate) * up,
+// half as many columns; else the rows of x are the pairs' own, and W_down[e] the columns e * K .. of w, whose
+// rows are w_row long.  out: bfloat16 [pairs, N], room for `pairs` of them.  K % 64 == 0, N % 4 == 0.
 template <bool FIRST>
 __global__ void __launch_bounds__(256, 2)
 routed_tiles_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__ w, const int* __restrict__ counts,
                     const int* __restrict__ lists, const float* __restrict__ scale, int scale_cols, uint16_t* __restrict__ out,
-                    int tokens, int experts, int pairs, int N, int K, int tiles_n) {
+                    int tokens, int experts, int pairs, int N, int K, int tiles_n, int gated, int w_row) {
   __shared__ __attribute__((aligned(16))) uint4 buffer0[2][kTilePieces];
   __shared__ __attribute__((aligned(16))) uint4 buffer1[2][kTilePieces];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -273,7 +274,7 @@ routed_tiles_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__
       from_w[i] = w + (static_cast<size_t>(tile.expert) * N + n) * K + c * 8;
       from_x[i] = x + static_cast<size_t>(list[m]) * K + c * 8;
     } else {
-      from_w[i] = w + static_cast<size_t>(n) * experts * K + static_cast<size_t>(tile.expert) * K + c * 8;
+      from_w[i] = w + static_cast<size_t>(n) * w_row + static_cast<size_t>(tile.expert) * K + c * 8;
       from_x[i] = x + static_cast<size_t>(min(tile.first_pair + m, pairs - 1)) * K + c * 8;
     }
   }
@@ -286,13 +287,19 @@ routed_tiles_kernel(const uint16_t* __restrict__ x, const uint16_t* __restrict__
     const int m = m0 + wave_m + fm * 32 + (lane & 31);
     if (m >= tile.rows || tile.first_pair + m >= pairs) continue;    // (a token with more experts than were made room for)
     const float s = FIRST ? scale[static_cast<size_t>(list[m]) * scale_cols + tile.expert] : 1.f;
-    uint16_t* to = out + static_cast<size_t>(tile.first_pair + m) * N;
+    uint16_t* to = out + static_cast<size_t>(tile.first_pair + m) * (gated ? N / 2 : N);
 #pragma unroll
     for (int fn = 0; fn < 2; ++fn)
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         const int n = n0 + wave_n + fn * 32 + g * 8 + high * 4;
         if (n >= N) continue;
+        if (FIRST && gated) {                                        // two gates with their ups
+          const float first = s * gated_value(acc[fn][fm][g * 4], acc[fn][fm][g * 4 + 1], 0, 1.f, 0.f);
+          const float second = s * gated_value(acc[fn][fm][g * 4 + 2], acc[fn][fm][g * 4 + 3], 0, 1.f, 0.f);
+          *reinterpret_cast<uint32_t*>(to + n / 2) = pack_bf16(first, second);
+          continue;
+        }
         float v[4];
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
@@ -371,10 +378,12 @@ extern "C" int tlie_route_plan(const float* scale, int scale_cols, int tokens, i
 }
 
 // counts, lists: a plan of `tokens` tokens and `experts` experts, of which a token uses at most `most`.
-// first: x [tokens, K], w [experts * N, K], scale [tokens, scale_cols]; out [tokens * most, N] gets s * max(y, 0)^2 of every pair.
-// else: x [tokens * most, K] the pairs' rows, w [N, experts * K]; out [tokens * most, N].  K % 64 == 0, N % 4 == 0.
+// first 1: x [tokens, K], w [experts * N (or more), K], scale [tokens, scale_cols]; out [tokens * most, N] gets s * max(y, 0)^2 of
+// every pair; first 2: w's rows alternate gate and up, out [tokens * most, N / 2] gets s * silu(gate) * up.
+// first 0: x [tokens * most, K] the pairs' rows, w [N, w_row], w_row at least experts * K; out [tokens * most, N].  K % 64 == 0, N % 4 == 0.
 extern "C" int tlie_routed_tiles(const void* x, const void* w, const int* counts, const int* lists, const float* scale, int scale_cols,
-                                 void* out, int tokens, int experts, int most, int N, int K, int first, void* stream) {
+                                 void* out, int tokens, int experts, int most, int N, int K, int first, int w_row, void* stream) {
+  if (first < 0 || first > 2 || (first == 0 && (w_row < experts * K || (w_row & 7) != 0))) return kBadArgument;
   if (tokens <= 0 || experts <= 0 || most <= 0 || most > experts || N <= 0 || K <= 0 || (K % kTileK) != 0 || (N & 3) != 0) return kBadArgument;
   if (x == nullptr || w == nullptr || out == nullptr || counts == nullptr || lists == nullptr || (first && (scale == nullptr || scale_cols < experts)))
     return kBadArgument;
@@ -388,10 +397,10 @@ extern "C" int tlie_routed_tiles(const void* x, const void* w, const int* counts
   hipStream_t s = (hipStream_t)stream;
   if (first)
     hipLaunchKernelGGL(routed_tiles_kernel<true>, grid, dim3(256), 0, s, (const uint16_t*)x, (const uint16_t*)w, counts, lists, scale,
-                       scale_cols, (uint16_t*)out, tokens, experts, (int)pairs, N, K, tiles_n);
+                       scale_cols, (uint16_t*)out, tokens, experts, (int)pairs, N, K, tiles_n, first == 2 ? 1 : 0, w_row);
   else
     hipLaunchKernelGGL(routed_tiles_kernel<false>, grid, dim3(256), 0, s, (const uint16_t*)x, (const uint16_t*)w, counts, lists, scale,
-                       scale_cols, (uint16_t*)out, tokens, experts, (int)pairs, N, K, tiles_n);
+                       scale_cols, (uint16_t*)out, tokens, experts, (int)pairs, N, K, tiles_n, first == 2 ? 1 : 0, w_row);
   return launch_status();
 }
 

@@ -2,7 +2,8 @@
 //   o[t, h, :]   = a[t, h, :]                                            one result a head, or
 //                = a[t, first(h), :] - lambda * a[t, second(h), :]      two maps of attention a head, combined
 //   out[t, h, e] = o[e] / sqrt(mean(o^2) + eps) * weight[h * dv + e] * mult * f(gate[t, h * dv + e])
-// f is the sigmoid (gate_kind 0) or z * sigmoid(z) (gate_kind 1); weight and gate are optional (null: 1).  Everything is float; `a` holds floats, the gate is read from a
+// f is the sigmoid (gate_kind 0) or z * sigmoid(z) (gate_kind 1); weight and gate are optional (null: 1).  With gate_first
+// the gate joins before the norm: o[e] is a[e] * f(gate[e]) (one result a head only).  Everything is float; `a` holds floats, the gate is read from a
 // product's columns (any type, possibly partial sums), out is in the activation type.
 //
 // Two maps: `a` then holds 2 * heads results a token in the order in which the attention kernel wants its
@@ -18,7 +19,7 @@ template <typename D, typename W, typename A>
 __global__ void __launch_bounds__(256)
 head_combine_kernel(const float* __restrict__ a, int heads, int dv, int pair_group, int parts, float lambda, float eps,
                     const W* __restrict__ weight, float mult, const D* __restrict__ gate, int gate_nsplit,
-                    size_t gate_split_stride, int gate_row, int gate_col, int gate_kind, A* __restrict__ out) {
+                    size_t gate_split_stride, int gate_row, int gate_col, int gate_kind, int gate_first, A* __restrict__ out) {
   const int t = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int h = blockIdx.y * 4 + wave;
   if (h >= heads) return;                              // (a whole wave; no barrier follows)
@@ -27,8 +28,15 @@ head_combine_kernel(const float* __restrict__ a, int heads, int dv, int pair_gro
   const int piece = dv / parts;
   const int g = pair_group > 0 ? h / pair_group : 0, i = pair_group > 0 ? h - g * pair_group : 0;
   const float* row = a + static_cast<size_t>(t) * (pair_group > 0 ? 2 : 1) * heads * dv;
+  auto gate_value = [&](int e) {
+    const float z = sum_splits(gate + static_cast<size_t>(t) * gate_row + gate_col + h * dv + e, gate_nsplit, gate_split_stride);
+    return (gate_kind == 1 ? z : 1.f) / (1.f + expf(-z));
+  };
   auto value = [&](int e) {
-    if (pair_group <= 0) return row[static_cast<size_t>(h) * dv + e];
+    if (pair_group <= 0) {
+      const float o = row[static_cast<size_t>(h) * dv + e];
+      return gate_first ? o * gate_value(e) : o;
+    }
     const int p = e / piece, inside = e - p * piece;
     const float first = row[((static_cast<size_t>(2 * g) * parts + p) * pair_group + i) * piece + inside];
     const float second = row[((static_cast<size_t>(2 * g + 1) * parts + p) * pair_group + i) * piece + inside];
@@ -38,10 +46,7 @@ head_combine_kernel(const float* __restrict__ a, int heads, int dv, int pair_gro
     const int c = h * dv + e;
     float v = normed * mult;
     if (weight != nullptr) v *= to_float(weight[c]);
-    if (gate != nullptr) {
-      const float z = sum_splits(gate + static_cast<size_t>(t) * gate_row + gate_col + c, gate_nsplit, gate_split_stride);
-      v *= (gate_kind == 1 ? z : 1.f) / (1.f + expf(-z));
-    }
+    if (gate != nullptr && !gate_first) v *= gate_value(e);
     out[static_cast<size_t>(t) * heads * dv + c] = from_float<A>(v);
   };
   // a lane's dims (lane, lane + 64, ...) are read once and kept, up to 512 dims a head; beyond, read again
@@ -79,25 +84,42 @@ template <typename D, typename W, typename A>
 __global__ void __launch_bounds__(256)
 head_combine_wide_kernel(const float* __restrict__ a, int heads, int dv, float eps, const W* __restrict__ weight, float mult,
                          const D* __restrict__ gate, int gate_nsplit, size_t gate_split_stride, int gate_row, int gate_col,
-                         int gate_kind, A* __restrict__ out) {
+                         int gate_kind, int gate_first, A* __restrict__ out) {
   __shared__ float scratch[16];
   constexpr int kKept = 2;
   const int t = blockIdx.x, h = blockIdx.y;
   const size_t base = (static_cast<size_t>(t) * heads + h) * dv;
   float kept[kKept][8];
   float squares = 0.f;
+  auto gates = [&](int e, float (&v)[8]) {             // v *= f(gate) of dims e .. e + 7
+    float z[8];
+    const D* from = gate + static_cast<size_t>(t) * gate_row + gate_col + h * dv + e;
+    load8(from, z);
+    for (int s = 1; s < gate_nsplit; ++s) {
+      float more[8];
+      load8(from + s * gate_split_stride, more);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) z[j] += more[j];
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) v[j] *= (gate_kind == 1 ? z[j] : 1.f) / (1.f + expf(-z[j]));
+  };
+  auto result = [&](int e, float (&v)[8]) {
+    load8(a + base + e, v);
+    if (gate_first) gates(e, v);
+  };
 #pragma unroll
   for (int i = 0; i < kKept; ++i) {
     const int e = (threadIdx.x + i * blockDim.x) * 8;
     if (e < dv) {
-      load8(a + base + e, kept[i]);
+      result(e, kept[i]);
 #pragma unroll
       for (int j = 0; j < 8; ++j) squares += kept[i][j] * kept[i][j];
     }
   }
   for (int e = (threadIdx.x + kKept * blockDim.x) * 8; e < dv; e += blockDim.x * 8) {
     float v[8];
-    load8(a + base + e, v);
+    result(e, v);
 #pragma unroll
     for (int j = 0; j < 8; ++j) squares += v[j] * v[j];
   }
@@ -112,19 +134,7 @@ head_combine_wide_kernel(const float* __restrict__ a, int heads, int dv, float e
 #pragma unroll
       for (int j = 0; j < 8; ++j) v[j] *= w[j];
     }
-    if (gate != nullptr) {
-      float z[8];
-      const D* from = gate + static_cast<size_t>(t) * gate_row + gate_col + c;
-      load8(from, z);
-      for (int s = 1; s < gate_nsplit; ++s) {
-        float more[8];
-        load8(from + s * gate_split_stride, more);
-#pragma unroll
-        for (int j = 0; j < 8; ++j) z[j] += more[j];
-      }
-#pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] *= (gate_kind == 1 ? z[j] : 1.f) / (1.f + expf(-z[j]));
-    }
+    if (gate != nullptr && !gate_first) gates(e, v);
     store8(out + base + e, v);
   };
 #pragma unroll
@@ -134,7 +144,7 @@ head_combine_wide_kernel(const float* __restrict__ a, int heads, int dv, float e
   }
   for (int e = (threadIdx.x + kKept * blockDim.x) * 8; e < dv; e += blockDim.x * 8) {
     float v[8];
-    load8(a + base + e, v);
+    result(e, v);
     emit(e, v);
   }
 }
@@ -148,10 +158,11 @@ using namespace tlie;
 extern "C" int tlie_head_combine(const float* a, int tokens, int heads, int dv, int pair_group, int parts, float lambda, float eps,
                                  const void* weight, int weight_dtype, float mult, const void* gate, int gate_dtype,
                                  int gate_nsplit, long long gate_split_stride, int gate_row, int gate_col, int gate_kind,
-                                 void* out, int out_dtype, void* stream) {
+                                 int gate_first, void* out, int out_dtype, void* stream) {
   if (tokens <= 0 || heads <= 0 || dv <= 0 || pair_group < 0 || (pair_group > 0 && heads % pair_group != 0)) return kBadArgument;
   if (parts < 1 || dv % parts != 0 || (parts > 1 && pair_group <= 0) || gate_kind < 0 || gate_kind > 1) return kBadArgument;
   if (gate != nullptr && (gate_nsplit < 1 || gate_col < 0 || gate_row < gate_col + heads * dv)) return kBadArgument;
+  if (gate_first && (gate == nullptr || pair_group > 0)) return kBadArgument;
   if (heads > 4 * 65535) return kBadArgument;
   const dim3 grid(tokens, (heads + 3) / 4);
   hipStream_t s = (hipStream_t)stream;
@@ -164,12 +175,12 @@ extern "C" int tlie_head_combine(const float* a, int tokens, int heads, int dv, 
     if (wide) {                                                                                                          \
       hipLaunchKernelGGL((head_combine_wide_kernel<D, W, A>), dim3(tokens, heads), dim3(256), 0, s, a, heads, dv, eps,    \
                          (const W*)weight, mult, (const D*)gate, gate_nsplit, (size_t)gate_split_stride, gate_row,       \
-                         gate_col, gate_kind, (A*)out);                                                                  \
+                         gate_col, gate_kind, gate_first, (A*)out);                                                                  \
       return launch_status();                                                                                            \
     }                                                                                                                    \
     hipLaunchKernelGGL((head_combine_kernel<D, W, A>), grid, dim3(256), 0, s, a, heads, dv, pair_group, parts, lambda, eps,     \
                        (const W*)weight, mult, (const D*)gate, gate_nsplit, (size_t)gate_split_stride, gate_row, gate_col, \
-                       gate_kind, (A*)out);                                                                                          \
+                       gate_kind, gate_first, (A*)out);                                                                                          \
     return launch_status();                                                                                              \
   }
   TLIE_CASE(kF32, float, kF32, float, kF32, float)

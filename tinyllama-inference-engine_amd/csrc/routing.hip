@@ -231,6 +231,24 @@ relu_squared_kernel(const D* __restrict__ up, int nsplit, size_t split_stride, c
   }
 }
 
+// A choice without a router: the token's id names its experts.  scale[t, e] = weight for the `top` experts of row ids[t] of
+// the table, 0 for the others, and 1 in the `always` columns after them (experts that every token uses).
+__global__ void __launch_bounds__(256)
+table_scale_kernel(const int* __restrict__ ids, const int* __restrict__ table, float* __restrict__ scale, int tokens, int vocab,
+                   int experts, int always, int top, float weight) {
+  const int cols = experts + always;
+  const size_t total = static_cast<size_t>(tokens) * cols;
+  for (size_t i = blockIdx.x * static_cast<size_t>(256) + threadIdx.x; i < total; i += static_cast<size_t>(gridDim.x) * 256) {
+    const int t = static_cast<int>(i / cols), e = static_cast<int>(i % cols);
+    float v = e < experts ? 0.f : 1.f;
+    const int id = ids[t];
+    if (e < experts && id >= 0 && id < vocab)
+      for (int j = 0; j < top; ++j)
+        if (table[static_cast<size_t>(id) * top + j] == e) v = weight;
+    scale[i] = v;
+  }
+}
+
 // weigh 0: the score weighs the expert's input (act(s g) * (s u)); 1: its result (s * act(g, u)).  scale_cols: columns of a
 // row of the scale matrix; shared_scaled: the columns after the experts' take scale[t, experts], not 1.  kind, alpha:
 // the gate (see gated_value); limit, shared_limit: its limit for the experts' and for the shared expert's columns.
@@ -399,4 +417,15 @@ extern "C" int tlie_relu_squared(const void* up, int in_dtype, int nsplit, long 
   TLIE_CASE(kBF16, bf16, kBF16, bf16)
 #undef TLIE_CASE
   return kBadArgument;
+}
+
+// ids: int [tokens]; table: int [vocab, top]; scale: float [tokens, experts + always].
+extern "C" int tlie_table_scale(const int* ids, const int* table, float* scale, int tokens, int vocab, int experts, int always, int top,
+                                float weight, void* stream) {
+  if (tokens <= 0 || vocab <= 0 || experts <= 0 || always < 0 || top <= 0 || ids == nullptr || table == nullptr || scale == nullptr) return kBadArgument;
+  const long long total = static_cast<long long>(tokens) * (experts + always);
+  const long long blocks = (total + 255) / 256;
+  hipLaunchKernelGGL(table_scale_kernel, dim3(static_cast<unsigned>(blocks < 4096 ? blocks : 4096)), dim3(256), 0, (hipStream_t)stream, ids,
+                     table, scale, tokens, vocab, experts, always, top, weight);
+  return launch_status();
 }

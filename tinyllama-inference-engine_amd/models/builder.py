@@ -104,9 +104,15 @@ class DecoderModel:
             return block.entry_norm() if hasattr(block, "entry_norm") else None
         first_norm = entry_norm(self.blocks[runs[0].layer]) if runs[0].pass_input is None else None
         lazy = first_norm.lazy_params() if first_norm is not None else None
-        if few and hasattr(self.embedding, "forward_rows") and lazy is not None:
+        if few and hasattr(self.embedding, "forward_rows") and lazy is not None and getattr(self.embedding, "scale", 1.0) == 1.0:
             residual, normed = self.embedding.forward_rows(ctx.tokens, lazy)
             pending = ResidualUpdated(normed)
+        elif (self.dtype == torch.bfloat16 and getattr(self.blocks[runs[0].layer], "reads_residual", False)
+                and hasattr(self.embedding, "forward_copied") and getattr(self.embedding, "norm", None) is None
+                and not runs[0].add_embedding and runs[0].add_vector is None):
+            # (the first layer's sublayers read the residual itself: its writer leaves it in their type too)
+            residual, copy = self.embedding.forward_copied(ctx.tokens)
+            pending = ResidualUpdated(copy)
         else:
             residual, pending = self.embedding.forward(ctx.tokens, ctx), None
         if trace is not None:
@@ -211,6 +217,8 @@ class DecoderModel:
         """Adds what a block handed on into the residual now (a block whose result waits for the next norm)."""
         if isinstance(pending, ops.NormedDelta):
             ops.norm_add_rmsnorm(residual, pending.product, pending.weight, pending.eps, None, pending.eps, dtype)
+        elif isinstance(pending, ops.PostNormed):
+            ops.post_norm(residual, pending)
         elif isinstance(pending, ops.ScaledSum):
             ops.layer_norm(residual, pending, None, None, 0.0, dtype, want_out=False)
         elif not isinstance(pending, ResidualUpdated):

@@ -104,7 +104,7 @@ def as_product(value) -> Product:
         return value
     if isinstance(value, torch.Tensor) and value.dim() == 2:
         return Product(value.contiguous(), 1)
-    if hasattr(value, "first_scale"):                     # a ScaledSum: added up here for whoever does not fuse it
+    if hasattr(value, "first_scale") or hasattr(value, "first_weight"):      # a ScaledSum or a NormedPair: formed here for whoever does not fuse it
         return Product(value.dense(torch.float32).contiguous(), 1)
     raise invalid_argument("a part must return a [tokens, width] tensor or a Product")
 
@@ -118,16 +118,18 @@ def _check_product(product: Product, name: str) -> None:
 
 
 # ---------------------------------------------------------------------------------------------
-def embed_gather(tokens: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
-    """float32 residual[t, :] = table[tokens[t], :].  The caller has checked 0 <= token < vocab."""
+def embed_gather(tokens: torch.Tensor, table: torch.Tensor, scale: float = 1.0, copy: bool = False):
+    """float32 residual[t, :] = scale * table[tokens[t], :].  The caller has checked 0 <= token < vocab.  copy: the rows as
+    bfloat16 too; (residual, copy) is then returned."""
     _device_tensor(tokens, "tokens", torch.int32)
     _device_tensor(table, "embedding table", (torch.float32, torch.bfloat16))
     if tokens.dim() != 1 or table.dim() != 2:
         raise invalid_shape("embed_gather takes tokens [T] and a table [vocab, hidden]")
     out = torch.empty((tokens.shape[0], table.shape[1]), dtype=torch.float32, device=table.device)
-    _check(library().tlie_embed_gather(_ptr(tokens), _ptr(table), dtype_code(table.dtype), _ptr(out),
+    rows = torch.empty(out.shape, dtype=torch.bfloat16, device=table.device) if copy else None
+    _check(library().tlie_embed_gather(_ptr(tokens), _ptr(table), dtype_code(table.dtype), ctypes.c_float(scale), _ptr(out), _ptr(rows),
                                        tokens.shape[0], table.shape[1], _stream()), "embed_gather")
-    return out
+    return (out, rows) if copy else out
 
 
 def add_rmsnorm(residual: torch.Tensor, delta: Product | None, weight: torch.Tensor, eps: float,
@@ -615,7 +617,8 @@ HEAD_GATES = {"sigmoid": 0, "silu": 1}      # what a head's gate becomes: sigmoi
 
 def head_combine(a: torch.Tensor, heads: int, value_dim: int, eps: float, out_dtype: torch.dtype, pair_group: int = 0,
                  pair_lambda: float = 0.0, weight: torch.Tensor | None = None, mult: float = 1.0,
-                 gate: Product | None = None, gate_col: int = 0, parts: int = 1, gate_kind: str = "sigmoid") -> torch.Tensor:
+                 gate: Product | None = None, gate_col: int = 0, parts: int = 1, gate_kind: str = "sigmoid",
+                 gate_first: bool = False) -> torch.Tensor:
     """Each head's result normed by itself, on its way to the output product:
     out[t, h, :] = o / sqrt(mean(o^2) + eps) * weight[h] * mult * f(gate[t, h]) (f: `gate_kind`), with o = a[t, h] or, for two maps
     of attention a head (pair_group > 0: the query heads of one key head lie side by side in `a`, pair_group of them,
@@ -623,7 +626,8 @@ def head_combine(a: torch.Tensor, heads: int, value_dim: int, eps: float, out_dt
     [tokens, heads (or 2 * heads) * value_dim]; weight (or None): [heads * value_dim]; gate (or None): a product whose
     columns gate_col .. gate_col + heads * value_dim hold the gate's pre-activations.  parts > 1 (with pair_group): a
     map's result lies in `parts` pieces of value_dim / parts dims, each a head of its own of the attention kernel: the
-    pieces of a key head's query heads follow each other piece by piece (key head, piece, query head of the key head)."""
+    pieces of a key head's query heads follow each other piece by piece (key head, piece, query head of the key head).
+    gate_first: the gate joins before the norm, o = a[t, h] * f(gate[t, h]) (one map a head)."""
     _device_tensor(a, "a", torch.float32)
     if parts < 1 or value_dim % parts != 0 or (parts > 1 and pair_group <= 0):
         raise invalid_argument("head_combine: the pieces of a result must divide the value size (and go with two maps)")
@@ -634,6 +638,8 @@ def head_combine(a: torch.Tensor, heads: int, value_dim: int, eps: float, out_dt
         raise invalid_shape("head_combine: the heads of a key head must divide the heads")
     if not eps > 0.0:
         raise EngineError(ErrorCode.NUMERICAL, "a norm requires a positive epsilon")
+    if gate_first and (gate is None or pair_group > 0):
+        raise invalid_argument("head_combine: a gate in front of the norm needs a gate, and one result a head")
     tokens = a.shape[0]
     weight_code = F32
     if weight is not None:
@@ -653,7 +659,7 @@ def head_combine(a: torch.Tensor, heads: int, value_dim: int, eps: float, out_dt
     _check(library().tlie_head_combine(_ptr(a), tokens, heads, value_dim, pair_group, int(parts), ctypes.c_float(pair_lambda),
                                        ctypes.c_float(eps), _ptr(weight), weight_code, ctypes.c_float(mult),
                                        _ptr(gate.data if gate is not None else None), gate_code, gate_nsplit,
-                                       ctypes.c_longlong(gate_stride), gate_row, gate_col, HEAD_GATES[gate_kind], _ptr(out), dtype_code(out_dtype),
+                                       ctypes.c_longlong(gate_stride), gate_row, gate_col, HEAD_GATES[gate_kind], 1 if gate_first else 0, _ptr(out), dtype_code(out_dtype),
                                        _stream()), "head_combine")
     return out
 
@@ -808,6 +814,100 @@ def layer_norm(residual: torch.Tensor, delta, weight: torch.Tensor | None, bias:
         _ptr(history_weight if history_count > 0 else None), _ptr(mixed if history_count > 0 and rows is None else None),
         _ptr(weight if want_out else None), _ptr(bias if want_out else None), w_code, ctypes.c_float(eps if want_out else 1.0),
         _ptr(out), dtype_code(out_dtype), _ptr(rows), count, hidden, _stream()), "layer_norm")
+    return out
+
+
+@dataclass
+class NormedPair:
+    """What a mixer of two sides hands on whose results are RMS-normed each by itself (weights [width], eps inside the root):
+    mult * (first / rms(first) * first_weight + second / rms(second) * second_weight), not formed yet."""
+    first: Product
+    first_weight: torch.Tensor
+    second: Product
+    second_weight: torch.Tensor
+    eps: float
+    mult: float
+
+    def dense(self, dtype: torch.dtype | None = None) -> torch.Tensor:
+        def normed(product, weight):
+            x = product.dense(torch.float32)
+            return x / torch.sqrt((x * x).mean(dim=-1, keepdim=True) + self.eps) * weight.float()
+        out = self.mult * (normed(self.first, self.first_weight) + normed(self.second, self.second_weight))
+        return out if dtype is None else out.to(dtype)
+
+
+@dataclass
+class NormParams:
+    """A norm over a row as numbers: (x - mean) / sqrt(var + eps) * weight (+ bias), or, not centred, an RMS norm."""
+    weight: torch.Tensor
+    bias: torch.Tensor | None
+    eps: float
+    centred: bool
+
+
+@dataclass
+class PostNormed:
+    """A sublayer's result (a Product, a ScaledSum without numbers a row, or a NormedPair) that is normed before it joins the
+    residual: `post_norm` norms it, adds it and leaves what reads the residual next, in one kernel."""
+    value: object
+    norm: NormParams
+
+
+def post_norm(residual: torch.Tensor, delta: PostNormed | None, out_dtype: torch.dtype | None = None, last: NormParams | None = None,
+              rows: torch.Tensor | None = None) -> torch.Tensor | None:
+    """residual += norm(delta) (all rows, in place), then out_dtype: the new residual in that type, or its norm `last`.  With
+    `rows` (int32 indices) only those rows are computed, and the residual is left as it was.  delta None: the residual as it is."""
+    _device_tensor(residual, "residual", torch.float32)
+    if residual.dim() != 2:
+        raise invalid_shape("post_norm: the residual is [tokens, hidden]")
+    tokens, hidden = residual.shape
+    first = second = side1 = side2 = None
+    s1 = s2 = mult = 1.0
+    side_eps = 0.0
+    norm = delta.norm if delta is not None else None
+    if delta is not None:
+        value = delta.value
+        if isinstance(value, NormedPair):
+            first, second, side1, side2, side_eps, mult = value.first, value.second, value.first_weight, value.second_weight, value.eps, value.mult
+        elif isinstance(value, ScaledSum) and value.row_scale is None:
+            first, second, s1, s2 = value.first, value.second, value.first_scale, value.second_scale
+        else:
+            first = as_product(value)
+    for product in (first, second):
+        if product is not None:
+            _check_product(product, "delta")
+            if (product.rows, product.cols) != (tokens, hidden):
+                raise invalid_shape(f"post_norm: delta [{product.rows}, {product.cols}] does not fit residual {list(residual.shape)}")
+    weights = [side1, side2] + [w for params in (norm, last) if params is not None for w in (params.weight, params.bias)]
+    weights = [weight for weight in weights if weight is not None]
+    for weight in weights:
+        _device_tensor(weight, "norm weight", (torch.float32, torch.bfloat16))
+        if weight.shape != (hidden,) or weight.dtype != weights[0].dtype:
+            raise invalid_shape("post_norm: weights and biases have one entry per column and one type")
+    for params in (norm, last):
+        if params is not None and not params.eps > 0.0:
+            raise EngineError(ErrorCode.NUMERICAL, "a norm requires a positive epsilon")
+    if (rows is not None or last is not None) and out_dtype is None:
+        raise invalid_argument("post_norm: rows, or a norm of the residual, without a result")
+    count = tokens
+    if rows is not None:
+        _device_tensor(rows, "rows", torch.int32)
+        count = rows.shape[0]
+    out = torch.empty((count, hidden), dtype=out_dtype, device=residual.device) if out_dtype is not None else None
+    if count == 0 or tokens == 0:
+        return out
+    first_code = dtype_code(first.data.dtype) if first is not None else F32
+    second_code = dtype_code(second.data.dtype) if second is not None else first_code
+    _check(library().tlie_post_norm(
+        _ptr(residual), _ptr(first.data if first is not None else None), first_code, first.nsplit if first is not None else 1,
+        ctypes.c_longlong(first.split_stride if first is not None else 0), ctypes.c_float(s1), _ptr(second.data if second is not None else None),
+        second_code, second.nsplit if second is not None else 1, ctypes.c_longlong(second.split_stride if second is not None else 0),
+        ctypes.c_float(s2), _ptr(side1), _ptr(side2), ctypes.c_float(side_eps), ctypes.c_float(mult), _ptr(norm.weight if norm else None),
+        _ptr(norm.bias if norm else None), ctypes.c_float(norm.eps if norm else 1.0), 1 if norm is None or norm.centred else 0,
+        _ptr(last.weight if last else None), _ptr(last.bias if last else None), ctypes.c_float(last.eps if last else 1.0),
+        1 if last is None or last.centred else 0, dtype_code(weights[0].dtype) if weights else F32, _ptr(out),
+        dtype_code(out_dtype) if out_dtype is not None else dtype_code(weights[0].dtype if weights else torch.float32),
+        _ptr(rows), count, hidden, _stream()), "post_norm")
     return out
 
 
@@ -1017,6 +1117,154 @@ def decay_scan(q: tuple[Product, int], k: tuple[Product, int], v: tuple[Product,
     return out
 
 
+SHORT_CONV_MAX_TAPS = 8
+SHORT_CONV_MAX_HEAD = 256
+_CONV_NORMS = {None: 0, "length": 1, "rms": 2}
+_CONV_TARGETS = {"out": 0, "keys": 1, "values": 2}
+
+
+@dataclass
+class ConvSegment:
+    """Channels of `short_conv` that go one way, in heads of `head` channels (for a plain stretch of channels, neither
+    normed nor turned, the heads are just pieces).  norm: None, "length" or "rms" (eps inside the root) with a weight
+    [head] that the heads share, or none; then times scale; then turned by the token's position if rotated; then to
+    columns out_col .. of the result ("out") or to the cache's "keys" or "values"."""
+    channels: int
+    head: int
+    norm: str | None = None
+    weight: torch.Tensor | None = None
+    eps: float = 0.0
+    scale: float = 1.0
+    rotated: bool = False
+    target: str = "out"
+    out_col: int = 0
+
+
+def short_conv_state_floats(channels: int, taps: int) -> int:
+    """Of a request's state: the last taps - 1 inputs, oldest first (a multiple of 4, so that what follows stays aligned)."""
+    return ((taps - 1) * channels + 3) // 4 * 4
+
+
+def short_conv(fused: Product, col: int, taps: torch.Tensor, bias: torch.Tensor | None, state: torch.Tensor | None, ctx,
+               segments: list[ConvSegment], out_cols: int, out_dtype: torch.dtype, silu: bool = False, inv_freq: torch.Tensor | None = None,
+               rot_dim: int = 0, cache: torch.Tensor | None = None, slot_map: torch.Tensor | None = None, num_kv_heads: int = 0,
+               head_dim: int = 0, value_dim: int = 0) -> torch.Tensor:
+    """A short causal convolution on the columns col .. of a product, and what becomes of its result head by head (see
+    csrc/short_conv.hip).  taps [channels, n]: tap j weighs the input n - 1 - j tokens back; bias [channels] or None; state:
+    float32 rows [slots, at least (n - 1) * channels] whose first floats are a request's last n - 1 inputs (None for one tap), read for what
+    came before the step and brought up to its last token.  The segments follow each other in the channels' order.  Returns
+    [tokens, out_cols] of out_dtype, which is the cache's type too (rows of tokens that belong to no request: zeros or unwritten)."""
+    _check_product(fused, "fused")
+    _device_tensor(taps, "taps", (torch.float32, torch.bfloat16))
+    if taps.dim() != 2 or not 1 <= taps.shape[1] <= SHORT_CONV_MAX_TAPS or not 1 <= len(segments) <= 3:
+        raise invalid_shape(f"short_conv: taps [channels, 1 to {SHORT_CONV_MAX_TAPS}] and one to three segments")
+    channels, count = taps.shape
+    tokens, sequences = fused.rows, ctx.seq_slot.shape[0]
+    if sum(segment.channels for segment in segments) != channels or col < 0 or col + channels > fused.cols:
+        raise invalid_shape("short_conv: the segments are not the channels, or these do not lie in the product")
+    if bias is not None:
+        _device_tensor(bias, "bias", taps.dtype)
+        if bias.shape != (channels,):
+            raise invalid_shape("short_conv: one bias a channel")
+    if count > 1 and (not isinstance(state, torch.Tensor) or not state.is_cuda or state.dtype != torch.float32 or state.dim() != 2
+                      or state.stride(1) != 1 or state.shape[1] < (count - 1) * channels):
+        raise invalid_shape(f"short_conv: state rows of at least {(count - 1) * channels} floats on the GPU")
+    if ctx.token_seq.shape != (tokens,) or ctx.token_slot.shape != (tokens,) or ctx.seq_start.shape != (sequences + 1,):
+        raise invalid_shape("short_conv: the step's arrays do not fit the tokens")
+    page_size = 1
+    if any(segment.target != "out" for segment in segments):
+        _device_tensor(cache, "cache", out_dtype)
+        _device_tensor(slot_map, "slot_map", torch.int32)
+        if slot_map.shape != (tokens,):
+            raise invalid_shape("short_conv: slot_map needs one entry per token")
+        page_size = _check_cache(cache, num_kv_heads, head_dim, "short_conv", value_dim, num_kv_heads)
+    if inv_freq is not None:
+        _device_tensor(inv_freq, "inv_freq", torch.float32)
+        if rot_dim % 2 != 0 or rot_dim <= 0 or inv_freq.shape != (rot_dim // 2,) or ctx.positions.shape != (tokens,):
+            raise invalid_shape("short_conv: inv_freq needs rot_dim / 2 entries, rot_dim even")
+    else:
+        rot_dim = 0
+    out = torch.empty((tokens, out_cols), dtype=out_dtype, device=fused.data.device)
+    if tokens == 0 or sequences == 0:
+        return out
+    table, weights, first = [], [], 0
+    for segment in segments:
+        if segment.weight is not None:
+            _device_tensor(segment.weight, "norm weight", torch.float32)
+            if segment.weight.shape != (segment.head,):
+                raise invalid_shape("short_conv: a norm's weight has one entry a channel of a head")
+        table += [first, segment.channels, segment.head, _CONV_NORMS[segment.norm], 1 if segment.rotated else 0,
+                  _CONV_TARGETS[segment.target], segment.out_col]
+        weights.append(segment.weight.data_ptr() if segment.weight is not None else None)
+        first += segment.channels
+    n = len(segments)
+    _check(library().tlie_short_conv(
+        _ptr(fused.data), dtype_code(fused.data.dtype), fused.nsplit, ctypes.c_longlong(fused.split_stride), fused.cols, int(col), _ptr(taps),
+        _ptr(bias), dtype_code(taps.dtype), _ptr(state if count > 1 else None), ctypes.c_longlong(state.stride(0) if count > 1 else 0),
+        _ptr(ctx.token_seq), _ptr(ctx.token_slot), _ptr(ctx.seq_start), _ptr(ctx.seq_slot), tokens, sequences, int(ctx.max_new), channels, count,
+        1 if silu else 0, n, (ctypes.c_int * (7 * n))(*table), (ctypes.c_void_p * n)(*weights),
+        (ctypes.c_float * n)(*[segment.eps for segment in segments]), (ctypes.c_float * n)(*[segment.scale for segment in segments]),
+        _ptr(ctx.positions if inv_freq is not None else None), _ptr(inv_freq), rot_dim, _ptr(out), out_cols, dtype_code(out_dtype), _ptr(cache),
+        _ptr(slot_map), num_kv_heads, head_dim, value_dim, page_size, _stream()), "short_conv")
+    return out
+
+
+GATED_SCAN_MAX_DIM = 256
+GATED_SCAN_CHUNK, GATED_SCAN_CHUNKED_FROM = 32, 24      # tokens of a chunk; tokens a sequence brings from which it is taken in chunks
+
+
+def gated_scan_state_floats(heads: int, dim: int, value_dim: int) -> int:
+    """Of a request's state: per head and tile of 64 value columns, S as [dim][64]."""
+    return heads * ((value_dim + 63) // 64) * dim * 64
+
+
+def gated_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, gates: Product, a_col: int, rate: torch.Tensor, bias: torch.Tensor,
+               state: torch.Tensor, ctx, heads: int, groups: int, dim: int, value_dim: int, b_col: int | None = None,
+               skip: torch.Tensor | None = None) -> torch.Tensor:
+    """A matrix state per head that decays by one number a token and head, over the step's tokens (see csrc/gated_scan.hip).
+    qkv: float32 [tokens, n] with q and k (groups * dim each; head h uses those of group h // (heads / groups)) and v
+    (heads * value_dim) at the named columns; gates: a product whose columns a_col .. a_col + heads hold z_a; rate, bias:
+    float32 [heads].  b_col None: S' = g S + w k v^T, o = S'^T q + skip v, with w = softplus(z_a + bias), g = exp(-exp(rate) w);
+    b_col: the delta rule, S' = g S + k u^T, u = w (v - g S^T k), o = S'^T q, with w = sigmoid(z_b), g = exp(-exp(rate)
+    softplus(z_a + bias)).  state: float32 rows [slots, floats] that begin with `gated_scan_state_floats` floats, carried for
+    sequences whose slot is not negative.  Returns float32 [tokens, heads * value_dim]."""
+    _device_tensor(qkv, "qkv", torch.float32)
+    _check_product(gates, "gates")
+    delta = b_col is not None
+    if not 0 < dim <= GATED_SCAN_MAX_DIM or heads <= 0 or groups <= 0 or heads % groups != 0 or value_dim <= 0:
+        raise invalid_argument(f"gated_scan: heads of 1 to {GATED_SCAN_MAX_DIM} query dims, a multiple of the groups")
+    for name, numbers in (("rate", rate), ("bias", bias), ("skip", skip)):
+        if numbers is not None:
+            _device_tensor(numbers, name, torch.float32)
+            if numbers.shape != (heads,):
+                raise invalid_shape(f"gated_scan: {name} has one number a head")
+    if delta and skip is not None:
+        raise invalid_argument("gated_scan: a skip goes with the additive update")
+    tokens, sequences = qkv.shape[0], ctx.seq_slot.shape[0]
+    if qkv.dim() != 2 or gates.rows != tokens or ctx.seq_start.shape != (sequences + 1,):
+        raise invalid_shape("gated_scan: one row a token, and seq_start one entry more than there are sequences")
+    for first, size, width in ((q_col, groups * dim, qkv.shape[1]), (k_col, groups * dim, qkv.shape[1]), (v_col, heads * value_dim, qkv.shape[1]),
+                               (a_col, heads, gates.cols), (b_col if delta else 0, heads, gates.cols)):
+        if first < 0 or first + size > width:
+            raise invalid_shape("gated_scan: columns that do not lie in their array")
+    if (not isinstance(state, torch.Tensor) or not state.is_cuda or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1
+            or state.shape[1] < gated_scan_state_floats(heads, dim, value_dim) or state.stride(0) % 4 != 0 or state.data_ptr() % 16 != 0):
+        raise invalid_shape("gated_scan: state rows that hold the heads' states, at multiples of 16 bytes")
+    out = torch.empty((tokens, heads * value_dim), dtype=torch.float32, device=qkv.device)
+    if tokens == 0 or sequences == 0:
+        return out
+    chunks, parts = 0, None
+    if int(ctx.max_new) >= GATED_SCAN_CHUNKED_FROM:
+        chunks = (min(int(ctx.max_new), tokens) + GATED_SCAN_CHUNK - 1) // GATED_SCAN_CHUNK
+        parts = torch.empty((sequences, chunks, heads, library().tlie_gated_scan_part_floats()), dtype=torch.float32, device=qkv.device)
+    _check(library().tlie_gated_scan(_ptr(qkv), qkv.shape[1], q_col, k_col, v_col, _ptr(gates.data), dtype_code(gates.data.dtype), gates.nsplit,
+                                     ctypes.c_longlong(gates.split_stride), gates.cols, a_col, b_col if delta else 0, _ptr(rate), _ptr(bias),
+                                     _ptr(skip), 1 if delta else 0, _ptr(state), ctypes.c_longlong(state.stride(0)), _ptr(ctx.seq_start),
+                                     _ptr(ctx.seq_slot), _ptr(out), sequences, heads, groups, dim, value_dim, chunks, _ptr(parts), _stream()),
+           "gated_scan")
+    return out
+
+
 ROUTER_SCORES = {"sigmoid": 0, "softmax_of_chosen": 1}
 
 
@@ -1140,6 +1388,19 @@ def routed_gate(gate_up: Product, scale: torch.Tensor, block: int, out_dtype: to
                                       _stream()), "routed_gate")
     return out
 
+
+def table_scale(ids: torch.Tensor, table: torch.Tensor, experts: int, always: int = 0) -> torch.Tensor:
+    """A routed feed-forward's scale matrix without a router: float32 [tokens, experts + always], 1 / top for the `top` experts
+    that row ids[t] of the table (int32 [vocab, top]) names, 0 for the others, 1 in the last `always` columns."""
+    _device_tensor(ids, "ids", torch.int32)
+    _device_tensor(table, "table", torch.int32)
+    if ids.dim() != 1 or table.dim() != 2 or experts <= 0 or always < 0 or table.shape[1] > experts:
+        raise invalid_shape("table_scale: ids [tokens], a table [vocab, top] and at least `top` experts")
+    scale = torch.empty((ids.shape[0], experts + always), dtype=torch.float32, device=ids.device)
+    if ids.shape[0] > 0:
+        _check(library().tlie_table_scale(_ptr(ids), _ptr(table), _ptr(scale), ids.shape[0], table.shape[0], experts, always, table.shape[1],
+                                          ctypes.c_float(1.0 / table.shape[1]), _stream()), "table_scale")
+    return scale
 
 
 def sigmoid_gate(values: torch.Tensor, pre: Product, col: int) -> torch.Tensor:
@@ -1496,9 +1757,9 @@ def route_plan(scale: torch.Tensor, experts: int, most: int) -> RoutePlan:
 
 
 def routed_tiles_take(up: torch.Tensor, down: torch.Tensor, experts: int) -> bool:
-    """Whether the tiles take these matrices: up [experts * size, width], down [width, experts * size]."""
+    """Whether the tiles take these matrices: up [experts * size (twice that, with gates), width], down [width, experts * size]."""
     return (up.dtype == torch.bfloat16 and down.dtype == torch.bfloat16 and up.shape[1] % 64 == 0
-            and (up.shape[0] // experts) % 64 == 0)
+            and down.shape[1] % experts == 0 and (down.shape[1] // experts) % 64 == 0)
 
 
 def routed_products_pay(rows: int, up: torch.Tensor, down: torch.Tensor, experts: int, most: int) -> bool:
@@ -1510,19 +1771,29 @@ def routed_products_pay(rows: int, up: torch.Tensor, down: torch.Tensor, experts
     return rows > SKINNY_MAX_ROWS and experts >= 2 * most and down.shape[0] % 8 == 0 and routed_tiles_take(up, down, experts)
 
 
+def routed_gated(x: torch.Tensor, gate_up: torch.Tensor, plan: RoutePlan) -> torch.Tensor:
+    """bfloat16 [tokens * most, size]: s * silu(gate) * up of every pair (see `routed_relu_squared`).  gate_up: bfloat16
+    [experts * 2 * size, width], an expert's rows alternating gate and up."""
+    return _routed_first(x, gate_up, plan, 2)
+
+
 def routed_relu_squared(x: torch.Tensor, up: torch.Tensor, plan: RoutePlan) -> torch.Tensor:
     """bfloat16 [tokens * most, size]: s * max(W_up[e] x, 0)^2 of every pair of an expert and a token that uses it, an
     expert's pairs side by side, the experts in order (what lies beyond the last pair is not written).  up: bfloat16
     [experts * size, width]; s: the token's number for the expert."""
+    return _routed_first(x, up, plan, 1)
+
+
+def _routed_first(x: torch.Tensor, w: torch.Tensor, plan: RoutePlan, kind: int) -> torch.Tensor:
     _device_tensor(x, "x", torch.bfloat16)
-    _device_tensor(up, "up", torch.bfloat16)
-    if x.dim() != 2 or up.dim() != 2 or x.shape != (plan.tokens, up.shape[1]) or up.shape[0] % plan.experts != 0:
-        raise invalid_shape(f"routed_relu_squared: x {list(x.shape)} and up {list(up.shape)} do not fit {plan.tokens} tokens and {plan.experts} experts")
-    size = up.shape[0] // plan.experts
-    out = torch.empty((plan.tokens * plan.most, size), dtype=torch.bfloat16, device=x.device)
+    _device_tensor(w, "w", torch.bfloat16)
+    if x.dim() != 2 or w.dim() != 2 or x.shape != (plan.tokens, w.shape[1]) or w.shape[0] % (plan.experts * kind) != 0:
+        raise invalid_shape(f"routed products: x {list(x.shape)} and w {list(w.shape)} do not fit {plan.tokens} tokens and {plan.experts} experts")
+    rows = w.shape[0] // plan.experts
+    out = torch.empty((plan.tokens * plan.most, rows // kind), dtype=torch.bfloat16, device=x.device)
     if plan.tokens > 0:
-        _check(library().tlie_routed_tiles(_ptr(x), _ptr(up), _ptr(plan.counts), _ptr(plan.lists), _ptr(plan.scale), plan.scale.shape[1], _ptr(out),
-                                           plan.tokens, plan.experts, plan.most, size, up.shape[1], 1, _stream()), "routed_tiles")
+        _check(library().tlie_routed_tiles(_ptr(x), _ptr(w), _ptr(plan.counts), _ptr(plan.lists), _ptr(plan.scale), plan.scale.shape[1], _ptr(out),
+                                           plan.tokens, plan.experts, plan.most, rows, w.shape[1], kind, w.shape[1], _stream()), "routed_tiles")
     return out
 
 
@@ -1537,7 +1808,7 @@ def routed_down(hidden: torch.Tensor, down: torch.Tensor, plan: RoutePlan) -> to
     out = torch.empty((hidden.shape[0], down.shape[0]), dtype=torch.bfloat16, device=hidden.device)
     if plan.tokens > 0:
         _check(library().tlie_routed_tiles(_ptr(hidden), _ptr(down), _ptr(plan.counts), _ptr(plan.lists), _ptr(None), 0, _ptr(out), plan.tokens,
-                                           plan.experts, plan.most, down.shape[0], hidden.shape[1], 0, _stream()), "routed_tiles")
+                                           plan.experts, plan.most, down.shape[0], hidden.shape[1], 0, down.shape[1], _stream()), "routed_tiles")
     return out
 
 

@@ -19,7 +19,7 @@ from ..config.spec import PartSpec, TensorSpec
 from ..errors import invalid_config
 from ..registry import lookup, register
 from ..weights.arena import keep_in
-from .base import Binding, CacheNeed, Mixer, PositionEncoding
+from .base import Binding, CacheNeed, Mixer, PositionEncoding, StateNeed
 from .linear import Linear
 
 
@@ -38,18 +38,21 @@ class Attention(Mixer):
       q_temp             (coef, every): the query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)
       values_are_keys    there is no value projection: a key head as projected, before any norm and rotation, is also
                          its value head
-      qk_norm            "whole": all of a token's query columns together, and all of its key columns together, are
+      conv               taps of a short causal convolution over time that each column of q, k and v passes on its way out
+                         of the projection (no bias), before norm and rotation; its last inputs are the layer's state
+      qk_norm            "head": every query and every key head is RMS-normed by itself (norm_eps) with a weight of head_dim
+                         entries that the heads share (q_norm, k_norm), before the rotation; "whole": all of a token's query columns together, and all of its key columns together, are
                          RMS-normed (norm_eps) with a weight of that many entries (q_norm, k_norm), before the rotation
       head_temp          a learned number per head (temp) that multiplies the head's scaled scores
       head_gate          a head's result is multiplied by sigmoid(W_g x)_h, one number a head (W_g: head_gate), before the
                          output projection
       names              the tensors' names after the prefix, by role (q, k, v, o, q_bias .. o_bias, sink, q_norm, k_norm, temp,
-                         head_gate)
+                         head_gate, q_conv, k_conv, v_conv)
     Tensors: `<prefix>{q,k,v,o}_proj.weight` (and `.bias` when bias) unless `names` says otherwise."""
     NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight",
              "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias", "o_bias": "o_proj.bias",
              "sink": "sinks", "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "temp": "temperature",
-             "head_gate": "gate.weight"}
+             "head_gate": "gate.weight", "q_conv": "q_conv.weight", "k_conv": "k_conv.weight", "v_conv": "v_conv.weight"}
 
     def __init__(self, spec: PartSpec, dtype, device):
         super().__init__(spec, dtype, device)
@@ -97,17 +100,27 @@ class Attention(Mixer):
             raise invalid_config("attention: a query temperature is (coef, every) with a positive period")
         if self.values_are_keys and (self.dv != self.d or self.reads_other_cache or self.bias):
             raise invalid_config("attention: values that are the keys have the keys' size, and the layer its own keys and no biases")
-        if self.qk_norm not in (None, "whole") or (self.qk_norm is not None and (not self.norm_eps > 0.0 or self.reads_other_cache)):
-            raise invalid_config("attention: qk_norm is \"whole\" (with a positive norm_eps, on a layer with keys of its own) or absent")
+        if self.qk_norm not in (None, "whole", "head") or (self.qk_norm is not None and (not self.norm_eps > 0.0 or self.reads_other_cache)):
+            raise invalid_config("attention: qk_norm is \"whole\" or \"head\" (with a positive norm_eps, on a layer with keys of its own) or absent")
+        # a convolution, or a norm a head, goes through the kernel that has both (a norm alone: with one tap of 1)
+        self.taps = int(spec["conv"]) if spec.get("conv") is not None else None
+        self.by_conv = self.taps is not None or self.qk_norm == "head"
+        if self.by_conv:
+            if self.taps is not None and not 1 <= self.taps <= ops.SHORT_CONV_MAX_TAPS:
+                raise invalid_config(f"attention: a short convolution has 1 to {ops.SHORT_CONV_MAX_TAPS} taps")
+            if (self.reads_other_cache or self.values_are_keys or self.qk_norm == "whole" or self.q_temp is not None or self.head_temp
+                    or self.head_gate or (self.position.rotary_table() is None and type(self.position).apply_qk is not PositionEncoding.apply_qk)):
+                raise invalid_config("attention: a convolution of q, k and v, or a norm a head, goes with keys and values of the layer's own, a "
+                                     "rotation table or no positions, and no numbers a head")
         # what the kernels that are fused for the plain case (one head size, no sink, no chunks, own keys
         # and values, scores as they are) do not take goes through the kernels for any sizes
-        self.placed = self.q_temp is not None or self.values_are_keys or self.qk_norm is not None   # options of the placement kernel alone
+        self.placed = self.q_temp is not None or self.values_are_keys or self.qk_norm is not None or self.by_conv   # options of the placement kernels alone
         self.general = (self.dv != self.d or self.has_sink or self.chunk is not None or self.reads_other_cache
                         or self.softcap is not None or self.placed)
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
         # the heads' gates are columns of the q/k/v product, after those (as many as keep its rows' starts aligned)
         self.gate_cols = (self.nq + 7) // 8 * 8 if self.head_gate else 0
-        self.qkv = self.o = self.sink = self.q_norm = self.k_norm = self.temp = None
+        self.qkv = self.o = self.sink = self.q_norm = self.k_norm = self.temp = self.conv = None
 
     @classmethod
     def tensor_specs(cls, spec, prefix):
@@ -122,7 +135,12 @@ class Attention(Mixer):
                 shapes.append(("v", (nkv * dv, hidden)))
         shapes.append(("o", (hidden, nq * dv)))
         specs = [TensorSpec(prefix + names[role], shape) for role, shape in shapes]
-        if spec.get("qk_norm") is not None:
+        if spec.get("conv") is not None:
+            rows = {"q": nq * d, "k": nkv * d, "v": nkv * dv}
+            specs += [TensorSpec(prefix + names[role + "_conv"], (rows[role], int(spec["conv"])), init="taps") for role in ("q", "k", "v")]
+        if spec.get("qk_norm") == "head":
+            specs += [TensorSpec(prefix + names[role], (d,), init="norm") for role in ("q_norm", "k_norm")]
+        elif spec.get("qk_norm") is not None:
             specs += [TensorSpec(prefix + names["q_norm"], (nq * d,), init="norm"), TensorSpec(prefix + names["k_norm"], (nkv * d,), init="norm")]
         if spec.get("bias", False):
             specs += [TensorSpec(prefix + names[role + "_bias"], (shape[0],)) for role, shape in shapes]
@@ -163,6 +181,12 @@ class Attention(Mixer):
         if self.qk_norm is not None:                       # (norms are float)
             self.q_norm = keep(weights[prefix + names["q_norm"]].float().contiguous())
             self.k_norm = keep(weights[prefix + names["k_norm"]].float().contiguous())
+        if self.by_conv:
+            if self.taps is not None:
+                self.conv = torch.cat([weights[prefix + names[role + "_conv"]] for role in ("q", "k", "v")], dim=0).to(self.qkv.weight.dtype)
+            else:
+                self.conv = torch.ones((self.qkv.out_features, 1), dtype=self.qkv.weight.dtype, device=self.device)
+            self.conv = keep(self.conv.contiguous())
 
     @property
     def graph_safe(self) -> bool:
@@ -192,6 +216,21 @@ class Attention(Mixer):
             return CacheNeed((self.nkv,), self.d + self.dv, keep)
         return CacheNeed((2, self.nkv), self.d, keep)
 
+    def state_need(self):
+        """Of a convolution: the last taps - 1 columns of q, k and v as projected, oldest first."""
+        if self.taps is None or self.taps == 1:
+            return None
+        return StateNeed((ops.short_conv_state_floats((self.nq + self.nkv) * self.d + self.nkv * self.dv, self.taps),), torch.float32)
+
+    def _place_by_conv(self, fused, ctx, pages, binding, inv_freq, rot_dim):
+        norm = "rms" if self.qk_norm == "head" else None
+        segments = [ops.ConvSegment(self.nq * self.d, self.d, norm, self.q_norm, self.norm_eps, rotated=inv_freq is not None),
+                    ops.ConvSegment(self.nkv * self.d, self.d, norm, self.k_norm, self.norm_eps, rotated=inv_freq is not None, target="keys"),
+                    ops.ConvSegment(self.nkv * self.dv, self.dv, target="values")]
+        return ops.short_conv(fused, 0, self.conv, None, binding.state if self.conv.shape[1] > 1 else None, ctx, segments, self.nq * self.d,
+                              self.dtype, inv_freq=inv_freq, rot_dim=rot_dim, cache=binding.cache,
+                              slot_map=pages.slot_map if binding.writes else ctx.no_slots, num_kv_heads=self.nkv, head_dim=self.d, value_dim=self.dv)
+
     def _forward_general(self, x, ctx, binding: Binding):
         """Any sizes and masks: the product, a kernel that rotates (if there is a rotation) and places q, k
         and v, the plain attention kernel (softmax and scores float), the output product."""
@@ -207,7 +246,9 @@ class Attention(Mixer):
             # a step of few rows, one head size, own keys and values: the product places q and writes the cache itself
             q = self.qkv(x, rope=ops.RopeTarget(ctx.positions, pages.slot_map if writes else ctx.no_slots, None, 0, binding.cache,
                                                 self.nq, self.nkv, self.d, head_scale=self.temp))
-        if q is None or isinstance(q, ops.Product):
+        if self.by_conv:
+            q = self._place_by_conv(ops.as_product(self.qkv(x)), ctx, pages, binding, inv_freq, rot_dim)
+        elif q is None or isinstance(q, ops.Product):
             fused = ops.as_product(q if q is not None else self.qkv(x))
             q = ops.qkv_place(fused, ctx.positions, pages.slot_map if writes else ctx.no_slots, inv_freq,
                           rot_dim, binding.cache, self.nq, 0 if self.reads_other_cache else self.nkv, self.d, self.dv, self.dtype,

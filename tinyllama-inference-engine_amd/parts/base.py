@@ -110,8 +110,13 @@ class Norm(Part):
 
     def add_forward(self, residual: torch.Tensor, delta, rows: torch.Tensor | None = None, lazy: bool = False):
         """Unfused default: add in place, then norm; with `rows`, norm those rows of the sum only.
-        `delta` may be a `ResidualUpdated`: then the residual already holds it; or a `NormedDelta`:
-        then its norm is applied before the add."""
+        `delta` may be a `ResidualUpdated`: then the residual already holds it; or a `NormedDelta` or a
+        `PostNormed`: then its norm is applied before the add."""
+        if isinstance(delta, _ops.PostNormed):
+            if rows is None:
+                _ops.post_norm(residual, delta)
+                return self.forward(residual)
+            return self.forward(_ops.post_norm(residual, delta, torch.float32, rows=rows))
         if isinstance(delta, ResidualUpdated):
             delta = None
         if isinstance(delta, NormedDelta):

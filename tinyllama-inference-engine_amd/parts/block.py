@@ -288,6 +288,102 @@ class SandwichNormBlock:
         return None
 
 
+@register("block", "post_norm")
+class PostNormBlock:
+    """x += norm1(mixer(x)), then, if the layer has a feed-forward, x += norm2(feed_forward(x)): the sublayers read the
+    residual itself, and what they give is normed before it joins.  The norms are the layer's mixer_norm and
+    feed_forward_norm.  The block does not add its results itself: one waits, with its norm, as an `ops.PostNormed`, and
+    the kernel that norms and adds it also leaves the new residual in the type that the next sublayer's products read."""
+    reads_residual = True         # (whoever writes the residual before the first layer may leave it in that type)
+
+    def __init__(self, layer: LayerSpec, dtype, device):
+        from ..errors import invalid_config
+        self.layer = layer
+        self.dtype = dtype
+        self.mixer_norm = lookup("norm", layer.mixer_norm.kind)(layer.mixer_norm, dtype, device)
+        self.mixer = lookup("mixer", layer.mixer.kind)(layer.mixer, dtype, device)
+        self.feed_forward = self.feed_forward_norm = None
+        if layer.feed_forward is not None:
+            self.feed_forward = lookup("feed_forward", layer.feed_forward.kind)(layer.feed_forward, dtype, device)
+            self.feed_forward_norm = lookup("norm", layer.feed_forward_norm.kind)(layer.feed_forward_norm, dtype, device)
+        for norm in (self.mixer_norm, self.feed_forward_norm):
+            if norm is not None and not hasattr(norm, "params"):
+                raise invalid_config("a post_norm layer's norms are layer norms or RMS norms")
+
+    @classmethod
+    def _parts(cls, layer: LayerSpec):
+        """(attribute, registry table) of the parts this layer has, in the order they run."""
+        parts = [("mixer", "mixer"), ("mixer_norm", "norm")]
+        if layer.feed_forward is not None:
+            parts += [("feed_forward", "feed_forward"), ("feed_forward_norm", "norm")]
+        return parts
+
+    @classmethod
+    def tensor_specs(cls, layer: LayerSpec):
+        specs = []
+        for attribute, table in cls._parts(layer):
+            part_spec = getattr(layer, attribute)
+            specs += lookup(table, part_spec.kind).tensor_specs(part_spec, layer.prefix + getattr(layer, attribute + "_place"))
+        return specs
+
+    def load(self, weights):
+        for attribute, _ in self._parts(self.layer):
+            getattr(self, attribute).load(weights, self.layer.prefix + getattr(self.layer, attribute + "_place"))
+
+    def entry_norm(self):
+        return None
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(getattr(getattr(self, attribute), "graph_safe", False) for attribute, _ in self._parts(self.layer))
+
+    def _read(self, residual, pending):
+        """The residual, brought up to date, in the type the sublayers' products read (in 32-bit: the residual itself)."""
+        if isinstance(pending, ResidualUpdated):
+            if isinstance(pending.normed, torch.Tensor):
+                return pending.normed
+            pending = None
+        wide = self.dtype == torch.float32
+        if pending is not None and not isinstance(pending, ops.PostNormed):
+            ops.layer_norm(residual, pending, None, None, 0.0, self.dtype, want_out=False)       # (what another kind of layer left)
+            pending = None
+        if pending is not None or not wide:
+            copy = ops.post_norm(residual, pending, None if wide else self.dtype)
+            return residual if wide else copy
+        return residual
+
+    def forward(self, residual, pending, ctx, binding, next_norm=None):
+        """A step that keeps a trace leaves, under `ctx.trace_prefix`, "input_norm" (what the mixer reads: the residual),
+        "attention_output" (the mixer's result before its norm), with a feed-forward "post_attention_norm" and "mlp_output"
+        alike, then "output", the residual after the layer; it brings the residual up to date itself and hands on nothing."""
+        trace = getattr(ctx, "trace", None)
+
+        def keep(name, tensor):
+            if trace is not None:
+                trace[ctx.trace_prefix + name] = tensor.float().clone()
+
+        def waiting(result, norm):
+            if not isinstance(result, (ops.NormedPair, ops.ScaledSum)):
+                result = as_product(result)
+            return ops.PostNormed(result, norm.params())
+        x = self._read(residual, pending)
+        keep("input_norm", x)
+        out = waiting(self.mixer.forward(x, ctx, binding), self.mixer_norm)
+        if trace is not None:
+            keep("attention_output", as_product(out.value).dense(torch.float32))
+        if self.feed_forward is not None:
+            x = self._read(residual, out)
+            keep("post_attention_norm", x)
+            out = waiting(self.feed_forward.forward(x, ctx), self.feed_forward_norm)
+            if trace is not None:
+                keep("mlp_output", as_product(out.value).dense(torch.float32))
+        if trace is None:
+            return out
+        ops.post_norm(residual, out)
+        keep("output", residual)
+        return None
+
+
 @register("block", "parallel")
 class ParallelBlock:
     """x += scale * (mixer(norm(x)) + feed_forward(norm(x))): one norm, whose output both sublayers read; the

@@ -1,6 +1,6 @@
 """The two ends of the model: the token embedding and the output head.
 
-reference: the embedding is a row copy, unscaled (src/model.cpp:94-97); the head is a plain
+reference: the embedding is a row copy, unscaled (src/model.cpp:94-97; a scale is an option here); the head is a plain
 product of the final norm's output with `lm_head.weight`, no bias, no scaling
 (src/model.cpp:224-225).  With tied embeddings the head's matrix is the embedding table.
 Logits are float32 whatever the activation type."""
@@ -24,11 +24,12 @@ class TokenEmbedding(Part):
     NAME = "model.embed_tokens.weight"
 
     def __init__(self, spec: PartSpec, dtype, device):
-        """spec: vocab_size, hidden_size; optionally norm (a PartSpec of a norm whose result, as floats, is the
+        """spec: vocab_size, hidden_size; optionally scale (what the table's rows are multiplied by), norm (a PartSpec of a norm whose result, as floats, is the
         embedding's output) and norm_prefix (where that norm's tensors lie: a full name's start)."""
         super().__init__(spec, dtype, device)
         self.table = None
         self.norm = None
+        self.scale = float(spec.get("scale", 1.0))
         if spec.get("norm") is not None:
             norm = spec["norm"]
             norm = PartSpec(norm.kind, {**dict(norm.params), "out": "float32"})
@@ -53,8 +54,14 @@ class TokenEmbedding(Part):
     def forward(self, tokens: torch.Tensor, ctx=None) -> torch.Tensor:
         """The float32 residual [T, H] of the step's tokens.  `ctx` is the step's context: an
         embedding that depends on more than the token (positions learned per place, say) reads it."""
-        rows = ops.embed_gather(tokens, self.table)
+        rows = ops.embed_gather(tokens, self.table, self.scale)
         return rows if self.norm is None else self.norm.forward(rows)
+
+    def forward_copied(self, tokens: torch.Tensor):
+        """The residual, and its rows in bfloat16 for a layer whose sublayers read the residual itself."""
+        if self.norm is not None:
+            raise ops.invalid_argument("a normed embedding leaves no copy of its rows")
+        return ops.embed_gather(tokens, self.table, self.scale, copy=True)
 
     def forward_rows(self, tokens: torch.Tensor, next_norm: tuple):
         """For a step of few rows: the residual and the first norm's inputs in one launch."""

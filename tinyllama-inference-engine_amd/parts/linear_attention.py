@@ -21,10 +21,11 @@ the scan (`ops.decay_scan`, csrc/decay_scan.hip):
                                the state, with a bonus per key channel for the current token; each head's result divided
                                by its root mean square, times a weight, times silu(gate), output product
 
-and `side_by_side` runs two mixers on the same input and hands on their scaled sum.
+and `side_by_side` runs two mixers on the same input and hands on their scaled sum (or the sum of their normed results).
 """
 from __future__ import annotations
 
+from dataclasses import replace
 from functools import partial
 
 import torch
@@ -290,31 +291,50 @@ class TokenShiftMixing(Mixer):
 
 @register("mixer", "side_by_side")
 class SideBySide(Mixer):
-    """Two mixers that read the same input; the result is left_scale * left + right_scale * right.
-    spec: left and right (PartSpecs of mixers), left_scale, right_scale, left_place and right_place (what their tensors'
-    names continue the prefix with).  The cache manager gives a run one cache and one state row: at most one of the
-    two keeps pages and at most one keeps state."""
+    """Two mixers that read the same input; the result is left_scale * left + right_scale * right, or, with result_norm_eps,
+    scale * (left's result RMS-normed, times a weight, + right's likewise).
+    spec: left and right (PartSpecs of mixers), left_scale and right_scale, or result_norm_eps, scale and hidden_size;
+    left_place and right_place (what their tensors' names continue the prefix with), result_norm (what the two norms' names
+    continue those with; default "result_norm.weight").  Tensors, with result_norm_eps: `<side's place><result_norm>` [hidden].
+    The cache manager gives a run one cache and one state row: at most one of the two keeps pages; when both keep state
+    (each one row of floats), left's lies first in the row and right's after it, from a multiple of four floats on."""
 
     def __init__(self, spec: PartSpec, dtype, device):
         super().__init__(spec, dtype, device)
         self.left = lookup("mixer", spec["left"].kind)(spec["left"], dtype, device)
         self.right = lookup("mixer", spec["right"].kind)(spec["right"], dtype, device)
-        self.left_scale, self.right_scale = float(spec["left_scale"]), float(spec["right_scale"])
+        self.result_eps = float(spec["result_norm_eps"]) if spec.get("result_norm_eps") is not None else None
+        if self.result_eps is None:
+            self.left_scale, self.right_scale = float(spec["left_scale"]), float(spec["right_scale"])
+        else:
+            self.scale = float(spec["scale"])
+        self.left_norm = self.right_norm = None
         if self.left.cache_need() is not None and self.right.cache_need() is not None:
             raise invalid_config("side_by_side: only one of the two mixers may keep pages")
-        if self.left.state_need() is not None and self.right.state_need() is not None:
-            raise invalid_config("side_by_side: only one of the two mixers may keep state")
+        left, right = self.left.state_need(), self.right.state_need()
+        self.split = None                         # where right's part of the state row begins, when both keep state
+        if left is not None and right is not None:
+            if len(left.shape) != 1 or len(right.shape) != 1 or left.dtype != right.dtype:
+                raise invalid_config("side_by_side: two mixers that both keep state keep a row of one type each")
+            self.split = (left.shape[0] + 3) // 4 * 4
 
     @classmethod
     def tensor_specs(cls, spec, prefix):
         specs = []
         for side in ("left", "right"):
-            specs += lookup("mixer", spec[side].kind).tensor_specs(spec[side], prefix + str(spec.get(side + "_place", side + ".")))
+            place = prefix + str(spec.get(side + "_place", side + "."))
+            specs += lookup("mixer", spec[side].kind).tensor_specs(spec[side], place)
+            if spec.get("result_norm_eps") is not None:
+                specs.append(TensorSpec(place + str(spec.get("result_norm", "result_norm.weight")), (int(spec["hidden_size"]),), init="norm"))
         return specs
 
     def load(self, weights, prefix):
         self.left.load(weights, prefix + str(self.spec.get("left_place", "left.")))
         self.right.load(weights, prefix + str(self.spec.get("right_place", "right.")))
+        if self.result_eps is not None:
+            name = str(self.spec.get("result_norm", "result_norm.weight"))
+            self.left_norm, self.right_norm = (keep_in(weights, weights[prefix + str(self.spec.get(side + "_place", side + ".")) + name].contiguous())
+                                               for side in ("left", "right"))
 
     @property
     def graph_safe(self) -> bool:
@@ -324,9 +344,17 @@ class SideBySide(Mixer):
         return self.left.cache_need() or self.right.cache_need()
 
     def state_need(self):
-        return self.left.state_need() or self.right.state_need()
+        left, right = self.left.state_need(), self.right.state_need()
+        if self.split is not None:
+            return StateNeed(((self.split + right.shape[0] + 3) // 4 * 4,), left.dtype)
+        return left or right
 
     def forward(self, x, ctx, binding: Binding, into=None):
-        left = ops.as_product(self.left.forward(x, ctx, binding))
-        right = ops.as_product(self.right.forward(x, ctx, binding))
+        sides = (binding, binding)
+        if self.split is not None:
+            sides = (replace(binding, state=binding.state[:, :self.split]), replace(binding, state=binding.state[:, self.split:]))
+        left = ops.as_product(self.left.forward(x, ctx, sides[0]))
+        right = ops.as_product(self.right.forward(x, ctx, sides[1]))
+        if self.result_eps is not None:
+            return ops.NormedPair(left, self.left_norm, right, self.right_norm, self.result_eps, self.scale)
         return ops.ScaledSum(left, self.left_scale, right, self.right_scale)

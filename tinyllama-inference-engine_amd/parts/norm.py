@@ -48,7 +48,12 @@ class RMSNorm(Norm):
         # (a reader that wants floats reads no product's input: the norm is then formed by its own kernel)
         return (self.weight, self.eps) if self.out_dtype == self.dtype else None
 
+    def params(self) -> ops.NormParams:
+        return ops.NormParams(self.weight, None, self.eps, False)
+
     def add_forward(self, residual, delta, rows=None, lazy=False):
+        if isinstance(delta, ops.PostNormed):
+            return ops.post_norm(residual, delta, self.out_dtype, last=self.params(), rows=rows)
         if isinstance(delta, ResidualUpdated):
             # the residual holds the sum already; if its writer also left this norm's inputs and the
             # reader can fold the norm into its product, nothing is launched here
@@ -107,9 +112,14 @@ class LayerNorm(Norm):
     def forward(self, residual):
         return ops.layer_norm(residual, None, self.weight, self.bias, self.eps, self.out_dtype)
 
+    def params(self) -> ops.NormParams:
+        return ops.NormParams(self.weight, self.bias, self.eps, True)
+
     def add_forward(self, residual, delta, rows=None, lazy=False, **history):
         """history: `history`, `history_count`, `history_weight`, `mixed` of `ops.layer_norm`: the norm then reads a
         weighted sum over earlier residuals in the residual's place."""
+        if isinstance(delta, ops.PostNormed) and not history:
+            return ops.post_norm(residual, delta, self.out_dtype, last=self.params(), rows=rows)
         if isinstance(delta, ResidualUpdated):
             delta = None
         if isinstance(delta, NormedDelta):

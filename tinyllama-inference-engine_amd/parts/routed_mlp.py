@@ -18,6 +18,8 @@ Other designs of the same shape, as options:
     identity                    so many outputs of the router after the experts stand for the identity: their "result" is x
                                 itself, times the weight
     activation "relu_squared"   experts without a gate, down_e(max(up_e(x), 0)^2)
+    score "table"               no router: a table of integers [vocab, top] names each token id's experts (the entries of a
+                                row differ), each of weight 1 / top
     shared_gate                 the shared expert's result is multiplied by sigmoid(w_sg . x), one number a token
 
 All experts' gate and up matrices are one matrix, their rows side by side expert by expert (g0 u0 g1 u1 ...), the
@@ -26,8 +28,10 @@ products around a gate kernel that multiplies an expert's columns by the token's
 expert that the token does not use (silu(0) * 0 adds nothing to the second product, exactly).  Since the products
 are linear, s (W x) stands for W (s x); a weight on an expert's result multiplies the columns of the second product's
 input in the result's place; and the shared expert's gate is one more row of the router's matrix, which stands outside
-the choice.  An expert without a gate has its up rows alone in the first matrix.  In a step of many tokens the
-products of such experts run over the pairs of an expert and a token that uses it (`ops.route_plan`), where that pays.  The
+the choice.  An expert without a gate has its up rows alone in the first matrix.  With a table, a shared expert whose size
+is a multiple of the experts' counts as that many experts more that every token uses with weight 1 (a sum over its inner
+columns, cut).  In a step of many tokens the
+products of experts without gates, or named by a table, run over the pairs of an expert and a token that uses it (`ops.route_plan`), where that pays.  The
 identities' weights together multiply the row x, which whoever adds the feed-forward's result into the residual adds beside it (`ops.ScaledSum`).
 """
 from __future__ import annotations
@@ -48,16 +52,16 @@ from .linear import Linear
 @register("feed_forward", "routed_mlp")
 class RoutedMLP(FeedForward):
     """spec: hidden_size, experts, top, expert_size, shared_size (0: no shared expert), score ("sigmoid",
-    "softmax_of_chosen", or "softmax_grouped" with groups, keep and identity), renormalize (the last score's weights are,
+    "softmax_of_chosen", "table" (with vocab_size), or "softmax_grouped" with groups, keep and identity), renormalize (the last score's weights are,
     the others' are not), weigh ("input" or "output"), router_bias (False), activation ("silu", "clamped_swish" with alpha,
     limit, shared_limit, or "relu_squared"), shared_gate (False), names (router, router_bias, correction, expert: a pattern
-    with {} for the expert's number, shared, shared_gate, gate, up, down).
-    Tensors: router [experts + identity, hidden] (and its bias [experts], or its correction [experts + identity]); per expert
+    with {} for the expert's number, shared, shared_gate, table, gate, up, down).
+    Tensors: table int32 [vocab, top], or router [experts + identity, hidden] (and its bias [experts], or its correction [experts + identity]); per expert
     and for the shared one gate (if the activation has one), up [size, hidden], down [hidden, size]; the shared expert's
     gate [1, hidden]."""
     graph_safe = True
     NAMES = {"router": "router.weight", "router_bias": "router.bias", "correction": "router.correction", "expert": "experts.{}.", "shared": "shared_expert.",
-             "shared_gate": "shared_expert_gate.weight", "gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
+             "shared_gate": "shared_expert_gate.weight", "table": "table", "gate": "gate_proj.weight", "up": "up_proj.weight", "down": "down_proj.weight"}
 
     def __init__(self, spec: PartSpec, dtype, device):
         super().__init__(spec, dtype, device)
@@ -72,12 +76,15 @@ class RoutedMLP(FeedForward):
         self.shared_limit = float(spec.get("shared_limit", self.limit))
         self.router_bias, self.shared_gate = bool(spec.get("router_bias", False)), bool(spec.get("shared_gate", False))
         self.grouped = self.score == "softmax_grouped"
+        self.by_table = self.score == "table"
         self.identity = int(spec.get("identity", 0))
         self.groups, self.keep_groups = int(spec.get("groups", 1)), int(spec.get("keep", 1))
-        if ((not self.grouped and self.score not in ops.ROUTER_SCORES) or self.weigh not in ("input", "output")
+        if self.by_table and (self.weigh != "output" or self.router_bias or self.shared_gate or self.activation != "silu" or int(spec["vocab_size"]) <= 0):
+            raise invalid_config("routed_mlp: a table of experts goes with SiLU gates, weights on the results, and no router's options")
+        if ((not self.grouped and not self.by_table and self.score not in ops.ROUTER_SCORES) or self.weigh not in ("input", "output")
                 or bool(spec.get("renormalize", False)) != self.grouped):
             raise invalid_config("routed_mlp: scores are sigmoids, the softmax over the chosen logits (both not renormalized) or the "
-                                 "softmax over all of them with a choice among groups (renormalized), and weigh the expert's input "
+                                 "softmax over all of them with a choice among groups (renormalized), or a table's, and weigh the expert's input "
                                  "or its output")
         if self.identity < 0 or (not self.grouped and (self.identity, self.groups, self.keep_groups) != (0, 1, 1)):
             raise invalid_config("routed_mlp: identities and groups go with the softmax over all logits")
@@ -100,7 +107,9 @@ class RoutedMLP(FeedForward):
         if self.score == "softmax_of_chosen" and self.top > 64:
             raise invalid_config("routed_mlp: the softmax over the chosen logits takes at most 64 of them")
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
-        self.router = self.router_b = self.correction = self.gate_up = self.down = None
+        # a shared expert as so many experts more that every token uses
+        self.always = self.shared_size // self.expert_size if self.by_table and self.shared_size % self.expert_size == 0 else 0
+        self.router = self.router_b = self.correction = self.gate_up = self.down = self.table = None
 
     @classmethod
     def _prefixes(cls, spec, prefix, names):
@@ -116,7 +125,10 @@ class RoutedMLP(FeedForward):
         names = {**cls.NAMES, **dict(spec.get("names") or {})}
         hidden = int(spec["hidden_size"])
         outputs, gated = int(spec["experts"]) + int(spec.get("identity", 0)), spec.get("activation", "silu") != "relu_squared"
-        specs = [TensorSpec(prefix + names["router"], (outputs, hidden))]
+        if spec.get("score", "sigmoid") == "table":
+            specs = [TensorSpec(prefix + names["table"], (int(spec["vocab_size"]), int(spec["top"])), init="choice", choices=int(spec["experts"]))]
+        else:
+            specs = [TensorSpec(prefix + names["router"], (outputs, hidden))]
         if spec.get("score", "sigmoid") == "softmax_grouped":
             specs.append(TensorSpec(prefix + names["correction"], (outputs,), init="offset"))
         if spec.get("router_bias", False):
@@ -131,17 +143,13 @@ class RoutedMLP(FeedForward):
 
     def load(self, weights, prefix):
         names, keep = self.names, partial(keep_in, weights)
-        router = weights[prefix + names["router"]]
-        bias = weights[prefix + names["router_bias"]].to(router.dtype) if self.router_bias else None
-        if self.shared_gate:
-            # the gate's row stands after the experts' rows, outside the choice (its bias: none)
-            router = torch.cat([router, weights[prefix + names["shared_gate"]].to(router.dtype).reshape(1, self.hidden)], dim=0)
-            if bias is not None:
-                bias = torch.cat([bias, torch.zeros(1, dtype=bias.dtype, device=bias.device)])
-        self.router = keep(router.contiguous())
-        self.router_b = keep(bias.contiguous()) if bias is not None else None
-        if self.grouped:                                   # (it enters the router's choice, which is float)
-            self.correction = keep(weights[prefix + names["correction"]].float().contiguous())
+        if self.by_table:
+            table = weights[prefix + names["table"]]
+            if table.dtype != torch.int32 or table.numel() == 0 or int(table.min()) < 0 or int(table.max()) >= self.experts:
+                raise invalid_config(f"routed_mlp: '{prefix}{names['table']}' must hold integers from 0 to {self.experts - 1}")
+            self.table = keep(table.contiguous())
+        else:
+            self._load_router(weights, prefix, keep)
         rows, columns = [], []
         for place, size in self._prefixes(self.spec, prefix, names):
             up = weights[place + names["up"]]
@@ -153,13 +161,39 @@ class RoutedMLP(FeedForward):
         self.gate_up = Linear(torch.cat(rows, dim=0).contiguous(), None, self.dtype, keep=keep)
         self.down = Linear(torch.cat(columns, dim=1).contiguous(), None, self.dtype, keep=keep)
 
+    def _load_router(self, weights, prefix, keep):
+        names = self.names
+        router = weights[prefix + names["router"]]
+        bias = weights[prefix + names["router_bias"]].to(router.dtype) if self.router_bias else None
+        if self.shared_gate:
+            # the gate's row stands after the experts' rows, outside the choice (its bias: none)
+            router = torch.cat([router, weights[prefix + names["shared_gate"]].to(router.dtype).reshape(1, self.hidden)], dim=0)
+            if bias is not None:
+                bias = torch.cat([bias, torch.zeros(1, dtype=bias.dtype, device=bias.device)])
+        self.router = keep(router.contiguous())
+        self.router_b = keep(bias.contiguous()) if bias is not None else None
+        if self.grouped:                                   # (it enters the router's choice, which is float)
+            self.correction = keep(weights[prefix + names["correction"]].float().contiguous())
+
     def forward(self, x, ctx, into=None):
         if self.activation == "relu_squared":
             return self._forward_ungated(x)
+        if self.by_table:
+            return self._forward_table(x, ctx)
         scale = ops.few_outputs(x, self.router, self.router_b, top=self.top, score=self.score, extra=1 if self.shared_gate else 0)
         hidden = ops.routed_gate(ops.as_product(self.gate_up(x)), scale, self.expert_size, self.dtype, weigh=self.weigh,
                                  shared_scaled=self.shared_gate, gate=self.activation, alpha=self.alpha, limit=self.limit,
                                  shared_limit=self.shared_limit)
+        return self.down(hidden)
+
+    def _forward_table(self, x, ctx):
+        scale = ops.table_scale(ctx.tokens, self.table, self.experts, self.always)
+        experts, most = self.experts + self.always, self.top + self.always
+        whole = self.always > 0 or self.shared_size == 0          # (no columns beside the experts')
+        if whole and x.dtype == torch.bfloat16 and ops.routed_products_pay(x.shape[0], self.gate_up.weight, self.down.weight, experts, most):
+            plan = ops.route_plan(scale, experts, most)
+            return ops.routed_sum(ops.routed_down(ops.routed_gated(x, self.gate_up.weight, plan), self.down.weight, plan), plan)
+        hidden = ops.routed_gate(ops.as_product(self.gate_up(x)), scale, self.expert_size, self.dtype, weigh="output")
         return self.down(hidden)
 
     def _forward_ungated(self, x):

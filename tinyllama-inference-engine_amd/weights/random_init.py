@@ -34,7 +34,10 @@ def random_tensors(specs: list[TensorSpec], seed: int, std: float = 0.02, norm_s
 
 def _draw(spec: TensorSpec, seed: int, std: float, norm_std: float, dtype: torch.dtype, device) -> torch.Tensor:
     generator = _generator(seed, spec.name, device)
-    spec = TensorSpec(spec.name, tuple(spec.free_extent if extent == -1 else extent for extent in spec.shape), spec.init)
+    spec = TensorSpec(spec.name, tuple(spec.free_extent if extent == -1 else extent for extent in spec.shape), spec.init, choices=spec.choices)
+    if spec.init == "choice":
+        drawn = torch.rand((spec.shape[0], spec.choices), generator=generator, dtype=torch.float32, device=device)
+        return drawn.argsort(dim=1)[:, :spec.shape[1]].to(torch.int32).contiguous()
     values = torch.randn(spec.shape, generator=generator, dtype=torch.float32, device=device)
     if spec.init == "normal":
         values = values * std
@@ -56,6 +59,12 @@ def _draw(spec: TensorSpec, seed: int, std: float, norm_std: float, dtype: torch
     elif spec.init == "spread":
         # numbers of order 1 whatever the other tensors' scale (a router's biases: they set the experts well apart)
         values = values * 2.0
+    elif spec.init == "taps":
+        values = values * 0.5
+    elif spec.init in ("log_rate", "step_bias"):
+        share = torch.rand(spec.shape, generator=_generator(seed, spec.name + "#", device), dtype=torch.float32, device=device)
+        # (as such mixers are commonly started: rates spread over 1 .. 16, steps over 0.001 .. 0.1 by their logarithm)
+        values = torch.log(1.0 + 15.0 * share) if spec.init == "log_rate" else torch.log(torch.expm1(0.001 * 100.0 ** share))
     elif spec.init == "near_identity":
         values = values * 0.15 + torch.eye(spec.shape[-1], device=device)
     elif spec.init == "share":
@@ -79,7 +88,7 @@ def resident_random_tensors(specs: list[TensorSpec], seed: int, std: float = 0.0
         count = 1
         for extent in spec.shape:
             count *= int(spec.free_extent if extent == -1 else extent)
-        sizes[spec.name] = count * dtype.itemsize
+        sizes[spec.name] = count * (4 if spec.init == "choice" else dtype.itemsize)
     return ResidentWeights({spec.name: draw(spec) for spec in wanted}, sizes, device)
 
 
