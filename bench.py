@@ -334,13 +334,46 @@ def paluzen_configs(sizes):
     return paluzen, llama
 
 
+# layer sizes for `--design barilix`: the same widths, feed-forwards and vocabulary; attention with Llama's heads over a window of
+# 1024 beside a state-space side of twice the width in heads of 64 (state 128, as published models of the kind have it);
+# delta-rule heads of 128 x 128 over the width, a query/key head for two; eight experts of a quarter of the feed-forward of
+# which a token uses two, beside a shared one of half of it; four layers
+BARILIX_SIZES = {
+    "w2048": dict(width=2048, ff=5632, vocab=32000, heads=32, kv_heads=4, dim=64, window=1024, taps=4, space_heads=64, space_dim=64, space_state=128,
+                  space_groups=1, delta_heads=16, delta_kv_heads=8, delta_dim=128, experts=8, top=2, expert_ff=1408, shared_ff=2816),
+    "w4096": dict(width=4096, ff=14336, vocab=32000, heads=32, kv_heads=8, dim=128, window=1024, taps=4, space_heads=128, space_dim=64, space_state=128,
+                  space_groups=8, delta_heads=32, delta_kv_heads=16, delta_dim=128, experts=8, top=2, expert_ff=3584, shared_ff=7168),
+}
+
+
+def barilix_configs(sizes):
+    """(the Barilix configuration, the Llama configuration of equal sizes): attention beside a state-space mixer with a dense
+    feed-forward, the delta rule with experts named by a table, and both with the other's feed-forward; beside four Llama layers."""
+    s = sizes
+    dense = {"kind": "dense", "ff": s["ff"]}
+    routed = {"kind": "moe", "expert": {"ff": s["expert_ff"]}, "router": {"experts": s["experts"], "top": s["top"]}, "shared": {"ff": s["shared_ff"]}}
+    side = {"left": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["dim"], "conv": s["taps"], "scale": s["dim"] ** -0.5,
+                     "mask": {"size": s["window"]}, "rot": {"base": 500000.0, "dims": s["dim"],
+                                                            "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+            "right": {"heads": s["space_heads"], "vdim": s["space_dim"], "state": s["space_state"], "groups": s["space_groups"],
+                      "norm_groups": s["space_groups"], "conv": s["taps"]}}
+    delta = {"heads": s["delta_heads"], "kv_heads": s["delta_kv_heads"], "dim": s["delta_dim"], "vdim": s["delta_dim"], "conv": s["taps"]}
+    layers = [{"type": "parallel", "mixer": side, "mlp": dense}, {"type": "delta", "mixer": delta, "mlp": routed},
+              {"type": "parallel", "mixer": side, "mlp": routed}, {"type": "delta", "mixer": delta, "mlp": dense}]
+    barilix = {"architecture": "Barilix", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-5},
+               "embedding": {"scale": s["width"] ** 0.5}, "layers": layers}
+    llama = dict(TINYLLAMA, hidden_size=s["width"], intermediate_size=s["ff"], num_hidden_layers=len(layers),
+                 num_attention_heads=s["heads"], num_key_value_heads=s["kv_heads"], vocab_size=s["vocab"], max_position_embeddings=4096)
+    return barilix, llama
+
+
 def bench_design(args, torch) -> int:
-    """`--design fadutar|raketar|tugalix|narolorn|paluzen`: one JSON line.  Per size: tokens a second of a prompt step of 2048 tokens and of decode steps
+    """`--design fadutar|raketar|tugalix|narolorn|paluzen|barilix`: one JSON line.  Per size: tokens a second of a prompt step of 2048 tokens and of decode steps
     at the record's batch and context, for that decoder and for the Llama decoder of equal sizes (random
     weights, bfloat16, through the engine's own loop), and every kernel the design adds alone, beside the like kernel."""
     from tlie_amd import Engine, ops
-    from tlie_amd.kernel_bench import (bench_design_kernels, bench_narolorn_kernels, bench_paluzen_kernels, bench_raketar_kernels,
-                                       bench_tugalix_kernels)
+    from tlie_amd.kernel_bench import (bench_barilix_kernels, bench_design_kernels, bench_narolorn_kernels, bench_paluzen_kernels,
+                                       bench_raketar_kernels, bench_tugalix_kernels)
     peaks = ops.measured_peaks("cuda:0")
     record = {"metric": f"{args.design}: prefill and decode tok/s beside the Llama decoder of equal sizes", "unit": "tokens/s",
               "n_gpus": 1, "dtype": "bf16", "data": "synthetic: uniform random token ids, random weights",
@@ -350,9 +383,10 @@ def bench_design(args, torch) -> int:
                                    "raketar": (RAKETAR_SIZES, raketar_configs, bench_raketar_kernels),
                                    "tugalix": (TUGALIX_SIZES, tugalix_configs, bench_tugalix_kernels),
                                    "narolorn": (NAROLORN_SIZES, narolorn_configs, bench_narolorn_kernels),
-                                   "paluzen": (PALUZEN_SIZES, paluzen_configs, bench_paluzen_kernels)}[args.design]
+                                   "paluzen": (PALUZEN_SIZES, paluzen_configs, bench_paluzen_kernels),
+                                   "barilix": (BARILIX_SIZES, barilix_configs, bench_barilix_kernels)}[args.design]
     for name, sizes in all_sizes.items():
-        entry = {"layers": {"fadutar": 4 * sizes.get("groups", 0), "raketar": 6, "tugalix": 4, "narolorn": 6, "paluzen": 6}[args.design], "sizes": sizes}
+        entry = {"layers": {"fadutar": 4 * sizes.get("groups", 0), "raketar": 6, "tugalix": 4, "narolorn": 6, "paluzen": 6, "barilix": 4}[args.design], "sizes": sizes}
         for model, config in zip((args.design, "llama"), configs(sizes)):
             engine = Engine(None, dtype="bfloat16", config=config, random_seed=0, max_tokens=args.batch * args.context + 4096,
                             page_size=16, max_requests=args.batch + 1)
@@ -398,7 +432,7 @@ def main() -> int:
                         help="time the kernels of a decode step (--batch, --context) and of a prompt step one by one at the "
                              "shape's layer sizes, each inside a replayed recording that walks through copies of its weights; "
                              "NAME keeps the kernels whose name holds it; prints one JSON line per kernel")
-    parser.add_argument("--design", default=None, choices=["fadutar", "raketar", "tugalix", "narolorn", "paluzen"],
+    parser.add_argument("--design", default=None, choices=["fadutar", "raketar", "tugalix", "narolorn", "paluzen", "barilix"],
                         help="prefill and decode throughput of that decoder design at layer sizes of real models, beside the Llama "
                              "decoder at equal sizes, and its own kernels alone beside the like kernels (one JSON line of its own)")
     parser.add_argument("--shape", default="tinyllama", choices=["tinyllama", *OTHER_SHAPES],

@@ -927,3 +927,186 @@ def bench_paluzen_kernels(sizes: dict, batch: int = 8, context: int = 2048, prom
         row(f"{label}: SiLU gate (Llama's)", times, tokens * lff * 6)
         del up, down, hidden
     return rows
+
+
+def bench_barilix_kernels(sizes: dict, batch: int = 8, context: int = 2048, prompt: int = 2048, samples: int = 10, device="cuda:0",
+                          hbm_gbs: float = 8000.0, mfma_tflops: float = 2500.0) -> list[dict]:
+    """The kernels that the Barilix decoder adds or runs in a new form, each alone at a layer's sizes, for a decode step of
+    `batch` requests at `context` positions and a prompt step of `prompt` tokens, each beside the like kernel of the closest
+    model (retention's scan, Fadutar's convolution, Llama's attention, rotation, add + norm, gate and products); every row
+    carries the fraction of the roofline its bytes or flops reach (`frac`: of `hbm_gbs` for rows with bytes, of
+    `mfma_tflops` for rows with flops).
+    sizes: width, ff, vocab; heads, kv_heads, dim, window, taps (the attention side); space_heads, space_dim, space_state,
+    space_groups (the side beside it); delta_heads, delta_kv_heads, delta_dim; experts, top, expert_ff, shared_ff."""
+    device = torch.device(device)
+    torch.cuda.set_device(device)
+    bf, f32 = torch.bfloat16, torch.float32
+    width, ff, vocab, taps = sizes["width"], sizes["ff"], sizes["vocab"], sizes["taps"]
+    H, G, d, window = sizes["heads"], sizes["kv_heads"], sizes["dim"], sizes["window"]
+    experts, top, eff = sizes["experts"], sizes["top"], sizes["expert_ff"]
+    always = sizes["shared_ff"] // eff
+    page_size, rows = 16, []
+
+    def rand(*shape, scale=0.02, dtype=bf):
+        return (torch.randn(shape, device=device, dtype=f32) * scale).to(dtype)
+
+    def row(name, times, read_bytes=0, flops=0):
+        entry = _row(name, times, read_bytes, flops)
+        if read_bytes:
+            entry["frac"] = round(entry["gbs"] / hbm_gbs, 3)
+        elif flops:
+            entry["frac"] = round(entry["tflops"] / mfma_tflops, 4)
+        rows.append(entry)
+
+    def ints(values):
+        return torch.tensor(values, dtype=torch.int32, device=device)
+
+    for label, tokens, seqs, keys in ((f"decode b{batch}", batch, batch, context), (f"prompt {prompt}", prompt, 1, prompt)):
+        if tokens <= 0:
+            continue
+        decode = seqs == tokens
+        blocks = (keys + page_size - 1) // page_size
+        pages = seqs * blocks
+        table = torch.arange(pages, dtype=torch.int32, device=device).view(seqs, blocks).contiguous()
+        if decode:
+            positions = torch.full((tokens,), keys - 1, dtype=torch.int32, device=device)
+            token_seq, seq_start = ints(list(range(tokens))), ints(list(range(tokens + 1)))
+            slot_map = (table[:, -1] * page_size + (keys - 1) % page_size).to(torch.int32).contiguous()
+            host = {}
+        else:
+            positions = torch.arange(tokens, dtype=torch.int32, device=device)
+            token_seq, seq_start = torch.zeros(tokens, dtype=torch.int32, device=device), ints([0, tokens])
+            slot_map = positions.clone()
+            host = {"seq_start": np.asarray([0, tokens], dtype=np.int32), "seq_len": np.asarray([keys], dtype=np.int32)}
+        seq_slot = ints(list(range(seqs)))
+        ctx = SimpleNamespace(max_new=1 if decode else tokens, num_seqs=seqs, num_tokens=tokens, max_context=keys, scratch={}, tile_owner=None,
+                              compute_units=int(torch.cuda.get_device_properties(device).multi_processor_count), host=host, tokens=positions,
+                              positions=positions, token_seq=token_seq, token_slot=seq_slot[token_seq.long()].contiguous(), seq_start=seq_start,
+                              seq_slot=seq_slot)
+        # ---- attention over a window (flops: the keys a token sees), and what places its queries, keys and values ------------
+        cache = rand(pages, 2, G, page_size * d, scale=0.5)
+        q = rand(tokens, H * d, scale=1.0)
+        for name, reach in (("causal (Llama's)", None), (f"window of {window}", window)):
+            tiles, col_tiles, nsplit, split_len, waves, shared = ops.attention_plan(ctx, H // G, G, d, reach)
+            times = _timed(lambda i: ops.attention_mfma(q, cache, table, tiles, positions, H, G, d, reach, d ** -0.5, nsplit, split_len, col_tiles,
+                                                        waves, shared), 8, samples)
+            seen = min(keys, reach or keys)
+            flops = 4.0 * H * d * sum(min(p + 1, seen) for p in range(tokens)) if not decode else 0
+            row(f"{label}: attention, {name}, {H} heads of {d} on {G}", times, seqs * seen * 2 * G * d * 2 if decode else 0, flops)
+        columns = (H + 2 * G) * d
+        qkv = ops.Product(rand(tokens, columns, scale=1.0), 1)
+        inv_freq = torch.ones(d // 2, device=device)
+        times = _timed(lambda i: ops.rope_cache(qkv, positions, slot_map, inv_freq, d, cache, H, G, d, bf, paired=True), 8, samples)
+        row(f"{label}: rotation + cache write (Llama's)", times, tokens * columns * 2 * 2)
+        held = lambda channels: torch.zeros(seqs, ops.short_conv_state_floats(channels, taps), dtype=f32, device=device)      # noqa: E731
+        conv, state, norm_d = rand(columns, taps, scale=0.5), held(columns), rand(d, scale=1.0, dtype=f32)
+        segments = [ops.ConvSegment(H * d, d, "rms", norm_d, 1e-5, rotated=True), ops.ConvSegment(G * d, d, "rms", norm_d, 1e-5, rotated=True, target="keys"),
+                    ops.ConvSegment(G * d, d, target="values")]
+        times = _timed(lambda i: ops.short_conv(qkv, 0, conv, None, state, ctx, segments, H * d, bf, inv_freq=inv_freq, rot_dim=d, cache=cache,
+                                                slot_map=slot_map, num_kv_heads=G, head_dim=d, value_dim=d), 8, samples)
+        kept = seqs * (taps - 1) * 8                            # (a request's last inputs, read and written, a column)
+        row(f"{label}: convolution, norm a head, rotation + cache write", times, tokens * columns * 2 * 2 + kept * columns)
+        # ---- convolutions in front of the scans -------------------------------------------------------------------------------
+        sh, sv, sn, sg = sizes["space_heads"], sizes["space_dim"], sizes["space_state"], sizes["space_groups"]
+        dh, dg, dd = sizes["delta_heads"], sizes["delta_kv_heads"], sizes["delta_dim"]
+        inner, space = sh * sv, sh * sv + 2 * sg * sn
+        fused = ops.Product(rand(tokens, inner + space + (sh + 7) // 8 * 8, scale=1.0), 1)
+        lru_state, lru_taps = torch.zeros(seqs, taps, space, dtype=f32, device=device), rand(space, taps, scale=0.5)
+        times = _timed(lambda i: ops.causal_conv(fused, inner, lru_taps, None, lru_state, token_seq, ctx.token_slot, seq_start), 8, samples)
+        row(f"{label}: convolution (Fadutar's, without activation and new state), {space} channels", times, tokens * space * 6 + kept // 2 * space)
+        bias, state = rand(space, scale=0.1), held(space)
+        piece = [ops.ConvSegment(inner, sn, target="heads"), ops.ConvSegment(2 * sg * sn, sn, target="heads", out_col=inner)]
+        times = _timed(lambda i: ops.short_conv(fused, inner, lru_taps, bias, state, ctx, piece, space, f32, silu=True), 8, samples)
+        row(f"{label}: convolution and silu of the state-space side, {space} channels", times, tokens * space * 6 + kept * space)
+        mixed = ops.short_conv(fused, inner, lru_taps, bias, state, ctx, piece, space, f32, silu=True)
+        keys_d, channels = dg * dd, 2 * dg * dd + dh * dd
+        delta_fused = ops.Product(rand(tokens, channels + dh * dd + (2 * dh + 7) // 8 * 8, scale=1.0), 1)
+        conv, state = rand(channels, taps, scale=0.5), held(channels)
+        segments = [ops.ConvSegment(keys_d, dd, "length", None, 1e-6, dd ** -0.5, target="heads"),
+                    ops.ConvSegment(keys_d, dd, "length", None, 1e-6, target="heads", out_col=keys_d),
+                    ops.ConvSegment(dh * dd, dd, target="heads", out_col=2 * keys_d)]
+        times = _timed(lambda i: ops.short_conv(delta_fused, 0, conv, None, state, ctx, segments, channels, f32, silu=True), 8, samples)
+        row(f"{label}: convolution, silu and unit length of the delta rule, {channels} channels", times, tokens * channels * 6 + kept * channels)
+        delta_mixed = ops.short_conv(delta_fused, 0, conv, None, state, ctx, segments, channels, f32, silu=True)
+        # ---- the scans: a token costs 4 flops an element of S (the delta rule 6) -------------------------------------------------
+        for name, heads, dim, vdim in (("state-space", sh, sn, sv), ("delta rule", dh, dd, dd)):
+            plain = ops.Product(rand(tokens, 2 * heads * dim + heads * vdim, scale=1.0), 1)
+            scan_state = torch.zeros((seqs, *ops.decay_scan_state_shape(heads, dim, vdim)), dtype=f32, device=device)
+            decay = torch.full((heads,), 0.97, dtype=f32, device=device)
+            times = _timed(lambda i: ops.decay_scan((plain, 0), (plain, heads * dim), (plain, 2 * heads * dim), scan_state, seq_start, seq_slot, heads,
+                                                    dim, vdim, head_decay=decay, max_new=ctx.max_new), 8, samples)
+            row(f"{label}: scan (retention's at these sizes), {heads} heads of {dim} x {vdim}", times, seqs * heads * dim * vdim * 8 if decode else 0,
+                0 if decode else 4.0 * tokens * heads * dim * vdim)
+            gate_state = torch.zeros(seqs, ops.gated_scan_state_floats(heads, dim, vdim), dtype=f32, device=device)
+            rate, step, skip = torch.zeros(heads, device=device), torch.full((heads,), -3.0, device=device), torch.ones(heads, device=device)
+            if name == "state-space":
+                launch = lambda i: ops.gated_scan(mixed, inner + sg * sn, inner, 0, fused, inner + space, rate, step, gate_state, ctx, sh, sg, sn, sv, skip=skip, value_width=sn)      # noqa: E731
+            else:
+                launch = lambda i: ops.gated_scan(delta_mixed, 0, keys_d, 2 * keys_d, delta_fused, channels + dh * dd, rate, step, gate_state, ctx, dh, dg, dd,      # noqa: E731
+                                                  dd, b_col=channels + dh * dd + dh)
+            row(f"{label}: scan of the {name}, {heads} heads of {dim} x {vdim}", _timed(launch, 8, samples), seqs * heads * dim * vdim * 8 if decode else 0,
+                0 if decode else (6.0 if name == "delta rule" else 4.0) * tokens * heads * dim * vdim)
+        scanned, weight = rand(tokens, inner, scale=1.0, dtype=f32), rand(inner, scale=1.0)
+        times = _timed(lambda i: ops.head_combine(scanned, sh, sv, 1e-5, bf, weight=weight, gate=fused, gate_kind="silu"), 8, samples)
+        row(f"{label}: norm, then gate, head by head (retention's)", times, tokens * inner * (4 + 2 + 2))
+        times = _timed(lambda i: ops.head_combine(scanned, sg, inner // sg, 1e-5, bf, weight=weight, gate=fused, gate_kind="silu", gate_first=True), 8, samples)
+        row(f"{label}: gate, then norm in {sg} parts", times, tokens * inner * (4 + 2 + 2))
+        # ---- around a sublayer --------------------------------------------------------------------------------------------
+        residual = rand(tokens, width, scale=1.0, dtype=f32)
+        first, second = ops.Product(rand(tokens, width, scale=1.0), 1), ops.Product(rand(tokens, width, scale=1.0), 1)
+        norm_w = rand(width, scale=1.0)
+        params = ops.NormParams(norm_w, None, 1e-5, True)
+        times = _timed(lambda i: ops.add_rmsnorm(residual, first, norm_w, 1e-5, bf), 8, samples)
+        row(f"{label}: add + norm (Llama's)", times, tokens * width * (4 + 4 + 2 + 2))
+        times = _timed(lambda i: ops.post_norm(residual, ops.PostNormed(first, params), bf), 8, samples)
+        row(f"{label}: norm of the result + add", times, tokens * width * (4 + 4 + 2 + 2))
+        pair = ops.NormedPair(first, norm_w, second, norm_w, 1e-5, 0.5)
+        times = _timed(lambda i: ops.post_norm(residual, ops.PostNormed(pair, params), bf), 8, samples)
+        row(f"{label}: norms of both sides, their sum, its norm + add", times, tokens * width * (4 + 4 + 2 + 2 + 2))
+        # ---- feed-forwards --------------------------------------------------------------------------------------------------
+        x = rand(tokens, width, scale=1.0)
+        ids = torch.randint(0, vocab, (tokens,), dtype=torch.int32, device=device)
+        named = torch.rand(vocab, experts, device=device).argsort(dim=1)[:, :top].to(torch.int32).contiguous()
+        router = rand(experts, width)
+        times = _timed(lambda i: ops.few_outputs(x, router, None, top=top, score="softmax_of_chosen"), 8, samples)
+        row(f"{label}: router, softmax over the chosen {top} of {experts} (Narolorn's)", times, (tokens + experts) * width * 2)
+        times = _timed(lambda i: ops.table_scale(ids, named, experts, always), 8, samples)
+        row(f"{label}: experts named by a table", times, tokens * (experts + always) * 4)
+        scale = ops.table_scale(ids, named, experts, always)
+        used = float((scale > 0).any(dim=0).sum())
+        pairs = tokens * (top + always)
+        from .parts.linear import Linear
+        count = 2 if not decode else _copies(width * ff * 2)
+        ups, downs = [Linear(rand(2 * ff, width), None, bf) for _ in range(count)], [Linear(rand(width, ff), None, bf) for _ in range(count)]
+        times = _timed(lambda i: ops.silu_mul(ups[i](x), bf, interleaved=True) if not decode else ups[i](x, gated=True), count, samples)
+        row(f"{label}: feed-forward's first product and gate (Llama's) [{2 * ff} x {width}]", times, width * ff * 4 if decode else 0,
+            0 if decode else 4.0 * tokens * width * ff)
+        hidden = rand(tokens, ff, scale=1.0)
+        times = _timed(lambda i: downs[i](hidden), count, samples)
+        row(f"{label}: feed-forward's second product (Llama's) [{width} x {ff}]", times, width * ff * 2 if decode else 0,
+            0 if decode else 2.0 * tokens * width * ff)
+        del ups, downs
+        total = (experts + always) * eff
+        count = 2 if not decode else _copies(width * total * 2)
+        ups, downs = [Linear(rand(2 * total, width), None, bf) for _ in range(count)], [Linear(rand(width, total), None, bf) for _ in range(count)]
+        from .parts.routed_mlp import RoutedMLP
+        part = RoutedMLP.__new__(RoutedMLP)
+        part.dtype, part.experts, part.always, part.top, part.shared_size, part.expert_size, part.table = bf, experts, always, top, sizes["shared_ff"], eff, named
+        ctx.tokens = ids
+
+        def routed(i):
+            part.gate_up, part.down = ups[i], downs[i]
+            return part._forward_table(x, ctx)
+        times = _timed(routed, count, samples)
+        row(f"{label}: experts' whole feed-forward ({experts} of {eff} and {always} for all, {top + always} a token)", times,
+            width * eff * used * 6 if decode else 0, 0 if decode else 6.0 * pairs * width * eff)
+        if ops.routed_products_pay(tokens, ups[0].weight, downs[0].weight, experts + always, top + always):
+            plan = ops.route_plan(scale, experts + always, top + always)
+            times = _timed(lambda i: ops.routed_gated(x, ups[i].weight, plan), count, samples)
+            row(f"{label}: experts' first product and gate over the pairs", times, 0, 4.0 * pairs * width * eff)
+            paired = ops.routed_gated(x, ups[0].weight, plan)
+            times = _timed(lambda i: ops.routed_down(paired, downs[i].weight, plan), count, samples)
+            row(f"{label}: experts' second product over the pairs", times, 0, 2.0 * pairs * width * eff)
+            del paired
+        del ups, downs
+    return rows

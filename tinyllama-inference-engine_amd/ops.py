@@ -1120,7 +1120,7 @@ def decay_scan(q: tuple[Product, int], k: tuple[Product, int], v: tuple[Product,
 SHORT_CONV_MAX_TAPS = 8
 SHORT_CONV_MAX_HEAD = 256
 _CONV_NORMS = {None: 0, "length": 1, "rms": 2}
-_CONV_TARGETS = {"out": 0, "keys": 1, "values": 2}
+_CONV_TARGETS = {"out": 0, "keys": 1, "values": 2, "heads": 3}
 
 
 @dataclass
@@ -1128,7 +1128,9 @@ class ConvSegment:
     """Channels of `short_conv` that go one way, in heads of `head` channels (for a plain stretch of channels, neither
     normed nor turned, the heads are just pieces).  norm: None, "length" or "rms" (eps inside the root) with a weight
     [head] that the heads share, or none; then times scale; then turned by the token's position if rotated; then to
-    columns out_col .. of the result ("out") or to the cache's "keys" or "values"."""
+    columns out_col .. of the result ("out"), to the cache's "keys" or "values", or, "heads", to the result head by head: the
+    head of the channels c .. c + head - 1 (counted from out_col on) as a plane [rows, head] at c * rows, rows those of
+    `plane_rows`."""
     channels: int
     head: int
     norm: str | None = None
@@ -1138,6 +1140,12 @@ class ConvSegment:
     rotated: bool = False
     target: str = "out"
     out_col: int = 0
+
+
+def plane_rows(tokens: int) -> int:
+    """Rows of a head's plane for a step of so many tokens: a few more where there are many, so that the heads' planes do not all
+    begin in the same memory channel."""
+    return tokens + 8 if tokens >= 64 else tokens
 
 
 def short_conv_state_floats(channels: int, taps: int) -> int:
@@ -1153,7 +1161,7 @@ def short_conv(fused: Product, col: int, taps: torch.Tensor, bias: torch.Tensor 
     csrc/short_conv.hip).  taps [channels, n]: tap j weighs the input n - 1 - j tokens back; bias [channels] or None; state:
     float32 rows [slots, at least (n - 1) * channels] whose first floats are a request's last n - 1 inputs (None for one tap), read for what
     came before the step and brought up to its last token.  The segments follow each other in the channels' order.  Returns
-    [tokens, out_cols] of out_dtype, which is the cache's type too (rows of tokens that belong to no request: zeros or unwritten)."""
+    [tokens, out_cols] of out_dtype (with "heads": [plane_rows(tokens), out_cols] values laid out so), which is the cache's type too (rows of tokens that belong to no request: zeros or unwritten)."""
     _check_product(fused, "fused")
     _device_tensor(taps, "taps", (torch.float32, torch.bfloat16))
     if taps.dim() != 2 or not 1 <= taps.shape[1] <= SHORT_CONV_MAX_TAPS or not 1 <= len(segments) <= 3:
@@ -1172,7 +1180,7 @@ def short_conv(fused: Product, col: int, taps: torch.Tensor, bias: torch.Tensor 
     if ctx.token_seq.shape != (tokens,) or ctx.token_slot.shape != (tokens,) or ctx.seq_start.shape != (sequences + 1,):
         raise invalid_shape("short_conv: the step's arrays do not fit the tokens")
     page_size = 1
-    if any(segment.target != "out" for segment in segments):
+    if any(segment.target in ("keys", "values") for segment in segments):
         _device_tensor(cache, "cache", out_dtype)
         _device_tensor(slot_map, "slot_map", torch.int32)
         if slot_map.shape != (tokens,):
@@ -1184,7 +1192,11 @@ def short_conv(fused: Product, col: int, taps: torch.Tensor, bias: torch.Tensor 
             raise invalid_shape("short_conv: inv_freq needs rot_dim / 2 entries, rot_dim even")
     else:
         rot_dim = 0
-    out = torch.empty((tokens, out_cols), dtype=out_dtype, device=fused.data.device)
+    by_head = any(segment.target == "heads" for segment in segments)
+    if by_head and any(segment.target == "out" for segment in segments):
+        raise invalid_argument("short_conv: the result is laid out token by token or head by head, not both")
+    rows = plane_rows(tokens) if by_head else tokens
+    out = torch.empty((rows, out_cols), dtype=out_dtype, device=fused.data.device)
     if tokens == 0 or sequences == 0:
         return out
     table, weights, first = [], [], 0
@@ -1204,7 +1216,7 @@ def short_conv(fused: Product, col: int, taps: torch.Tensor, bias: torch.Tensor 
         _ptr(ctx.token_seq), _ptr(ctx.token_slot), _ptr(ctx.seq_start), _ptr(ctx.seq_slot), tokens, sequences, int(ctx.max_new), channels, count,
         1 if silu else 0, n, (ctypes.c_int * (7 * n))(*table), (ctypes.c_void_p * n)(*weights),
         (ctypes.c_float * n)(*[segment.eps for segment in segments]), (ctypes.c_float * n)(*[segment.scale for segment in segments]),
-        _ptr(ctx.positions if inv_freq is not None else None), _ptr(inv_freq), rot_dim, _ptr(out), out_cols, dtype_code(out_dtype), _ptr(cache),
+        _ptr(ctx.positions if inv_freq is not None else None), _ptr(inv_freq), rot_dim, _ptr(out), out_cols, rows, dtype_code(out_dtype), _ptr(cache),
         _ptr(slot_map), num_kv_heads, head_dim, value_dim, page_size, _stream()), "short_conv")
     return out
 
@@ -1218,18 +1230,20 @@ def gated_scan_state_floats(heads: int, dim: int, value_dim: int) -> int:
     return heads * ((value_dim + 63) // 64) * dim * 64
 
 
-def gated_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, gates: Product, a_col: int, rate: torch.Tensor, bias: torch.Tensor,
+def gated_scan(planes: torch.Tensor, q_first: int, k_first: int, v_first: int, gates: Product, a_col: int, rate: torch.Tensor, bias: torch.Tensor,
                state: torch.Tensor, ctx, heads: int, groups: int, dim: int, value_dim: int, b_col: int | None = None,
-               skip: torch.Tensor | None = None) -> torch.Tensor:
+               skip: torch.Tensor | None = None, value_width: int | None = None) -> torch.Tensor:
     """A matrix state per head that decays by one number a token and head, over the step's tokens (see csrc/gated_scan.hip).
-    qkv: float32 [tokens, n] with q and k (groups * dim each; head h uses those of group h // (heads / groups)) and v
-    (heads * value_dim) at the named columns; gates: a product whose columns a_col .. a_col + heads hold z_a; rate, bias:
+    planes: float32 [plane_rows(tokens), channels] values of q and k (groups * dim channels each; head h uses those of group
+    h // (heads / groups)) and v (heads * value_dim) from the named channels on, laid out head by head as the "heads" of
+    `short_conv` are, v in planes of value_width (default value_dim); gates: a product whose columns a_col .. a_col + heads hold z_a; rate, bias:
     float32 [heads].  b_col None: S' = g S + w k v^T, o = S'^T q + skip v, with w = softplus(z_a + bias), g = exp(-exp(rate) w);
     b_col: the delta rule, S' = g S + k u^T, u = w (v - g S^T k), o = S'^T q, with w = sigmoid(z_b), g = exp(-exp(rate)
     softplus(z_a + bias)).  state: float32 rows [slots, floats] that begin with `gated_scan_state_floats` floats, carried for
     sequences whose slot is not negative.  Returns float32 [tokens, heads * value_dim]."""
-    _device_tensor(qkv, "qkv", torch.float32)
+    _device_tensor(planes, "planes", torch.float32)
     _check_product(gates, "gates")
+    value_width = value_dim if value_width is None else int(value_width)
     delta = b_col is not None
     if not 0 < dim <= GATED_SCAN_MAX_DIM or heads <= 0 or groups <= 0 or heads % groups != 0 or value_dim <= 0:
         raise invalid_argument(f"gated_scan: heads of 1 to {GATED_SCAN_MAX_DIM} query dims, a multiple of the groups")
@@ -1240,24 +1254,24 @@ def gated_scan(qkv: torch.Tensor, q_col: int, k_col: int, v_col: int, gates: Pro
                 raise invalid_shape(f"gated_scan: {name} has one number a head")
     if delta and skip is not None:
         raise invalid_argument("gated_scan: a skip goes with the additive update")
-    tokens, sequences = qkv.shape[0], ctx.seq_slot.shape[0]
-    if qkv.dim() != 2 or gates.rows != tokens or ctx.seq_start.shape != (sequences + 1,):
+    tokens, sequences = gates.rows, ctx.seq_slot.shape[0]
+    if planes.dim() != 2 or value_width <= 0 or (heads * value_dim) % value_width != 0 or planes.shape[0] != plane_rows(tokens) or ctx.seq_start.shape != (sequences + 1,):
         raise invalid_shape("gated_scan: one row a token, and seq_start one entry more than there are sequences")
-    for first, size, width in ((q_col, groups * dim, qkv.shape[1]), (k_col, groups * dim, qkv.shape[1]), (v_col, heads * value_dim, qkv.shape[1]),
+    for first, size, width in ((q_first, groups * dim, planes.shape[1]), (k_first, groups * dim, planes.shape[1]), (v_first, heads * value_dim, planes.shape[1]),
                                (a_col, heads, gates.cols), (b_col if delta else 0, heads, gates.cols)):
         if first < 0 or first + size > width:
             raise invalid_shape("gated_scan: columns that do not lie in their array")
     if (not isinstance(state, torch.Tensor) or not state.is_cuda or state.dtype != torch.float32 or state.dim() != 2 or state.stride(1) != 1
             or state.shape[1] < gated_scan_state_floats(heads, dim, value_dim) or state.stride(0) % 4 != 0 or state.data_ptr() % 16 != 0):
         raise invalid_shape("gated_scan: state rows that hold the heads' states, at multiples of 16 bytes")
-    out = torch.empty((tokens, heads * value_dim), dtype=torch.float32, device=qkv.device)
+    out = torch.empty((tokens, heads * value_dim), dtype=torch.float32, device=planes.device)
     if tokens == 0 or sequences == 0:
         return out
     chunks, parts = 0, None
     if int(ctx.max_new) >= GATED_SCAN_CHUNKED_FROM:
         chunks = (min(int(ctx.max_new), tokens) + GATED_SCAN_CHUNK - 1) // GATED_SCAN_CHUNK
-        parts = torch.empty((sequences, chunks, heads, library().tlie_gated_scan_part_floats()), dtype=torch.float32, device=qkv.device)
-    _check(library().tlie_gated_scan(_ptr(qkv), qkv.shape[1], q_col, k_col, v_col, _ptr(gates.data), dtype_code(gates.data.dtype), gates.nsplit,
+        parts = torch.empty((sequences, chunks, heads, library().tlie_gated_scan_part_floats()), dtype=torch.float32, device=planes.device)
+    _check(library().tlie_gated_scan(_ptr(planes), planes.shape[0], planes.shape[1], q_first, k_first, v_first, value_width, _ptr(gates.data), dtype_code(gates.data.dtype), gates.nsplit,
                                      ctypes.c_longlong(gates.split_stride), gates.cols, a_col, b_col if delta else 0, _ptr(rate), _ptr(bias),
                                      _ptr(skip), 1 if delta else 0, _ptr(state), ctypes.c_longlong(state.stride(0)), _ptr(ctx.seq_start),
                                      _ptr(ctx.seq_slot), _ptr(out), sequences, heads, groups, dim, value_dim, chunks, _ptr(parts), _stream()),

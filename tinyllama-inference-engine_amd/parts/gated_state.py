@@ -36,6 +36,13 @@ def _padded(rows: torch.Tensor) -> torch.Tensor:
     return rows.contiguous() if more == 0 else torch.cat([rows, rows.new_zeros(more, rows.shape[1])], dim=0)
 
 
+def _value_width(value_dim: int) -> int:
+    """The values' planes on their way into the scan: a head's columns, or equal pieces of them where the convolution's kernel
+    takes no head so wide."""
+    pieces = next(count for count in range(1, value_dim + 1) if value_dim % count == 0 and value_dim // count <= ops.SHORT_CONV_MAX_HEAD)
+    return value_dim // pieces
+
+
 def _check_taps(kind, taps):
     if not 1 <= taps <= ops.SHORT_CONV_MAX_TAPS:
         raise invalid_config(f"{kind}: a short convolution has 1 to {ops.SHORT_CONV_MAX_TAPS} taps")
@@ -64,6 +71,8 @@ class StateSpace(Mixer):
             raise invalid_config(f"state_space: state_size {self.d} is beyond what the scan keeps in registers ({ops.GATED_SCAN_MAX_DIM})")
         _check_taps("state_space", self.taps)
         self.channels = self.inner + 2 * self.groups * self.d
+        # (planes as wide as those of B and C, where they go into the values evenly, leave the convolution no lane without work)
+        self.value_width = self.d if self.inner % self.d == 0 else _value_width(self.dv)
         self.scan_floats = ops.gated_scan_state_floats(self.heads, self.d, self.dv)
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
         self.first = self.o = self.conv = self.conv_bias = self.dt_bias = self.rate = self.skip = self.norm = None
@@ -97,13 +106,14 @@ class StateSpace(Mixer):
 
     def forward(self, x, ctx, binding: Binding, into=None):
         fused = ops.as_product(self.first(x))
-        piece = min(self.channels, ops.SHORT_CONV_MAX_HEAD)
-        mixed = ops.short_conv(fused, self.inner, self.conv, self.conv_bias, binding.state[:, self.scan_floats:], ctx,
-                               [ops.ConvSegment(self.channels, piece)], self.channels, torch.float32, silu=True)
-        b_col = self.inner
-        c_col = b_col + self.groups * self.d
-        scanned = ops.gated_scan(mixed, c_col, b_col, 0, fused, self.inner + self.channels, self.rate, self.dt_bias, binding.state, ctx,
-                                 self.heads, self.groups, self.d, self.dv, skip=self.skip)
+        b_first = self.inner
+        c_first = b_first + self.groups * self.d
+        segments = [ops.ConvSegment(self.inner, self.value_width, target="heads"),
+                    ops.ConvSegment(2 * self.groups * self.d, self.d, target="heads", out_col=b_first)]
+        mixed = ops.short_conv(fused, self.inner, self.conv, self.conv_bias, binding.state[:, self.scan_floats:], ctx, segments, self.channels,
+                               torch.float32, silu=True)
+        scanned = ops.gated_scan(mixed, c_first, b_first, 0, fused, self.inner + self.channels, self.rate, self.dt_bias, binding.state, ctx,
+                                 self.heads, self.groups, self.d, self.dv, skip=self.skip, value_width=self.value_width)
         normed = ops.head_combine(scanned, self.parts, self.inner // self.parts, self.eps, self.dtype, weight=self.norm, gate=fused, gate_col=0,
                                   gate_kind="silu", gate_first=True)
         return self.o(normed)
@@ -135,6 +145,7 @@ class GatedDelta(Mixer):
         _check_taps("gated_delta", self.taps)
         self.keys, self.values = self.groups * self.d, self.heads * self.dv
         self.channels = 2 * self.keys + self.values
+        self.value_width = _value_width(self.dv)
         self.scan_floats = ops.gated_scan_state_floats(self.heads, self.d, self.dv)
         self.names = {**self.NAMES, **dict(spec.get("names") or {})}
         self.first = self.o = self.conv = self.decay_bias = self.rate = self.norm = None
@@ -166,15 +177,14 @@ class GatedDelta(Mixer):
 
     def forward(self, x, ctx, binding: Binding, into=None):
         fused = ops.as_product(self.first(x))
-        piece = min(self.values, ops.SHORT_CONV_MAX_HEAD)
-        segments = [ops.ConvSegment(self.keys, self.d, "length", None, self.UNIT_EPS, float(self.d) ** -0.5),
-                    ops.ConvSegment(self.keys, self.d, "length", None, self.UNIT_EPS, out_col=self.keys),
-                    ops.ConvSegment(self.values, piece, out_col=2 * self.keys)]
+        segments = [ops.ConvSegment(self.keys, self.d, "length", None, self.UNIT_EPS, float(self.d) ** -0.5, target="heads"),
+                    ops.ConvSegment(self.keys, self.d, "length", None, self.UNIT_EPS, target="heads", out_col=self.keys),
+                    ops.ConvSegment(self.values, self.value_width, target="heads", out_col=2 * self.keys)]
         mixed = ops.short_conv(fused, 0, self.conv, None, binding.state[:, self.scan_floats:], ctx, segments, self.channels, torch.float32, silu=True)
         gate_col = self.channels
         a_col = gate_col + self.values
         scanned = ops.gated_scan(mixed, 0, self.keys, 2 * self.keys, fused, a_col, self.rate, self.decay_bias, binding.state, ctx,
-                                 self.heads, self.groups, self.d, self.dv, b_col=a_col + self.heads)
+                                 self.heads, self.groups, self.d, self.dv, b_col=a_col + self.heads, value_width=self.value_width)
         normed = ops.head_combine(scanned, self.heads, self.dv, self.eps, self.dtype, weight=self.norm, gate=fused, gate_col=gate_col,
                                   gate_kind="silu")
         return self.o(normed)
