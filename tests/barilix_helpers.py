@@ -109,11 +109,11 @@ def rewrite(folder, changes):
     return load_plain(folder)
 
 
-def allowed_rows(config, weights, tokens, dtype, want, draws=4):
+def allowed_rows(config, weights, tokens, dtype, want, draws=8):
     """Per row of logits, how far a run in `dtype` may be from `want`, relative to the row's largest value.  In bfloat16 the
     design amplifies rounding at some tokens (a key that is small before it is made a unit vector, a result divided by its
-    own size), so the plain implementation is run `draws` times more with every product's input and result moved by as much
-    as rounding moves them: a row may be off by the tolerance, or by four times what those runs differ at that row."""
+    own size), so the plain implementation is run `draws` times more with every product's input and result (and what the cache stores) moved
+    by as much as rounding moves them: a row may be off by the tolerance, or by four times what those runs differ at that row."""
     allowed = torch.full((len(tokens),), TOLERANCE[dtype], dtype=torch.float64)
     if dtype == "float32":
         return allowed

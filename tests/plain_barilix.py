@@ -28,8 +28,14 @@ def moved(x):
     return x * (1.0 + 2.0 ** -9 * (2.0 * torch.rand(x.shape, generator=NOISE, dtype=F64) - 1.0))
 
 
+def stored(x):
+    """x as a cache or a buffer of 16 bits would give it back, while `noisy` runs."""
+    return x if NOISE is None else moved(x)
+
+
 def noisy(seed, run):
-    """run() with every product's input and result moved at random: what 16-bit storage alone does to a result."""
+    """run() with every product's input and result, and attention's queries, keys and values, moved at random: what 16-bit
+    storage alone does to a result."""
     global NOISE
     NOISE = torch.Generator().manual_seed(seed)
     try:
@@ -122,6 +128,7 @@ def conv_attention(mixer, w, prefix, h, positions, eps):
     v = projected("v", G, vdim)
     if mixer.get("rot") is not None:
         q, k = rotate_halves(q, positions, mixer["rot"]), rotate_halves(k, positions, mixer["rot"])
+    q, k, v = stored(q), stored(k), stored(v)
     mask = window_mask(T, (mixer.get("mask") or {}).get("size"))
     heads = []
     for head in range(H):
